@@ -79,6 +79,8 @@ def build_hip(jobs: int = 8) -> str:
     headers = sorted(glob.glob(os.path.join(kdir, "*.h")))
     cflags = [
         f"--offload-arch={ARCH}", "-O3", "-fPIC", "-std=c++17", "-ffp-contract=fast",
+        # no packed FP32 arithmetic (v_pk_{add,mul,fma}_f32): some forms have given wrong results
+        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
         "-Wno-unused-result", f"-I{kdir}", *_pybind_includes(),
     ]
     # hipBLASLt: link the copy PyTorch ships (it is already loaded when torch

@@ -19,8 +19,11 @@ template <class T>
 static T* P(u64 p) { return reinterpret_cast<T*>(p); }
 static hipStream_t S(u64 s) { return reinterpret_cast<hipStream_t>(s); }
 
+void bind_hybrid(py::module_& m);  // bindings_hybrid.cpp
+
 PYBIND11_MODULE(_hipk, m) {
   m.doc() = "drtc_amd CDNA4 (gfx950) HIP kernels";
+  bind_hybrid(m);
   m.def("configure", []() { return drtc::configure_kernels(); });
   m.def("rmsnorm",
         [](u64 out, u64 residual, u64 x, u64 w, int rows, int H, float eps,

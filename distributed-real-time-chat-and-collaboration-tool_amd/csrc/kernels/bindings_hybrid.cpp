@@ -1,0 +1,96 @@
+// Bindings of the kernels of models with mixed layer kinds (hybrid_launchers.h).  Launch
+// arguments cross as a dict: addresses and sizes by the field names of the argument structs.
+#include <pybind11/pybind11.h>
+
+#include "hybrid_launchers.h"
+
+namespace py = pybind11;
+using u64 = std::uintptr_t;
+
+namespace {
+
+template <class T>
+T* P(u64 p) { return reinterpret_cast<T*>(p); }
+hipStream_t S(u64 s) { return reinterpret_cast<hipStream_t>(s); }
+
+struct Fields {
+  const py::dict& d;
+  template <class T>
+  void ptr(const char* k, T*& out) const {
+    if (d.contains(k)) out = reinterpret_cast<T*>(d[k].cast<u64>());
+  }
+  template <class T>
+  void val(const char* k, T& out) const { out = d[k].cast<T>(); }
+};
+
+#define PTR(n) f.ptr(#n, a.n)
+#define VAL(n) f.val(#n, a.n)
+
+drtc::DeltaArgs delta_args(const py::dict& d) {
+  const Fields f{d};
+  drtc::DeltaArgs a{};
+  PTR(proj); VAL(ldp); VAL(off_b); PTR(conv); PTR(conv_w); PTR(ring); PTR(state); PTR(decay);
+  VAL(ld_decay); PTR(gate); VAL(ld_gate); PTR(a_exp); PTR(dt_bias); PTR(norm_w); VAL(eps);
+  VAL(H); VAL(Hk); VAL(dim); VAL(vdim); VAL(taps); VAL(C); PTR(out);
+  PTR(seg_row); PTR(seg_len); PTR(seg_pos); PTR(seg_state); PTR(positions); PTR(row_state);
+  VAL(nseg); VAL(rows);
+  return a;
+}
+
+}  // namespace
+
+void bind_hybrid(py::module_& m) {
+  m.def("dyt", [](int f32, u64 out, u64 h, u64 y, int ldy, u64 ids, u64 embed, u64 w, u64 b,
+                  float alpha, int rows, int W, u64 st) {
+    return drtc::launch_dyt(f32, P<void>(out), P<float>(h), P<void>(y), ldy, P<const int>(ids),
+                            P<void>(embed), P<float>(w), P<float>(b), alpha, rows, W, S(st));
+  });
+  m.def("act_glu_f32", [](u64 out, u64 gu, int64_t T, int I, int stride, int act, u64 st) {
+    return drtc::launch_act_glu_f32(P<float>(out), P<float>(gu), T, I, stride, act, S(st));
+  });
+  m.def("latent_prep", [](int f32, const py::dict& d, u64 st) {
+    const Fields f{d};
+    drtc::LatentPrepArgs a{};
+    PTR(proj); VAL(ldp); VAL(off_kv); VAL(H); VAL(dim); VAL(rot); VAL(rot_dims); VAL(R); VAL(LW);
+    PTR(norm_w); VAL(eps); PTR(cos_sin); PTR(positions); PTR(slots); PTR(lat); PTR(cache);
+    PTR(qa); VAL(rows);
+    return drtc::launch_latent_prep(f32, a, S(st));
+  });
+  m.def("latent_gather", [](u64 out, u64 cache, u64 slots, int rows, int row_bytes, u64 st) {
+    return drtc::launch_latent_gather(P<void>(out), P<void>(cache), P<const int64_t>(slots), rows,
+                                      row_bytes, S(st));
+  });
+  m.def("latent_prefill", [](int f32, const py::dict& d, u64 st) {
+    const Fields f{d};
+    drtc::LatentPrefillArgs a{};
+    PTR(out); VAL(ldo); PTR(q); VAL(ldq); PTR(kv); VAL(ldkv); VAL(voff); PTR(lat); VAL(LW);
+    VAL(R); VAL(H); VAL(dim); VAL(rot); VAL(vdim); PTR(q_cu); PTR(k_cu); PTR(ctx); PTR(tile_seq);
+    PTR(tile_q0); VAL(ntiles); VAL(qtile); VAL(nseq); VAL(nq); VAL(window); VAL(scale); PTR(sink);
+    return drtc::launch_latent_prefill(f32, a, S(st));
+  });
+  m.def("latent_decode", [](int f32, const py::dict& d, u64 st) {
+    const Fields f{d};
+    drtc::LatentDecodeArgs a{};
+    PTR(out); PTR(part_o); PTR(part_ml); PTR(qa); PTR(cache); PTR(block_tables); VAL(bt_stride);
+    PTR(context_lens); VAL(B); VAL(H); VAL(R); VAL(LW); VAL(window); VAL(tiles_per_split);
+    VAL(nsplits); VAL(scale); PTR(sink);
+    return drtc::launch_latent_decode(f32, a, S(st));
+  });
+  m.def("head_gemm", [](int f32, u64 y, u64 x, u64 w, int B, int H, int N, int K, int64_t yb,
+                        int64_t yh, int64_t xb, int64_t xh, u64 st) {
+    return drtc::launch_head_gemm(f32, P<void>(y), P<void>(x), P<void>(w), B, H, N, K, yb, yh, xb,
+                                  xh, S(st));
+  });
+  m.def("short_conv", [](int f32, u64 out, u64 proj, int ldp, u64 w, u64 ring, u64 positions,
+                         u64 row_off, u64 row_state, int rows, int C, int taps, u64 st) {
+    return drtc::launch_short_conv(f32, P<void>(out), P<void>(proj), ldp, P<float>(w),
+                                   P<void>(ring), P<const int>(positions), P<const int>(row_off),
+                                   P<const int>(row_state), rows, C, taps, S(st));
+  });
+  m.def("delta_scan", [](int f32, const py::dict& d, int cpl, u64 st) {
+    return drtc::launch_delta_scan(f32, delta_args(d), cpl, S(st));
+  });
+  m.def("delta_decode", [](int f32, const py::dict& d, u64 st) {
+    return drtc::launch_delta_decode(f32, delta_args(d), S(st));
+  });
+}

@@ -1,4 +1,5 @@
 // One-time kernel attribute setup (dynamic LDS > 64 KiB for head_dim 256).
+#include "hybrid_launchers.h"
 #include "launchers.h"
 
 namespace drtc {
@@ -10,6 +11,8 @@ int configure_kernels() {
   e = configure_moe();
   if (e) return e;
   e = configure_gemm_w4();
+  if (e) return e;
+  e = configure_latent();
   if (e) return e;
   return configure_gemm_xd();
 }

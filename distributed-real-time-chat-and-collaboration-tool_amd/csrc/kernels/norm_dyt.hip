@@ -1,0 +1,127 @@
+// Dynamic Tanh on a 32-bit residual stream (gfx950).
+//
+//   h += y                        (the preceding sublayer's output, optional)
+//   h  = embed[ids]               (instead, at the first layer)
+//   out = tanh(alpha h) w + b
+//
+// Elementwise - no row statistics - so the grid runs over flat 8-element vectors of the
+// whole batch, and the residual add or the embedding lookup costs no pass of its own.
+#include "hybrid_launchers.h"
+#include "typed.h"
+
+namespace drtc {
+
+// 1 - 2 / (1 + exp(2 x)): absolute error of a few 2^-24, saturates at +-1
+DRTC_DEVICE float tanh_exp(float x) {
+  const float e = fast_exp2(x * (2.f * kLog2e));
+  return 1.f - 2.f * __frcp_rn(1.f + e);
+}
+template <class T>
+DRTC_DEVICE float tanh_as(float x);
+template <>
+DRTC_DEVICE float tanh_as<bf16_t>(float x) { return tanh_exp(x); }
+template <>
+DRTC_DEVICE float tanh_as<float>(float x) { return tanhf(x); }
+
+template <class T>
+__global__ __launch_bounds__(256) void dyt_vec_kernel(
+    T* __restrict__ out, float* __restrict__ h, const T* __restrict__ y, int ldy,
+    const int* __restrict__ ids, const T* __restrict__ embed, const float* __restrict__ w,
+    const float* __restrict__ b, float alpha, int64_t nvec, int vpr) {
+  const int64_t v = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (v >= nvec) return;
+  const int64_t row = v / vpr;
+  const int c = (int)(v - row * vpr) * 8;
+  const int64_t at = row * vpr * 8 + c;
+  float x[8], ww[8], bb[8];
+  load8(ww, w + c);
+  load8(bb, b + c);
+  if (ids) {
+    load8(x, embed + (int64_t)ids[row] * vpr * 8 + c);
+    store8(h + at, x);
+  } else {
+    load8(x, h + at);
+    if (y) {
+      float d[8];
+      load8(d, y + row * ldy + c);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] += d[j];
+      store8(h + at, x);
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < 8; ++j) x[j] = tanh_as<T>(alpha * x[j]) * ww[j] + bb[j];
+  store8(out + at, x);
+}
+
+template <class T>
+__global__ __launch_bounds__(256) void dyt_any_kernel(
+    T* __restrict__ out, float* __restrict__ h, const T* __restrict__ y, int ldy,
+    const int* __restrict__ ids, const T* __restrict__ embed, const float* __restrict__ w,
+    const float* __restrict__ b, float alpha, int64_t n, int W) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= n) return;
+  const int64_t row = i / W;
+  const int c = (int)(i - row * W);
+  float x;
+  if (ids) {
+    x = to_f32(embed[(int64_t)ids[row] * W + c]);
+    h[i] = x;
+  } else {
+    x = h[i];
+    if (y) {
+      x += to_f32(y[row * ldy + c]);
+      h[i] = x;
+    }
+  }
+  out[i] = from_f32<T>(tanh_as<T>(alpha * x) * w[c] + b[c]);
+}
+
+template <class T>
+static void dyt_t(void* out, float* h, const void* y, int ldy, const int* ids, const void* embed,
+                  const float* w, const float* b, float alpha, int rows, int W, hipStream_t st) {
+  if (W % 8 == 0 && ldy % 8 == 0) {
+    const int64_t n = (int64_t)rows * (W / 8);
+    dyt_vec_kernel<T><<<dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st>>>(
+        (T*)out, h, (const T*)y, ldy, ids, (const T*)embed, w, b, alpha, n, W / 8);
+  } else {
+    const int64_t n = (int64_t)rows * W;
+    dyt_any_kernel<T><<<dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st>>>(
+        (T*)out, h, (const T*)y, ldy, ids, (const T*)embed, w, b, alpha, n, W);
+  }
+}
+
+int launch_dyt(int f32, void* out, float* h, const void* y, int ldy, const int* ids,
+               const void* embed, const float* w, const float* b, float alpha, int rows, int W,
+               hipStream_t st) {
+  if (rows == 0) return 0;
+  if (f32) dyt_t<float>(out, h, y, ldy, ids, embed, w, b, alpha, rows, W, st);
+  else dyt_t<bf16_t>(out, h, y, ldy, ids, embed, w, b, alpha, rows, W, st);
+  return (int)hipGetLastError();
+}
+
+// Gated activation of the fp32 models; tanhf / expf instead of the bf16 kernels' fast forms.
+__global__ __launch_bounds__(256) void act_glu_f32_kernel(float* __restrict__ out,
+                                                          const float* __restrict__ gu, int64_t n,
+                                                          int I, int stride, int act) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= n) return;
+  const int64_t row = i / I;
+  const int c = (int)(i - row * I);
+  const float g = gu[row * stride + c], u = gu[row * stride + I + c];
+  const float a = act == 0 ? g / (1.f + expf(-g))
+                           : 0.5f * g * (1.f + tanhf(0.7978845608028654f *
+                                                     (g + 0.044715f * g * g * g)));
+  out[i] = a * u;
+}
+
+int launch_act_glu_f32(float* out, const float* gu, int64_t T, int I, int gu_stride, int act,
+                       hipStream_t st) {
+  const int64_t n = T * I;
+  if (n == 0) return 0;
+  act_glu_f32_kernel<<<dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st>>>(out, gu, n, I,
+                                                                           gu_stride, act);
+  return (int)hipGetLastError();
+}
+
+}  // namespace drtc

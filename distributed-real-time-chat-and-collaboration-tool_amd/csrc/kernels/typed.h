@@ -1,0 +1,78 @@
+// Activation element types of the kernels that run in bf16 and in fp32 (T = bf16_t or float):
+// conversions, 8-element rows and sub-wave reductions.
+#pragma once
+#include "common.h"
+
+namespace drtc {
+
+DRTC_DEVICE float to_f32(bf16_t x) { return (float)x; }
+DRTC_DEVICE float to_f32(float x) { return x; }
+template <class T>
+DRTC_DEVICE T from_f32(float x);
+template <>
+DRTC_DEVICE bf16_t from_f32<bf16_t>(float x) { return (bf16_t)x; }
+template <>
+DRTC_DEVICE float from_f32<float>(float x) { return x; }
+
+// 8 consecutive elements as floats (16-byte aligned for bf16, 32-byte chunks for float)
+DRTC_DEVICE void load8(float (&v)[8], const bf16_t* p) {
+  const bf16x8 x = load_bf16x8(p);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = bf2f(x[j]);
+}
+DRTC_DEVICE void load8(float (&v)[8], const float* p) {
+  const f32x4 a = *reinterpret_cast<const f32x4*>(p);
+  const f32x4 b = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) { v[j] = a[j]; v[4 + j] = b[j]; }
+}
+DRTC_DEVICE void store8(bf16_t* p, const float (&v)[8]) {
+  bf16x8 x;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) x[j] = f2bf(v[j]);
+  store_bf16x8(p, x);
+}
+DRTC_DEVICE void store8(float* p, const float (&v)[8]) {
+  f32x4 a, b;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) { a[j] = v[j]; b[j] = v[4 + j]; }
+  *reinterpret_cast<f32x4*>(p) = a;
+  *reinterpret_cast<f32x4*>(p + 4) = b;
+}
+
+// Sum over the 4 lanes of a quad (DPP quad_perm, no LDS traffic).
+DRTC_DEVICE float quad_sum(float v) {
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xF, 0xF, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xF, 0xF, true));
+  return v;
+}
+// Sum over aligned groups of 16 lanes.
+DRTC_DEVICE float sum16(float v) {
+#pragma unroll
+  for (int o = 8; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
+  return v;
+}
+
+// Block-wide sum / max for blocks of up to 16 waves; `red` holds 16 floats.
+DRTC_DEVICE float block_sum(float v, float* red) {
+  const int nw = (blockDim.x + 63) >> 6;
+  v = wave_sum(v);
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float s = 0.f;
+  for (int i = 0; i < nw; ++i) s += red[i];
+  return s;
+}
+DRTC_DEVICE float block_max(float v, float* red) {
+  const int nw = (blockDim.x + 63) >> 6;
+  v = wave_max(v);
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float s = kNegBig;
+  for (int i = 0; i < nw; ++i) s = fmaxf(s, red[i]);
+  return s;
+}
+
+}  // namespace drtc

@@ -1,0 +1,61 @@
+"""Checkpoint files: a safetensors reader (memory-mapped, no dependency)."""
+from __future__ import annotations
+
+import json
+import mmap
+import os
+
+import torch
+
+_DTYPES = {"BF16": torch.bfloat16, "F16": torch.float16, "F32": torch.float32,
+           "I32": torch.int32, "I64": torch.int64}
+
+
+def read_safetensors(path: str) -> dict[str, torch.Tensor]:
+    """name -> CPU tensor.  The file: 8-byte little-endian header length, a JSON header (name ->
+    dtype, shape, [begin, end) into the data), the data."""
+    out = {}
+    with open(path, "rb") as f:
+        size = os.fstat(f.fileno()).st_size
+        buf = mmap.mmap(f.fileno(), 0, access=mmap.ACCESS_COPY)
+    n = int.from_bytes(buf[:8], "little")
+    if 8 + n > size:
+        raise ValueError(f"{path}: truncated header")
+    for name, e in json.loads(buf[8:8 + n]).items():
+        if name == "__metadata__":
+            continue
+        dt = _DTYPES.get(e["dtype"])
+        if dt is None:
+            raise ValueError(f"{path}: {name} has unsupported dtype {e['dtype']}")
+        b, end = e["data_offsets"]
+        count = 1
+        for d in e["shape"]:
+            count *= d
+        if end - b != count * dt.itemsize or not 0 <= b <= end <= size - 8 - n:
+            raise ValueError(f"{path}: {name} does not fit its data range")
+        t = torch.frombuffer(bytearray(buf[8 + n + b:8 + n + end]), dtype=dt) if count else \
+            torch.empty(0, dtype=dt)
+        out[name] = t.reshape(e["shape"])
+    return out
+
+
+class Tensors:
+    """The tensors of a checkpoint, each taken once with its shape checked; ``finish`` refuses
+    leftovers, so a tensor the model does not know never passes unnoticed."""
+
+    def __init__(self, tensors: dict[str, torch.Tensor]):
+        self._t = dict(tensors)
+
+    def shape(self, name: str) -> tuple:
+        if name not in self._t:
+            raise KeyError(f"checkpoint has no tensor {name!r}")
+        return tuple(self._t[name].shape)
+
+    def take(self, name: str, *shape: int) -> torch.Tensor:
+        if self.shape(name) != shape:
+            raise ValueError(f"tensor {name!r} is {list(self._t[name].shape)}, expected {list(shape)}")
+        return self._t.pop(name)
+
+    def finish(self) -> None:
+        if self._t:
+            raise ValueError(f"checkpoint tensors without a place in the model: {sorted(self._t)[:8]}")

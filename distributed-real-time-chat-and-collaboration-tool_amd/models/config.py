@@ -6,10 +6,16 @@ The four families BASELINE.json names for the LLM service:
   * Gemma-2B    (smart reply, TP=1; MQA, head_dim 256, GELU-tanh, (1+w) norm)
   * Mixtral-8x7B (context suggestions; top-2 of 8 experts, EP)
 plus tiny variants of each for CPU tests.
+
+:class:`HybridConfig` describes models whose layers differ (mixer kind, sizes, window, with or
+without a feed-forward): the Ralesun design, latent attention and channel-wise gated delta-rule
+mixers.  Their checkpoints carry a config.json, parsed by :func:`config_from_dict`.
 """
 from __future__ import annotations
 
 import dataclasses
+import json
+import os
 from dataclasses import dataclass, field
 
 
@@ -111,12 +117,184 @@ TINY_MIXTRAL = ModelConfig(
     num_layers=2, num_heads=4, num_kv_heads=2, head_dim=64, rope_theta=1e6,
     max_position=1024, num_experts=4, experts_per_token=2, bos_token_id=1, eos_token_id=2)
 
+
+# ------------------------------------------------------------------ layers of mixed kinds
+@dataclass(frozen=True)
+class LatentAttention:
+    """Attention over per-token latents: heads of ``dim`` unrotated + ``rot_dim`` rotated query
+    dims, values of ``vdim``, latents of ``kv_rank``; ``window`` tokens visible (None: all);
+    the first ``rot_dims`` rotated dims turned in interleaved pairs; a softmax sink per head."""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    window: int | None
+    rot_base: float
+    rot_dims: int
+    sink: bool = True
+
+    def __post_init__(self):
+        if self.rot_dims % 2 or self.rot_dims > self.rot_dim:
+            raise ValueError(f"rotated dims {self.rot_dims} of a {self.rot_dim}-wide part")
+        if self.window is not None and self.window < 1:
+            raise ValueError("a window holds at least the token itself")
+        if self.kv_rank > 1024 or self.vdim > 1024:
+            raise ValueError("latent attention kernels take latents and values up to 1024")
+
+
+@dataclass(frozen=True)
+class ChannelDelta:
+    """Gated delta rule with one decay per head and key channel; ``conv`` taps of the short
+    convolutions; ``decay_rank`` / ``gate_rank``: inner sizes of the decay and gate projections
+    (a checkpoint's tensors set them)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    decay_rank: int | None = None
+    gate_rank: int | None = None
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError("heads must divide by kv_heads")
+        if self.dim > 256 or self.vdim > 512:
+            raise ValueError("delta-rule kernels take dim <= 256 and vdim <= 512")
+
+    @property
+    def channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+
+@dataclass(frozen=True)
+class Layer:
+    mixer: LatentAttention | ChannelDelta
+    ff: int | None = None  # gated feed-forward size; None: the layer is its mixer alone
+
+
+@dataclass(frozen=True)
+class HybridConfig:
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: tuple[Layer, ...]
+    norm_eps: float = 1e-6
+    act: str = "gelu_tanh"
+    max_position: int = 8192
+    bos_token_id: int = 1
+    eos_token_id: int = 2
+    init_std: float = 0.02
+    prefill_chunk: int = 16384
+
+    is_moe = False
+    tie_embeddings = False
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def windows(self) -> tuple:
+        """Distinct windows of the attention layers (None: unlimited)."""
+        return tuple(dict.fromkeys(l.mixer.window for l in self.layers
+                                   if isinstance(l.mixer, LatentAttention)))
+
+    def num_params(self) -> int:
+        W, n = self.hidden_size, 2 * self.vocab_size * self.hidden_size + 2 * self.hidden_size
+        for l in self.layers:
+            m = l.mixer
+            if isinstance(m, LatentAttention):
+                n += W * (m.heads * (m.dim + m.rot_dim + m.vdim) + m.kv_rank + m.rot_dim)
+                n += m.kv_rank * (m.heads * (m.dim + m.vdim) + 1) + (m.heads if m.sink else 0)
+            else:
+                ra, rg = m.decay_rank or m.dim, m.gate_rank or m.vdim
+                n += W * (m.channels + m.heads * (1 + m.vdim) + ra + rg)
+                n += m.channels * m.conv + m.heads * (m.dim * (ra + 1) + m.vdim * rg + 1) + m.vdim
+            n += 2 * W + 1
+            if l.ff:
+                n += 3 * W * l.ff + 2 * W + 1
+        return n
+
+    def replace(self, **kw) -> "HybridConfig":
+        return dataclasses.replace(self, **kw)
+
+
+def _ralesun(d: dict, name: str) -> HybridConfig:
+    layers = []
+    for e in d["layers"]:
+        m = e["mixer"]
+        if e["type"] == "latent_attention":
+            mixer = LatentAttention(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"],
+                                    float(m["scale"]), (m.get("mask") or {}).get("size"),
+                                    float(m["rot"]["base"]), m["rot"]["dims"])
+        elif e["type"] == "channel_delta":
+            mixer = ChannelDelta(m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["conv"])
+        else:
+            raise ValueError(f"unknown layer type {e['type']!r}")
+        mlp = e["mlp"]
+        if mlp is not None and mlp["kind"] != "dense":
+            raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+        layers.append(Layer(mixer, mlp["ff"] if mlp else None))
+    # the format names no special tokens: generation ends by length or by stop tokens
+    return HybridConfig(name, d["vocab"], d["width"], tuple(layers), float(d["norm"]["eps"]),
+                        max_position=d.get("max_position", 32768), bos_token_id=0, eos_token_id=-1)
+
+
+# checkpoint configuration ("architecture" key) -> parser
+ARCHITECTURES = {"Ralesun": _ralesun}
+
+
+def config_from_dict(d: dict, name: str = "") -> HybridConfig:
+    arch = d.get("architecture")
+    if arch not in ARCHITECTURES:
+        raise KeyError(f"unknown architecture {arch!r}; known: {sorted(ARCHITECTURES)}")
+    return ARCHITECTURES[arch](d, name or arch.lower())
+
+
+def load_config(path: str) -> HybridConfig:
+    """Configuration of a checkpoint folder."""
+    with open(os.path.join(path, "config.json")) as f:
+        return config_from_dict(json.load(f), os.path.basename(os.path.abspath(path)))
+
+
+def _stack(blocks: int, latent: LatentAttention, delta: ChannelDelta, ff: int) -> tuple:
+    """Latent-attention layers with a feed-forward, each followed by a bare delta-rule layer."""
+    return (Layer(latent, ff), Layer(delta)) * blocks
+
+
+# Random-init presets of the design at the layer sizes of Llama-3-8B and of half its width.
+RALESUN_8B = HybridConfig(
+    name="ralesun-8b", vocab_size=128256, hidden_size=4096, layers=_stack(
+        32, LatentAttention(32, 128, 64, 128, 512, 192 ** -0.5, 1024, 500000.0, 64),
+        ChannelDelta(32, 32, 128, 128, 4, 128, 128), 14336),
+    bos_token_id=128000, eos_token_id=128001)
+
+RALESUN_2B = HybridConfig(
+    name="ralesun-2b", vocab_size=128256, hidden_size=2048, layers=_stack(
+        24, LatentAttention(16, 128, 64, 128, 512, 192 ** -0.5, 1024, 500000.0, 64),
+        ChannelDelta(16, 16, 128, 128, 4, 128, 128), 7168),
+    bos_token_id=128000, eos_token_id=128001)
+
+TINY_RALESUN = HybridConfig(
+    name="tiny-ralesun", vocab_size=512, hidden_size=192, layers=(
+        Layer(ChannelDelta(4, 2, 16, 24, 3, 16, 24), 320),
+        Layer(LatentAttention(3, 24, 8, 40, 64, 0.2, 37, 10000.0, 8)),
+        Layer(ChannelDelta(2, 2, 40, 32, 4, 24, 16)),
+        Layer(LatentAttention(5, 16, 16, 32, 48, 0.15, 70, 50000.0, 16), 256)),
+    max_position=1024, init_std=0.06)
+
 REGISTRY = {c.name: c for c in (LLAMA3_8B, LLAMA3_70B, GEMMA_2B, MIXTRAL_8X7B,
-                                TINY_LLAMA, TINY_GEMMA, TINY_MIXTRAL)}
+                                TINY_LLAMA, TINY_GEMMA, TINY_MIXTRAL, RALESUN_8B, RALESUN_2B,
+                                TINY_RALESUN)}
 
 
-def get_config(name: str) -> ModelConfig:
+def get_config(name: str) -> ModelConfig | HybridConfig:
+    """Configuration of a registered model, or of a checkpoint folder."""
     try:
         return REGISTRY[name]
     except KeyError:
+        if os.path.isfile(os.path.join(name, "config.json")):
+            return load_config(name)
         raise KeyError(f"unknown model {name!r}; known: {sorted(REGISTRY)}") from None

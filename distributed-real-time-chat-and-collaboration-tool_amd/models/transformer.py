@@ -79,6 +79,7 @@ class PrefillMeta:
     decode: "DecodeMeta | None" = None
     n_prefill: int = 0
     max_len: int | None = None   # longest sequence (prefill attention launch form)
+    extra: object = None         # the model's own step metadata (HybridLM.step_meta)
 
 
 @dataclass
@@ -89,6 +90,7 @@ class DecodeMeta:
     context_lens: torch.Tensor   # int32 [B]
     blocks_per_part: int
     workspace: object            # ops.DecodeWorkspace
+    state: torch.Tensor | None = None  # int32 [B] recurrent state slots (-1: none)
 
 
 class ShardInfo:
@@ -249,6 +251,29 @@ class TransformerLM:
         if not self.cfg.tie_embeddings:
             n += self.lm_head.numel()
         return n * self.embed.element_size()
+
+    # ------------------------------------------------------------ engine hooks
+    portions = False  # prompts run whole: prefill attention reads the step's own rows
+
+    def new_cache(self, num_blocks: int, max_batch: int):
+        from ..engine.kv_cache import PagedKVCache
+
+        return PagedKVCache(self.cfg, self.sh.hkv, num_blocks, self.device, self.dtype)
+
+    def auto_num_blocks(self, max_batch: int, **kw) -> int:
+        from ..engine.kv_cache import PagedKVCache
+
+        return PagedKVCache.auto_num_blocks(self.cfg, self.sh.hkv, self.device, **kw)
+
+    def decode_buffer(self, max_batch: int) -> torch.Tensor:
+        return torch.zeros((max_batch, self.sh.hq, self.cfg.head_dim), dtype=self.dtype,
+                           device=self.device)
+
+    def decode_meta(self, Bb: int, max_blocks: int, **tensors) -> DecodeMeta:
+        sh, D = self.sh, self.cfg.head_dim
+        bpp, max_parts = ops.decode_partitioning(Bb, sh.hkv, max_blocks, D=D)
+        ws = ops.DecodeWorkspace(Bb, sh.hq, D, max_parts, self.device)
+        return DecodeMeta(blocks_per_part=bpp, workspace=ws, **tensors)
 
     # ------------------------------------------------------------ forward
     def _embed(self, ids: torch.Tensor) -> torch.Tensor:

@@ -15,10 +15,14 @@ from .activation import act_glu, act_glu_ref
 from .attention import (KV_BLOCK, DecodeWorkspace, decode_partitioning, paged_decode_attention,
                         paged_decode_attention_rope, set_prefill_persist,
                         paged_decode_ref, prefill_attention, prefill_attention_ref, prefill_tiles)
-from .gemm import (fused_glu_ok, glu_linear, linear, linear_residual, mfma_gemm, norm_glu,
+from .delta import DeltaWeights, Portions, delta_decode, delta_scan, short_conv
+from .gemm import (fused_glu_ok, gated, glu_linear, linear, linear_residual, mfma_gemm, norm_glu,
                    norm_linear, residual_fusable, w4_glu_ok)
+from .latent import (LatentDecodeWorkspace, PortionKeys, build_interleaved_rope, head_linear,
+                     latent_decode_attention, latent_gather, latent_prefill_attention,
+                     latent_prep, latent_qtile, latent_width, portion_tiles, window_reach)
 from .moe import fused_moe, fused_moe_ref, router_logits
-from .norm import PendingNorm, rmsnorm, rmsnorm_ref
+from .norm import PendingNorm, dyt, dyt_ref, rmsnorm, rmsnorm_ref
 from .rope import build_rope_cache, kv_write_v, kv_write_v_ref, rope_kv_, rope_kv_ref
 from .sampling import sample, sample_ref
 
@@ -30,5 +34,9 @@ __all__ = [
     "decode_partitioning", "paged_decode_attention", "paged_decode_attention_rope",
     "paged_decode_ref", "prefill_attention", "prefill_attention_ref", "prefill_tiles",
     "set_prefill_persist", "rmsnorm", "rmsnorm_ref", "build_rope_cache", "rope_kv_",
-    "rope_kv_ref", "kv_write_v", "kv_write_v_ref", "sample", "sample_ref",
+    "rope_kv_ref", "kv_write_v", "kv_write_v_ref", "sample", "sample_ref", "dyt", "dyt_ref",
+    "gated", "DeltaWeights", "Portions", "delta_decode", "delta_scan", "short_conv",
+    "LatentDecodeWorkspace", "PortionKeys", "build_interleaved_rope", "head_linear",
+    "latent_decode_attention", "latent_gather", "latent_prefill_attention", "latent_prep",
+    "latent_qtile", "latent_width", "portion_tiles", "window_reach",
 ]

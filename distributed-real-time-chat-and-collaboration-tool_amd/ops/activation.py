@@ -32,13 +32,18 @@ def act_glu(gu: torch.Tensor, act: str = "silu", out: torch.Tensor | None = None
             out.copy_(r)
             return out
         return r
-    assert gu.dim() == 2 and gu.dtype == torch.bfloat16 and gu.stride(1) == 1
+    assert gu.dim() == 2 and gu.stride(1) == 1
+    assert gu.dtype in (torch.bfloat16, torch.float32)
     T, two_i = gu.shape
     inter = two_i // 2
-    assert inter % 8 == 0
+    assert gu.dtype == torch.float32 or inter % 8 == 0
     if out is None:
         out = torch.empty((T, inter), dtype=gu.dtype, device=gu.device)
     assert out.is_contiguous() and out.shape == (T, inter)
+    if gu.dtype == torch.float32:
+        check(hipk().act_glu_f32(out.data_ptr(), gu.data_ptr(), T, inter, gu.stride(0), ACTS[act],
+                                 stream_ptr(gu)), "act_glu_f32")
+        return out
     check(hipk().act_glu(out.data_ptr(), gu.data_ptr(), T, inter, gu.stride(0),
                          ACTS[act], stream_ptr(gu)), "act_glu")
     return out

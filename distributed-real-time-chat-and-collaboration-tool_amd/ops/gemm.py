@@ -807,6 +807,21 @@ def norm_glu(p, w: torch.Tensor, act: str = "silu") -> torch.Tensor:
     return act_glu(norm_linear(p, w), act)
 
 
+def gated(x: torch.Tensor, w: torch.Tensor, act: str = "silu") -> torch.Tensor:
+    """h = act(x @ gate^T) * (x @ up^T) for normed rows x and the fused [gate; up] weight, by
+    the same choice of kernels as ``norm_glu``."""
+    from .activation import act_glu
+
+    if fused_glu_ok(x, w, act):
+        M, K = x.shape
+        form = glu_form(M, w.shape[0], K, x.stride(0))
+        if form:
+            return xd_gemm(x, w, act, form=form)
+        return mfma_gemm(x, w, act, variant=_w4v(K),
+                         group_m=w4_group_m(M, w.shape[0] // 2, K, glu=True))
+    return act_glu(linear(x, w), act)
+
+
 # ------------------------------------------------------------------ XCD-partitioned decode GEMM
 XD_EPI = {"store": 0, "residual": 1, "silu": 2, "gelu_tanh": 3}
 # tile shapes built in gemm_xd.hip, (mt, nf) -> LDS ring depth (128 mt x 32 nf tiles); a form

@@ -1,4 +1,5 @@
-"""RMSNorm (+ fused residual add).  HIP kernel: csrc/kernels/norm_act_rope.hip."""
+"""Norms.  RMSNorm (+ fused residual add): csrc/kernels/norm_act_rope.hip; Dynamic Tanh on a
+32-bit residual stream (+ fused residual add or embedding lookup): csrc/kernels/norm_dyt.hip."""
 from __future__ import annotations
 
 import torch
@@ -45,6 +46,35 @@ def rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, gemma: bool = False,
     check(hipk().rmsnorm(out.data_ptr(), ptr(residual), x.data_ptr(), w.data_ptr(),
                          rows, H, float(eps), x.stride(0), out.stride(0), res_stride,
                          bool(gemma), stream_ptr(x)), "rmsnorm")
+    return out
+
+
+def dyt_ref(h, w, b, alpha, y=None, ids=None, embed=None, dtype=torch.bfloat16):
+    if ids is not None:
+        h.copy_(embed[ids.long()])
+    elif y is not None:
+        h += y.float()
+    return (torch.tanh(alpha * h) * w + b).to(dtype)
+
+
+def dyt(h: torch.Tensor, w: torch.Tensor, b: torch.Tensor, alpha: float,
+        y: torch.Tensor | None = None, ids: torch.Tensor | None = None,
+        embed: torch.Tensor | None = None, dtype=torch.bfloat16) -> torch.Tensor:
+    """tanh(alpha h) w + b of the 32-bit residual stream h [rows, W], after h += y (the
+    preceding sublayer's output) or h = embed[ids]; h is updated in place.  w, b: float32."""
+    if not on_gpu(h):
+        return dyt_ref(h, w, b, alpha, y, ids, embed, dtype)
+    rows, W = h.shape
+    assert h.dtype == w.dtype == b.dtype == torch.float32 and h.is_contiguous()
+    assert w.numel() == b.numel() == W and w.is_contiguous() and b.is_contiguous()
+    assert y is None or (y.shape == (rows, W) and y.stride(1) == 1 and y.dtype == dtype)
+    assert ids is None or (ids.dtype == torch.int32 and ids.numel() == rows and ids.is_contiguous()
+                           and embed.is_contiguous() and embed.dtype == dtype
+                           and embed.shape[1] == W)
+    out = torch.empty((rows, W), dtype=dtype, device=h.device)
+    check(hipk().dyt(int(dtype == torch.float32), out.data_ptr(), h.data_ptr(), ptr(y),
+                     y.stride(0) if y is not None else 0, ptr(ids), ptr(embed), w.data_ptr(),
+                     b.data_ptr(), float(alpha), rows, W, stream_ptr(h)), "dyt")
     return out
 
 
