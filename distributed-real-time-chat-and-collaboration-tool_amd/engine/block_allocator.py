@@ -65,6 +65,11 @@ def _native_cls():
         return None
 
 
+def native_missing() -> bool:
+    """Whether the native runtime module has not been built in this checkout."""
+    return _native_cls() is None
+
+
 def BlockAllocator(num_blocks: int, reserved: int = 0):
     cls = _native_cls()
     if cls is None:

@@ -45,16 +45,17 @@ class DecodeRunner:
         self.device = dev
         self.use_graphs = bool(use_graphs and dev.type == "cuda")
         self.buckets = sorted({b for b in buckets if b < max_batch} | {max_batch})
-        cfg, sh = model.cfg, model.sh
         B, MB = max_batch, max_blocks
         # ---- device buffers (persistent: graphs capture these addresses)
-        n_i32 = 3 * B + B * MB + B
+        n_i32 = 3 * B + B * MB + B + B
         self.i32 = torch.zeros(n_i32, dtype=torch.int32, device=dev)
         self.ids = self.i32[0:B]
         self.positions = self.i32[B:2 * B]
         self.ctx = self.i32[2 * B:3 * B]
         self.topk = self.i32[3 * B:4 * B]
         self.bt = self.i32[4 * B:4 * B + B * MB].view(B, MB)
+        self.state = self.i32[4 * B + B * MB:]  # recurrent state slot per sequence (-1: none)
+        self.has_state = getattr(kv_cache, "states", None) is not None
         # int64 staging: KV slot per sequence | source row of the input token
         # in the previous step's sampled tokens (-1: take ``ids`` from the host)
         self.i64 = torch.full((2 * B,), -1, dtype=torch.int64, device=dev)
@@ -65,7 +66,10 @@ class DecodeRunner:
         self.topp = self.f32[B:2 * B]
         self.step_ctr = torch.zeros(1, dtype=torch.int64, device=dev)
         self.out = torch.zeros(B, dtype=torch.int32, device=dev)
-        self.attn_out = torch.zeros((B, sh.hq, cfg.head_dim), dtype=model.dtype, device=dev)
+        self.attn_out = model.decode_buffer(B)
+        # the step's logits per bucket, for callers that read them instead of the samples
+        self.keep_logits = False
+        self.logits: dict[int, torch.Tensor] = {}
         # ---- pinned host staging, double-buffered: step t+1 is staged while
         # step t's copies may still be pending (pipelined decode)
         pin = dev.type == "cuda"
@@ -110,13 +114,10 @@ class DecodeRunner:
     def _meta(self, Bb: int) -> DecodeMeta:
         m = self._metas.get(Bb)
         if m is None:
-            sh = self.model.sh
-            bpp, max_parts = ops.decode_partitioning(Bb, sh.hkv, self.max_blocks,
-                                                     D=self.model.cfg.head_dim)
-            ws = ops.DecodeWorkspace(Bb, sh.hq, self.model.cfg.head_dim, max_parts, self.device)
-            m = DecodeMeta(positions=self.positions[:Bb], slots=self.slots[:Bb],
-                           block_tables=self.bt[:Bb], context_lens=self.ctx[:Bb],
-                           blocks_per_part=bpp, workspace=ws)
+            m = self.model.decode_meta(
+                Bb, self.max_blocks, positions=self.positions[:Bb], slots=self.slots[:Bb],
+                block_tables=self.bt[:Bb], context_lens=self.ctx[:Bb],
+                state=self.state[:Bb] if self.has_state else None)
             self._metas[Bb] = m
         return m
 
@@ -129,8 +130,11 @@ class DecodeRunner:
                           self.ids[:Bb])
         if self.ep:
             self.ids_used[:Bb].copy_(ids)
-        logits = self.model.forward_decode(ids, meta, self.kv, self.attn_out[:Bb])
-        ops.sample(logits, self.temp[:Bb], self.topk[:Bb], self.topp[:Bb], seed=self.seed,
+        logits = self.model.forward_decode(ids, meta, self.kv,
+                                           None if self.attn_out is None else self.attn_out[:Bb])
+        if self.keep_logits:
+            self.logits[Bb] = logits
+        ops.sample(logits.to(torch.bfloat16), self.temp[:Bb], self.topk[:Bb], self.topp[:Bb], seed=self.seed,
                    step=self.step_ctr, out=self.out[:Bb])
         self.step_ctr.add_(1)
         if not (self.device.type == "cuda" and torch.cuda.is_current_stream_capturing()):
@@ -139,6 +143,11 @@ class DecodeRunner:
     def capture(self, Bb: int) -> None:
         if not self.use_graphs or Bb in self._graphs:
             return
+        # the warm-up below runs the step once more than asked: without sequences (no context,
+        # no cache write, no state slot), because a recurrent state must not advance twice
+        self.i32.zero_()
+        self.state.fill_(-1)
+        self.i64.fill_(-1)
         # warm up on a side stream (lazy hipBLASLt / allocator init), then capture
         s = torch.cuda.Stream(self.device)
         s.wait_stream(torch.cuda.current_stream(self.device))
@@ -154,6 +163,12 @@ class DecodeRunner:
         torch.cuda.synchronize(self.device)
         self._graphs[Bb] = g
 
+    def read_logits(self, n: int) -> None:
+        """Keep the logits of every later step of ``n`` sequences in ``logits[bucket(n)]``."""
+        self.keep_logits = True
+        if self.bucket(n) not in self.logits:
+            self._graphs.pop(self.bucket(n), None)  # captured without
+
     def capture_all(self, up_to: int | None = None) -> None:
         for Bb in sorted(self.buckets, reverse=True):
             if up_to is None or Bb <= self.bucket(min(up_to, self.max_batch)):
@@ -162,7 +177,7 @@ class DecodeRunner:
     # ------------------------------------------------------------------
     def launch(self, n: int, ids: np.ndarray | None, positions: np.ndarray, ctx: np.ndarray,
                slots: np.ndarray, block_rows: np.ndarray, temp: np.ndarray, topk: np.ndarray,
-               topp: np.ndarray) -> tuple[int, int]:
+               topp: np.ndarray, state: np.ndarray | None = None) -> tuple[int, int]:
         """Enqueue one decode step for ``n`` sequences (arrays of length n,
         block_rows [n, max_blocks]) without waiting for it.  ``ids=None``
         takes every input token from the previous step's samples on the device
@@ -170,6 +185,8 @@ class DecodeRunner:
         :meth:`wait`."""
         Bb = self.bucket(n)
         B, MB = self.max_batch, self.max_blocks
+        if self.use_graphs:
+            self.capture(Bb)  # before the staging: it clears the device copies
         k = self._k
         self._k ^= 1
         hi = self.h_i32[k].numpy()
@@ -185,6 +202,9 @@ class DecodeRunner:
         btv = hi[4 * B:4 * B + B * MB].reshape(B, MB)
         btv[:n] = block_rows
         btv[n:Bb] = 0
+        hs = hi[4 * B + B * MB:]
+        hs[:n] = state if state is not None else -1
+        hs[n:Bb] = -1
         hl = self.h_i64[k].numpy()
         hl[:n] = slots
         hl[n:Bb] = -1
@@ -200,9 +220,6 @@ class DecodeRunner:
         self.i64.copy_(self.h_i64[k], non_blocking=nb)
         self.f32.copy_(self.h_f32[k], non_blocking=nb)
         g = self._graphs.get(Bb)
-        if g is None and self.use_graphs:
-            self.capture(Bb)
-            g = self._graphs[Bb]
         timing = nb and self.time_gpu
         if timing:
             ev0 = torch.cuda.Event(enable_timing=True)

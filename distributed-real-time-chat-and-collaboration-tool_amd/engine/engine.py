@@ -39,7 +39,6 @@ from ..utils import tracing
 from ..utils.metrics import METRICS
 from ..models.transformer import DecodeMeta, PrefillMeta, TransformerLM
 from .decode_runner import DEFAULT_BUCKETS, DecodeRunner
-from .kv_cache import PagedKVCache
 from .request import Request, RequestState, SamplingParams
 
 BS = ops.KV_BLOCK
@@ -89,14 +88,14 @@ class LLMEngine:
         # fraction and the ranks agree on the smallest resulting block count
         self.hbm_budget = hbm_budget
         if num_blocks is None:
-            num_blocks = PagedKVCache.auto_num_blocks(
-                cfg, model.sh.hkv, self.device, kv_fraction, hbm_budget=hbm_budget,
+            num_blocks = model.auto_num_blocks(
+                max_batch, kv_fraction=kv_fraction, hbm_budget=hbm_budget,
                 weight_bytes=model.weight_bytes() if hbm_budget is not None else None,
                 min_blocks=self.max_blocks)
         # lockstep (SPMD) TP/EP ranks must schedule identically: every rank
         # sizes its cache from the same (smallest) block count
         num_blocks = model.pc.agree_min(num_blocks)
-        self.kv = PagedKVCache(cfg, model.sh.hkv, num_blocks, self.device, model.dtype)
+        self.kv = model.new_cache(num_blocks, max_batch)
         self.alloc = self.kv.allocator
         self.runner = DecodeRunner(model, self.kv, max_batch, self.max_blocks,
                                    use_graphs=use_graphs, seed=seed, buckets=buckets)
@@ -117,6 +116,7 @@ class LLMEngine:
         self.max_new = np.zeros(max_batch, dtype=np.int32)
         self.eos_stop = np.zeros(max_batch, dtype=bool)       # stop on EOS (not ignore_eos)
         self.nblk = np.zeros(max_batch, dtype=np.int32)       # cache blocks held
+        self.sstate = np.full(max_batch, -1, dtype=np.int32)  # recurrent state slot held
         self.stop_ids: dict[int, tuple] = {}                  # slot -> custom stop ids
         self.running: list[Request] = []
         # pipelined decode: the launched-but-unread step, and requests that
@@ -171,7 +171,7 @@ class LLMEngine:
             raise ValueError("empty prompt")
         if n >= self.max_model_len:
             raise ValueError(f"prompt of {n} tokens exceeds max_model_len {self.max_model_len}")
-        if n > self.max_prefill_tokens:
+        if n > self.max_prefill_tokens and not self.model.portions:
             raise ValueError("prompt exceeds max_prefill_tokens")
         with self.lock:
             req.state = RequestState.WAITING
@@ -407,6 +407,8 @@ class LLMEngine:
             self.waiting.popleft()
             self._waiting_tokens -= n
             r.blocks = list(self.alloc.allocate(need))
+            if self.kv.states is not None:  # one per batch slot: a free batch slot has one
+                r.state_slot = self.kv.states.allocate_one()
             batch.append(r)
             tokens += n
         return batch
@@ -425,6 +427,7 @@ class LLMEngine:
         self.max_new[s] = r.params.max_new_tokens
         self.eos_stop[s] = not r.params.ignore_eos
         self.nblk[s] = len(r.blocks)
+        self.sstate[s] = r.state_slot
         if r.params.stop_token_ids and not r.params.ignore_eos:
             self.stop_ids[s] = tuple(r.params.stop_token_ids)
         return s
@@ -437,7 +440,7 @@ class LLMEngine:
             self.running[s] = m
             m.slot = s
             for arr in (self.bt, self.ctx, self.last, self.temp, self.topk, self.topp, self.gen,
-                        self.max_new, self.eos_stop, self.nblk):
+                        self.max_new, self.eos_stop, self.nblk, self.sstate):
                 arr[s] = arr[last]
             moved = self.stop_ids.pop(last, None)
             if moved is not None:
@@ -451,6 +454,9 @@ class LLMEngine:
         if r.blocks:
             self.alloc.free(r.blocks)
             r.blocks = []
+        if r.state_slot >= 0:
+            self.kv.states.free([r.state_slot])
+            r.state_slot = -1
 
     def _finish_check(self, r: Request, tok: int) -> str:
         p = r.params
@@ -481,19 +487,26 @@ class LLMEngine:
             if cur and tok + n > limit:
                 chunks.append(cur)
                 cur, tok = [], 0
-            cur.append(r)
+            if self.model.portions:  # a prompt above the chunk size: portions of it alone
+                while n > limit:
+                    done = r.num_tokens - n
+                    chunks.append([(r, done, limit)])
+                    n -= limit
+                cur.append((r, r.num_tokens - n, n))
+            else:
+                cur.append((r, 0, n))
             tok += n
         chunks.append(cur)
         launched = [self._launch_prefill(c) for c in chunks]
         finished = []
-        for reqs, lens, h_tok, ev in launched:
+        for segs, h_tok, ev in launched:
             if ev is not None:
                 ev.synchronize()
-            h_tok = self._ep_redo_prefill(reqs, 0, h_tok)
-            finished += self._finish_prefill(reqs, lens, h_tok.numpy())
+            h_tok = self._ep_redo_prefill(segs, 0, h_tok)
+            finished += self._finish_prefill(segs, h_tok.numpy())
         return finished
 
-    def _ep_redo_prefill(self, batch: list[Request], n_dec: int, h_tok):
+    def _ep_redo_prefill(self, segs: list[tuple], n_dec: int, h_tok):
         """Capacity-factor EP dispatch (parallel/expert_parallel.py): when the
         chunk's forward dropped (token, expert) pairs on any EP rank, run it
         again at worst-case capacity (same KV slots, same requests; chunks are
@@ -506,29 +519,63 @@ class LLMEngine:
         # the step counter this chunk's first run sampled with (chunks launched after it
         # advanced the counter already): the redo draws from the same stream
         with worst_case_capacity():
-            _, _, h_tok, ev = self._launch_prefill(batch, n_dec=n_dec, step=ent[1])
+            _, h_tok, ev = self._launch_prefill(segs, n_dec=n_dec, step=ent[1])
         if ev is not None:
             ev.synchronize()
         self._h_ovf.pop(id(h_tok), None)
         self.stats["prefill_steps"] -= 1
-        self.stats["prefill_tokens"] -= int(sum(r.num_tokens for r in batch))
+        self.stats["prefill_tokens"] -= sum(n for _, _, n in segs)
         self.stats["ep_redo_steps"] = self.stats.get("ep_redo_steps", 0) + 1
         return h_tok
 
-    def _launch_prefill(self, batch: list[Request], n_dec: int = 0, step: int | None = None):
-        """Enqueue one packed prefill of ``batch``.  ``n_dec > 0`` makes it a
-        mixed step: one decode row per running slot 0..n_dec-1 (padded to the
-        decode bucket) rides in the same forward pass - same GEMM launches,
-        paged attention for those rows - and is sampled with the prefill rows.  ``step``:
-        the sampler's step counter for a redo (default: the next one)."""
+    def _launch_prefill(self, segs: list[tuple], n_dec: int = 0, step: int | None = None):
+        """Enqueue one packed prefill of ``segs`` - (request, first token, tokens): whole
+        prompts, or portions of them (models with ``portions``) - and sample a token after
+        each.  ``n_dec > 0`` makes it a mixed step: one decode row per running slot
+        0..n_dec-1 (padded to the decode bucket) rides in the same forward pass - same GEMM
+        launches, paged attention for those rows - and is sampled with the prefill rows.
+        ``step``: the sampler's step counter for a redo (default: the next one)."""
+        if step is None:
+            self._prefill_step += 1
+            step = self._prefill_step
+        st = self._stage_prefill(
+            [(r, (r.all_ids if r.output_ids else r.prompt_ids)[a:a + n], a) for r, a, n in segs],
+            np.arange(n_dec), self.last[:n_dec], step=step)
+        logits = self.model.forward_prefill(st["ids"], st["meta"], self.kv)
+        cuda = self.device.type == "cuda"
+        toks = ops.sample(logits.to(torch.bfloat16), st["temp"], st["topk"], st["topp"],
+                          seed=self.seed, step=st["step"])
+        h_tok = torch.empty(toks.numel(), dtype=torch.int32, pin_memory=cuda)
+        h_tok.copy_(toks, non_blocking=cuda)
+        ovf = getattr(self.model, "ep_overflow", None)
+        if ovf is not None:  # EP dropped-pair count, read with the tokens
+            h_ovf = torch.empty(1, dtype=torch.int32, pin_memory=cuda)
+            h_ovf.copy_(ovf.count, non_blocking=cuda)
+            self._h_ovf[id(h_tok)] = (h_ovf, step)
+        ev = None
+        if cuda:
+            ev = torch.cuda.Event()
+            ev.record()
+        self.stats["prefill_steps"] += 1
+        self.stats["prefill_tokens"] += sum(n for _, _, n in segs)
+        return segs, h_tok, ev
+
+    def _stage_prefill(self, segs: list[tuple], dec: np.ndarray, dec_ids: np.ndarray,
+                       rows: list | None = None, step: int = 0) -> dict:
+        """Device inputs of one packed step.  ``segs``: (request, token ids, position of the
+        first); ``dec``: running slots that ride along with one token each (``dec_ids``, at
+        position ctx), padded to their decode bucket.  ``rows``: the rows to take logits of,
+        (segment, token) pairs, -1 for a decode row's segment (default: each segment's last
+        token, then every decode row of the bucket)."""
         dev = self.device
         cuda = dev.type == "cuda"
         # host metadata, vectorised over the batch (a 1024-prompt prefill is
         # ~150k tokens: per-request numpy calls would idle the GPU for ~50 ms)
-        seqs = [r.all_ids if r.output_ids else r.prompt_ids for r in batch]
-        nseq = len(batch)
+        batch = [r for r, _, _ in segs]
+        seqs = [ids for _, ids, _ in segs]
+        nseq, n_dec = len(segs), len(dec)
+        starts = np.fromiter((a for _, _, a in segs), dtype=np.int64, count=nseq)
         lens_a = np.fromiter((len(x) for x in seqs), dtype=np.int64, count=nseq)
-        lens = lens_a.tolist()
         cu_a = np.zeros(nseq + 1, dtype=np.int64)
         np.cumsum(lens_a, out=cu_a[1:])
         cu = cu_a.tolist()
@@ -544,16 +591,17 @@ class LLMEngine:
         ids = np.zeros(Tp, dtype=np.int32)
         ids[:T] = np.fromiter(itertools.chain.from_iterable(seqs), dtype=np.int32, count=T)
         seq_of = np.repeat(np.arange(nseq), lens_a)
-        p_tok = np.arange(T, dtype=np.int64) - np.repeat(cu_a[:-1], lens_a)
+        p_tok = np.arange(T, dtype=np.int64) - np.repeat(cu_a[:-1] - starts, lens_a)
         pos = np.zeros(Tp, dtype=np.int32)
         pos[:T] = p_tok
-        nblk = -(-lens_a // BS)
-        blk_tab = np.zeros((nseq, int(nblk.max())), dtype=np.int64)
+        nblk = -(-(starts + lens_a) // BS)
+        blk_tab = np.zeros((nseq, int(nblk.max()) if nseq else 1), dtype=np.int64)
         for i, r in enumerate(batch):
             blk_tab[i, :nblk[i]] = r.blocks[:nblk[i]]
         slots = np.full(Tp, -1, dtype=np.int64)
         slots[:T] = blk_tab[seq_of, p_tok // BS] * BS + p_tok % BS
-        # one V-write segment per (sequence, cache block)
+        # one V-write segment per (sequence, cache block); whole prompts only (the models
+        # with portions have no V cache)
         s_seq = np.repeat(np.arange(nseq), nblk)
         s_j = np.arange(int(nblk.sum()), dtype=np.int64) - np.repeat(np.cumsum(nblk) - nblk, nblk)
         seg_tok = (cu_a[s_seq] + BS * s_j).astype(np.int32)
@@ -561,9 +609,6 @@ class LLMEngine:
         seg_blk = blk_tab[s_seq, s_j].astype(np.int32)
         last_idx = np.asarray(cu[1:], dtype=np.int64) - 1
         ts, tq = ops.prefill_tiles(cu)
-        if step is None:
-            self._prefill_step += 1
-            step = self._prefill_step
         params = np.array([(r.params.temperature, r.params.top_p, r.params.top_k) for r in batch],
                           dtype=np.float64).reshape(nseq, 3)
         dec_i32 = []
@@ -571,15 +616,15 @@ class LLMEngine:
             # decode rows: exactly the staging of a decode step of bucket Bb
             # (padding rows: context 0, no cache write, greedy)
             n, MB = n_dec, self.max_blocks
-            d_pos = self.ctx[:n]
-            d_ids = np.zeros(Bb, np.int32); d_ids[:n] = self.last[:n]
+            d_pos = self.ctx[dec]
+            d_ids = np.zeros(Bb, np.int32); d_ids[:n] = dec_ids
             d_p = np.zeros(Bb, np.int32); d_p[:n] = d_pos
             d_slot = np.full(Bb, -1, np.int64)
-            d_slot[:n] = self.bt[np.arange(n), d_pos // BS].astype(np.int64) * BS + d_pos % BS
+            d_slot[:n] = self.bt[dec, d_pos // BS].astype(np.int64) * BS + d_pos % BS
             d_ctx = np.zeros(Bb, np.int32); d_ctx[:n] = d_pos + 1
-            d_bt = np.zeros((Bb, MB), np.int32); d_bt[:n] = self.bt[:n]
+            d_bt = np.zeros((Bb, MB), np.int32); d_bt[:n] = self.bt[dec]
             d_par = np.zeros((Bb, 3)); d_par[:, 1] = 1.0
-            d_par[:n, 0], d_par[:n, 1], d_par[:n, 2] = self.temp[:n], self.topp[:n], self.topk[:n]
+            d_par[:n, 0], d_par[:n, 1], d_par[:n, 2] = self.temp[dec], self.topp[dec], self.topk[dec]
             ids = np.concatenate([ids, d_ids])
             pos = np.concatenate([pos, d_p])
             slots = np.concatenate([slots, d_slot])
@@ -588,13 +633,24 @@ class LLMEngine:
             dec_i32 = [d_ctx, d_bt.reshape(-1)]
             # the V of decode rows goes through rope_kv_'s own write
             seg_tok = seg_len = seg_blk = np.zeros(0, np.int32)
-        R, ns_all = Tp + Bb, nseq + Bb
+        if rows is not None:  # at least one: the forward pass has no empty form
+            last_idx = np.asarray([Tp + t if q < 0 else cu[q] + t for q, t in rows] or [0], np.int64)
+        R, ns_all, n_rows = Tp + Bb, nseq + Bb, len(last_idx)
+        x32, x64, x_host = {}, {}, None
+        if self.kv.states is not None:
+            d_state = np.full(Bb, -1, np.int64); d_state[:n_dec] = self.sstate[dec]
+            d_start = np.zeros(Bb, np.int64); d_start[:n_dec] = self.ctx[dec]
+            x32, x64, x_host = self.model.step_arrays(
+                lens_a, starts, blk_tab,
+                np.fromiter((r.state_slot for r in batch), np.int64, count=nseq), Tp, d_state,
+                d_start)
         h_i32 = torch.from_numpy(np.concatenate([
             ids, pos, np.asarray(cu, np.int32), np.asarray(ts, np.int32),
             np.asarray(tq, np.int32), seg_tok, seg_len, seg_blk,
-            params[:, 2].astype(np.int32)] + dec_i32))
+            params[:, 2].astype(np.int32)] + dec_i32
+            + [v.astype(np.int32) for v in x32.values()]))
         h_i64 = torch.from_numpy(np.concatenate([
-            slots, last_idx, np.array([step + (1 << 40)], dtype=np.int64)]))
+            slots, last_idx, np.array([step + (1 << 40)], dtype=np.int64), *x64.values()]))
         h_f32 = torch.from_numpy(params[:, :2].T.astype(np.float32).reshape(-1))
         if cuda:  # pinned staging: the copies stay asynchronous to the host
             h_i32, h_i64, h_f32 = h_i32.pin_memory(), h_i64.pin_memory(), h_f32.pin_memory()
@@ -616,37 +672,33 @@ class LLMEngine:
             rm = self.runner._meta(Bb)  # decode partitioning + workspace of bucket Bb
             ctx_d = t_i32[o:o + Bb]; o += Bb
             bt_d = t_i32[o:o + Bb * self.max_blocks].view(Bb, self.max_blocks)
+            o += Bb * self.max_blocks
             dmeta = DecodeMeta(positions=d_pos[Tp:], slots=t_i64[Tp:R], block_tables=bt_d,
                                context_lens=ctx_d, blocks_per_part=rm.blocks_per_part,
                                workspace=rm.workspace)
+        extra = None
+        if x_host is not None:
+            t32, t64, q = {}, {}, R + n_rows + 1
+            for k, v in x32.items():
+                t32[k] = t_i32[o:o + v.size]; o += v.size
+            for k, v in x64.items():
+                t64[k] = t_i64[q:q + v.size]; q += v.size
+            extra = self.model.step_meta(t32, t64, x_host)
         meta = PrefillMeta(positions=d_pos, slots=t_i64[:R], cu_seqlens=d_cu, cu_host=cu,
-                           tiles=(d_ts, d_tq), last_idx=t_i64[R:R + ns_all],
+                           tiles=(d_ts, d_tq), last_idx=t_i64[R:R + n_rows],
                            v_segs=None if n_dec else d_segs, decode=dmeta, n_prefill=Tp,
-                           max_len=int(lens_a.max()))
-        d_step = t_i64[R + ns_all:R + ns_all + 1]
-        temp, topp = t_f32[:ns_all], t_f32[ns_all:]
-        logits = self.model.forward_prefill(d_ids, meta, self.kv)
-        toks = ops.sample(logits, temp, topk, topp, seed=self.seed, step=d_step)
-        h_tok = torch.empty(ns_all, dtype=torch.int32, pin_memory=cuda)
-        h_tok.copy_(toks, non_blocking=cuda)
-        ovf = getattr(self.model, "ep_overflow", None)
-        if ovf is not None:  # EP dropped-pair count, read with the tokens
-            h_ovf = torch.empty(1, dtype=torch.int32, pin_memory=cuda)
-            h_ovf.copy_(ovf.count, non_blocking=cuda)
-            self._h_ovf[id(h_tok)] = (h_ovf, step)
-        ev = None
-        if cuda:
-            ev = torch.cuda.Event()
-            ev.record()
-        self.stats["prefill_steps"] += 1
-        self.stats["prefill_tokens"] += T
-        return batch, lens, h_tok, ev
+                           max_len=int(lens_a.max()) if nseq else 0, extra=extra)
+        return {"ids": d_ids, "meta": meta, "temp": t_f32[:ns_all], "topp": t_f32[ns_all:],
+                "topk": topk, "step": t_i64[R + n_rows:R + n_rows + 1]}
 
-    def _finish_prefill(self, batch: list[Request], lens: list[int], toks) -> list[Request]:
+    def _finish_prefill(self, segs: list[tuple], toks) -> list[Request]:
         """Slot assignment + first-token bookkeeping of one prefill chunk."""
         now = time.perf_counter()
         finished = []
-        for r, n, tok in zip(batch, lens, toks):
+        for (r, a, n), tok in zip(segs, toks):
+            n += a
+            if n < r.num_tokens:
+                continue  # a portion: its prompt goes on in a later chunk
             tok = int(tok)
             s = self._assign_slot(r)
             self.ctx[s] = n
@@ -669,10 +721,11 @@ class LLMEngine:
         launches instead of waiting for the prefill to finish."""
         n = len(self.running)
         reqs = list(self.running)
-        _, lens, h_tok, ev = self._launch_prefill(batch, n_dec=n)
+        segs = [(r, 0, r.num_tokens) for r in batch]
+        _, h_tok, ev = self._launch_prefill(segs, n_dec=n)
         if ev is not None:
             ev.synchronize()
-        h_tok = self._ep_redo_prefill(batch, n, h_tok)
+        h_tok = self._ep_redo_prefill(segs, n, h_tok)
         self.stats["mixed_steps"] += 1
         self.stats["decode_tokens"] += n
         self.ctx[:n] += 1
@@ -685,7 +738,81 @@ class LLMEngine:
         nseq = len(batch)
         st["toks"] = toks[nseq:nseq + n].copy()
         done = self._process(st, later_inflight=False)
-        return done + self._finish_prefill(batch, lens, toks[:nseq])
+        return done + self._finish_prefill(segs, toks[:nseq])
+
+    # ------------------------------------------------------------ given tokens
+    def feed(self, entries: list[tuple[Request, list, list]]) -> list[torch.Tensor]:
+        """One step over given tokens instead of sampled ones: for each (request, next tokens,
+        wanted) runs the tokens after those the request holds and returns the logits of the
+        ``wanted`` places among them, [len(wanted), vocab].  All entries are one batch: single
+        tokens of started requests are decode rows (alone: a decode step through the batch
+        bucket's graph), everything else packed prompt portions.  A request is admitted by its
+        first entry and stays until :meth:`release`; the scheduler (``step``) must be idle."""
+        if self.waiting or self._inflight is not None:
+            raise RuntimeError("feed() while the scheduler has work")
+        segs, dec = [], []
+        for r, toks, _ in entries:
+            if not toks:
+                raise ValueError(f"{r.request_id}: no tokens")
+            if r.state is RequestState.FINISHED:
+                raise ValueError(f"{r.request_id}: finished")
+            if r.slot < 0:
+                if len(self.running) >= self.max_batch:
+                    raise RuntimeError("no free batch slot")
+                if self.kv.states is not None:
+                    r.state_slot = self.kv.states.allocate_one()
+                self._assign_slot(r)
+                self.ctx[r.slot] = 0
+        for e, (r, toks, _) in enumerate(entries):
+            s, start = r.slot, int(self.ctx[r.slot])
+            if start + len(toks) > self.max_model_len:
+                raise ValueError(f"{r.request_id}: longer than max_model_len {self.max_model_len}")
+            if start and len(toks) > 1 and not self.model.portions:
+                raise ValueError(f"{self.cfg.name}: prompts cannot be cut into portions")
+            grow = math.ceil((start + len(toks)) / BS) - len(r.blocks)
+            if grow > 0:
+                r.blocks += self.alloc.allocate(grow)
+                self.bt[s, :len(r.blocks)] = r.blocks
+                self.nblk[s] = len(r.blocks)
+            (dec if start and len(toks) == 1 else segs).append((e, r, start))
+        dslots = np.array([r.slot for _, r, _ in dec], dtype=np.int64)
+        dids = np.array([entries[e][1][0] for e, _, _ in dec], dtype=np.int32)
+        out: list = [None] * len(entries)
+        if segs:
+            rows, owner = [], []
+            for q, (e, r, _) in enumerate(segs):
+                rows += [(q, t) for t in entries[e][2]]
+                owner += [e] * len(entries[e][2])
+            for q, (e, _, _) in enumerate(dec):
+                rows += [(-1, q) for _ in entries[e][2]]
+                owner += [e] * len(entries[e][2])
+            st = self._stage_prefill([(r, entries[e][1], a) for e, r, a in segs], dslots, dids, rows)
+            logits = self.model.forward_prefill(st["ids"], st["meta"], self.kv)
+            for e in range(len(entries)):
+                out[e] = logits[[i for i, o in enumerate(owner) if o == e]]
+        else:
+            pos = self.ctx[dslots]
+            n = len(dec)
+            self.runner.read_logits(n)
+            h = self.runner.launch(n, dids, pos, pos + 1,
+                                   self.bt[dslots, pos // BS].astype(np.int64) * BS + pos % BS,
+                                   self.bt[dslots], np.zeros(n, np.float32),
+                                   np.zeros(n, np.int32), np.ones(n, np.float32),
+                                   self.sstate[dslots])
+            self.runner.wait(h)
+            logits = self.runner.logits[self.runner.bucket(n)]
+            for q, (e, _, _) in enumerate(dec):
+                out[e] = logits[[q] * len(entries[e][2])]
+        for r, toks, _ in entries:
+            self.ctx[r.slot] += len(toks)
+            r.prompt_ids = list(r.prompt_ids) + list(toks)
+        return out
+
+    def release(self, r: Request) -> None:
+        """Finish a request driven by :meth:`feed`: its cache blocks and state slot are free."""
+        if r.slot >= 0:
+            self._release_slot(r)
+        r.mark_finished("released")
 
     # ------------------------------------------------------------ decode
     def _ensure_blocks(self) -> None:
@@ -771,7 +898,7 @@ class LLMEngine:
             return
         order = np.argsort(-ctx, kind="stable")
         for arr in (self.bt, self.ctx, self.last, self.temp, self.topk, self.topp, self.gen,
-                    self.max_new, self.eos_stop, self.nblk):
+                    self.max_new, self.eos_stop, self.nblk, self.sstate):
             arr[:n] = arr[:n][order]
         new_of = np.empty(n, dtype=np.int64)
         new_of[order] = np.arange(n)
@@ -826,7 +953,8 @@ class LLMEngine:
         bidx = pos // BS
         slots = self.bt[np.arange(n), bidx].astype(np.int64) * BS + pos % BS
         handle = self.runner.launch(n, None if pipelined else self.last[:n], pos, pos + 1, slots,
-                                    self.bt[:n], self.temp[:n], self.topk[:n], self.topp[:n])
+                                    self.bt[:n], self.temp[:n], self.topk[:n], self.topp[:n],
+                                    self.sstate[:n])
         self.stats["decode_steps"] += 1
         self.stats["decode_tokens"] += n
         if pipelined:

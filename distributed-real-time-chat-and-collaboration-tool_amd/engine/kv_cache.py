@@ -16,8 +16,8 @@ from __future__ import annotations
 
 import torch
 
-from ..ops import KV_BLOCK
-from ..models.config import ModelConfig
+from ..ops import KV_BLOCK, latent_width
+from ..models.config import HybridConfig, LatentAttention, ModelConfig
 from .block_allocator import BlockAllocator
 
 
@@ -47,6 +47,7 @@ class PagedKVCache:
             self.layers.append((k, v))
         # block 0 is reserved as the padding target of graph-padded slots
         self.allocator = BlockAllocator(self.num_blocks, reserved=1)
+        self.states = None  # no recurrent state
 
     def __getitem__(self, i):
         return self.layers[i]
@@ -73,27 +74,109 @@ class PagedKVCache:
         hbm_budget x the GPU's total HBM after the group's weights (``weight_bytes``; this
         process's allocations when not given) and the reserve, whatever the other groups on the
         GPU - in other processes or in this one - hold or start in what order."""
-        dev = torch.device(device)
-        if dev.type == "cuda":
-            # blocks the caching allocator holds but no tensor uses are free HBM here: release
-            # them so that neither the free figure nor this process's own share counts them
-            torch.cuda.empty_cache()
-            free, total = torch.cuda.mem_get_info(dev)
-            budget = int(max(0, free - reserve_bytes) * kv_fraction)
-            if hbm_budget is not None:
-                mine = torch.cuda.memory_reserved(dev) if weight_bytes is None else weight_bytes
-                left = int(hbm_budget * total) - mine - reserve_bytes
-                if blocks_for_budget(cfg, hkv_local, cfg.num_layers, max(left, 0)) < min_blocks:
-                    # ``min_blocks``: the cache of one max_model_len sequence
-                    raise ValueError(
-                        f"{cfg.name}: an HBM budget of {hbm_budget:.2f} x {total / 1e9:.0f} GB "
-                        f"on {dev} leaves {left / 1e9:.1f} GB for the KV cache after "
-                        f"{mine / 1e9:.1f} GB of weights and the {reserve_bytes / 1e9:.0f} GB "
-                        f"reserve: less than one {min_blocks}-block sequence needs")
-                budget = min(budget, max(left, 0))
-        else:
-            budget = 256 << 20
-        n = blocks_for_budget(cfg, hkv_local, cfg.num_layers, budget)
-        if max_blocks is not None:
-            n = min(n, max_blocks)
-        return max(n, 2)
+        per_block = 2 * cfg.num_layers * hkv_local * KV_BLOCK * cfg.head_dim * 2
+        return _budget_blocks(cfg.name, per_block, 0, device, kv_fraction, reserve_bytes,
+                              max_blocks, hbm_budget, weight_bytes, min_blocks)
+
+
+def _budget_blocks(name: str, per_block: int, fixed: int, device, kv_fraction: float,
+                   reserve_bytes: int, max_blocks: int | None, hbm_budget: float | None,
+                   weight_bytes: int | None, min_blocks: int) -> int:
+    """Blocks of ``per_block`` bytes beside ``fixed`` bytes of other cache (see
+    PagedKVCache.auto_num_blocks)."""
+    dev = torch.device(device)
+    if dev.type == "cuda":
+        # blocks the caching allocator holds but no tensor uses are free HBM here: release
+        # them so that neither the free figure nor this process's own share counts them
+        torch.cuda.empty_cache()
+        free, total = torch.cuda.mem_get_info(dev)
+        budget = int(max(0, free - reserve_bytes) * kv_fraction)
+        if hbm_budget is not None:
+            mine = torch.cuda.memory_reserved(dev) if weight_bytes is None else weight_bytes
+            left = int(hbm_budget * total) - mine - reserve_bytes
+            if max(left - fixed, 0) // max(1, per_block) < min_blocks:
+                # ``min_blocks``: the cache of one max_model_len sequence
+                raise ValueError(
+                    f"{name}: an HBM budget of {hbm_budget:.2f} x {total / 1e9:.0f} GB "
+                    f"on {dev} leaves {left / 1e9:.1f} GB for the KV cache after "
+                    f"{mine / 1e9:.1f} GB of weights and the {reserve_bytes / 1e9:.0f} GB "
+                    f"reserve: less than one {min_blocks}-block sequence needs")
+            budget = min(budget, max(left, 0))
+    else:
+        budget = 256 << 20
+    n = max(0, budget - fixed) // max(1, per_block)
+    if max_blocks is not None:
+        n = min(n, max_blocks)
+    return max(n, 2)
+
+
+class HybridCache:
+    """Cache of a model with mixed layer kinds: paged latents for its attention layers, and
+    state slots - one per live sequence - for its recurrent layers.
+
+      latent layer : [num_blocks, 32, latent_width]      (ops/latent.py)
+      delta layer  : ring  [slots, taps, channels]       last convolution inputs
+                     state [slots, heads, dim, vdim]     fp32
+
+    Blocks come from ``allocator`` (block 0 is the padding target), slots from ``states``.
+    A slot needs no clearing: a sequence starts from zero at its position 0 whatever the slot
+    holds (csrc/kernels/delta_rule.hip)."""
+
+    def __init__(self, cfg: HybridConfig, num_blocks: int, num_slots: int,
+                 device: torch.device | str, dtype=torch.bfloat16):
+        self.cfg, self.block_size = cfg, KV_BLOCK
+        self.num_blocks, self.num_slots = int(num_blocks), int(num_slots)
+        self.layers = []
+        for l in cfg.layers:
+            m = l.mixer
+            if isinstance(m, LatentAttention):
+                # zero-filled: rows behind a sequence's end are read (and masked) with its block
+                self.layers.append(torch.zeros(
+                    (self.num_blocks, KV_BLOCK, latent_width(m.kv_rank, m.rot_dim)), dtype=dtype,
+                    device=device))
+            else:
+                self.layers.append((
+                    torch.zeros((self.num_slots, m.conv, m.channels), dtype=dtype, device=device),
+                    torch.zeros((self.num_slots, m.heads, m.dim, m.vdim), dtype=torch.float32,
+                                device=device)))
+        self.allocator = BlockAllocator(self.num_blocks, reserved=1)
+        self.states = BlockAllocator(self.num_slots, reserved=0)
+
+    def __getitem__(self, i):
+        return self.layers[i]
+
+    def __len__(self):
+        return len(self.layers)
+
+    @property
+    def bytes(self) -> int:
+        ts = [t for l in self.layers for t in (l if isinstance(l, tuple) else (l,))]
+        return sum(t.numel() * t.element_size() for t in ts)
+
+    @property
+    def capacity_tokens(self) -> int:
+        return (self.num_blocks - 1) * KV_BLOCK
+
+    @staticmethod
+    def sizes(cfg: HybridConfig, dtype_bytes: int) -> tuple[int, int]:
+        """(bytes of a block over all layers, bytes of a state slot over all layers)."""
+        block = slot = 0
+        for l in cfg.layers:
+            m = l.mixer
+            if isinstance(m, LatentAttention):
+                block += KV_BLOCK * latent_width(m.kv_rank, m.rot_dim) * dtype_bytes
+            else:
+                slot += m.conv * m.channels * dtype_bytes + m.heads * m.dim * m.vdim * 4
+        return block, slot
+
+    @staticmethod
+    def auto_num_blocks(cfg: HybridConfig, num_slots: int, device, dtype=torch.bfloat16,
+                        kv_fraction: float = 0.85, reserve_bytes: int = 8 << 30,
+                        max_blocks: int | None = None, hbm_budget: float | None = None,
+                        weight_bytes: int | None = None, min_blocks: int = 0) -> int:
+        """Blocks beside ``num_slots`` state slots (budget: PagedKVCache.auto_num_blocks).  A
+        model without attention layers pays nothing for blocks; 1M of them at most."""
+        block, slot = HybridCache.sizes(cfg, torch.empty((), dtype=dtype).element_size())
+        n = _budget_blocks(cfg.name, block, slot * num_slots, device, kv_fraction, reserve_bytes,
+                           max_blocks, hbm_budget, weight_bytes, min_blocks)
+        return min(n, 1 << 20) if block == 0 else n

@@ -46,6 +46,7 @@ class Request:
     # engine-managed state
     output_ids: list = field(default_factory=list)
     blocks: list = field(default_factory=list)
+    state_slot: int = -1  # recurrent state held (models with recurrent layers)
     state: RequestState = RequestState.WAITING
     slot: int = -1
     finish_reason: str = ""
