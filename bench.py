@@ -41,7 +41,7 @@ from drtc_amd.engine import ChatTokenizer, LLMEngine, Request, SamplingParams  #
 from drtc_amd.engine.engine import freeze_gc  # noqa: E402
 from drtc_amd.llm import prompts as P  # noqa: E402
 from drtc_amd.llm.service import FeatureParams  # noqa: E402
-from drtc_amd.models import TransformerLM, get_config  # noqa: E402
+from drtc_amd.models import build_model, get_config  # noqa: E402
 from drtc_amd.parallel import init_distributed  # noqa: E402
 from drtc_amd.utils.synthetic import channel_history  # noqa: E402
 
@@ -287,7 +287,7 @@ def main() -> None:
     else:
         pc = None
     dp_rank = 0 if tp > 1 else rank
-    model = TransformerLM(cfg, device, pc=pc, seed=1234, full_then_shard=False)
+    model = build_model(cfg, device, pc=pc, seed=1234, full_then_shard=False)
     eng = LLMEngine(model, max_batch=args.batch, max_model_len=args.max_model_len,
                     max_prefill_tokens=max(16384, args.batch * 400),
                     kv_fraction=args.kv_fraction, use_graphs=not args.no_graphs, seed=dp_rank)

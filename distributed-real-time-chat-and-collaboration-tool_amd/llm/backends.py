@@ -110,13 +110,13 @@ def _worker_main(rank: int, device: str, model_name: str, engine_kw: dict, inq, 
 
     from ..engine.engine import EngineLoop, LLMEngine, freeze_gc
     from ..engine.tokenizer import ChatTokenizer
-    from ..models import TransformerLM, get_config
+    from ..models import load_model
 
     try:
         if device.startswith("cuda"):
             torch.cuda.set_device(torch.device(device))
-        cfg = get_config(model_name)
-        model = TransformerLM(cfg, device, seed=seed, full_then_shard=False)
+        model = load_model(model_name, device, seed=seed, full_then_shard=False)
+        cfg = model.cfg
         eng = LLMEngine(model, seed=rank, **engine_kw)
         # prompt text is tokenized (and replies detokenized) here, beside the engine, so the
         # gRPC front-end's single GIL only carries RPC handling (llm/backends.py ReplicaRouter)

@@ -91,11 +91,11 @@ def build_backend(args, devices: list[int] | None = None):
     n = len(devices) if devices else args.gpus
     if n <= 1 and (getattr(args, "in_process", False) or not torch.cuda.is_available()):
         from ..engine.engine import LLMEngine
-        from ..models import TransformerLM
+        from ..models import load_model
         from .backends import EngineBackend
 
         dev = f"cuda:{devices[0] if devices else 0}" if torch.cuda.is_available() else "cpu"
-        model = TransformerLM(cfg, dev, seed=1234, full_then_shard=False)
+        model = load_model(args.model, dev, seed=1234, full_then_shard=False)
         eng = LLMEngine(model, **engine_kw)
         eng.warmup(capture=True)
         return EngineBackend(eng, tok)
@@ -309,7 +309,9 @@ def main(argv=None):
     ap = argparse.ArgumentParser(description="drtc_amd LLM service (on-GPU inference)")
     ap.add_argument("--port", type=int, default=50055)
     ap.add_argument("--backend", choices=("engine", "scripted"), default="engine")
-    ap.add_argument("--model", default="llama-3-8b")
+    ap.add_argument("--model", default="llama-3-8b",
+                    help="a registered model (random weights), or a checkpoint folder with "
+                         "config.json and model.safetensors")
     ap.add_argument("--gpus", type=int, default=1, help="data-parallel replicas (1 process/GPU)")
     ap.add_argument("--tp", type=int, default=1, help="tensor-parallel degree")
     ap.add_argument("--custom-allreduce", dest="custom_allreduce", action="store_true",

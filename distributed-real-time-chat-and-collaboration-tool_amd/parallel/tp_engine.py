@@ -54,7 +54,7 @@ def tp_worker(rank: int, world: int, port: int, model_name: str, engine_kw: dict
     import torch.distributed as dist
 
     from ..engine.engine import LLMEngine
-    from ..models import TransformerLM, get_config
+    from ..models import build_model, get_config
     from .comm import ParallelContext, init_distributed
 
     try:
@@ -74,7 +74,7 @@ def tp_worker(rank: int, world: int, port: int, model_name: str, engine_kw: dict
         if custom_ar and dev.type == "cuda":
             pc.enable_custom_allreduce()
         cfg = get_config(model_name)
-        model = TransformerLM(cfg, dev, pc=pc, seed=1234)
+        model = build_model(cfg, dev, pc=pc, seed=1234)
         eng = LLMEngine(model, seed=0, **engine_kw)
         # ranks finish weight init at different times; the custom all-reduce's
         # flag waits are time-bounded, so enter the captured warm-up together

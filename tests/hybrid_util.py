@@ -1,0 +1,130 @@
+"""Small random models of mixed layer kinds for the tests: configuration dicts in the
+checkpoint's format, weights under its names, checkpoint folders, and error measures."""
+from __future__ import annotations
+
+import json
+import os
+import struct
+
+import torch
+
+
+def latent(heads, dim, rot, vdim, rank, window, base=10000.0, scale=None, ff=None):
+    return {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff} if ff else None,
+            "mixer": {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": rank,
+                      "scale": scale or (dim + rot) ** -0.5, "mask": {"size": window},
+                      "rot": {"base": base, "dims": rot}}}
+
+
+def delta(heads, kv_heads, dim, vdim, taps, ff=None):
+    return {"type": "channel_delta", "mlp": {"kind": "dense", "ff": ff} if ff else None,
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": taps}}
+
+
+def config(vocab, width, *layers, eps=1e-5):
+    return {"architecture": "Ralesun", "vocab": vocab, "width": width, "norm": {"eps": eps},
+            "layers": list(layers)}
+
+
+CONFIGS = {
+    # grouped key heads, both kinds with and without a feed-forward, two windows
+    "mixed": config(320, 192, delta(4, 2, 16, 24, 3, ff=320), latent(3, 24, 8, 40, 64, 37),
+                    delta(2, 2, 40, 32, 4), latent(5, 16, 16, 32, 48, 70, 500.0, 0.3, ff=256)),
+    # two head tiles in decode, window a multiple of nothing, three heads to a key head
+    "wide": config(256, 512, latent(20, 64, 32, 64, 160, 100, ff=96), delta(6, 2, 72, 136, 2)),
+    # sizes no vector path takes
+    "odd": config(203, 100, latent(2, 12, 6, 20, 52, 33, ff=50), delta(3, 1, 20, 17, 5, ff=30)),
+    # large latents and heads, more heads than a decode workgroup, long rows of state
+    "large": config(128, 256, latent(70, 64, 64, 128, 448, 90), delta(2, 1, 160, 300, 1),
+                    latent(17, 128, 64, 136, 512, 64), delta(2, 2, 128, 128, 4)),
+    # windows of one and two tokens, a window larger than any prompt
+    "narrow": config(96, 64, latent(2, 16, 8, 16, 32, 1), latent(2, 16, 8, 16, 32, 2),
+                     delta(1, 1, 8, 8, 2), latent(2, 32, 32, 64, 40, 5000, ff=64)),
+    # recurrent layers only
+    "recurrent": config(96, 64, delta(2, 2, 24, 16, 4, ff=72), delta(4, 1, 16, 32, 3)),
+}
+
+
+def weights(cfg, seed=0):
+    """Random tensors (bf16-representable).  Queries are loud, so that single keys stand out of a
+    window, and decays span slow and fast channels."""
+    g = torch.Generator().manual_seed(seed)
+    out = {}
+
+    def put(name, *shape, std=None, mean=0.0):
+        std = shape[-1] ** -0.5 if std is None else std
+        out[name] = (torch.randn(*shape, generator=g) * std + mean).to(torch.bfloat16)
+
+    def norm(name, W):
+        put(name, W, std=0.2, mean=1.0)
+        put(name + ".b", W, std=0.1)
+        out[name + ".alpha"] = (0.3 + 0.5 * torch.rand((), generator=g)).to(torch.bfloat16)
+
+    V, W = cfg["vocab"], cfg["width"]
+    put("embed", V, W, std=1.5)
+    for i, l in enumerate(cfg["layers"]):
+        m, p = l["mixer"], f"l{i}.mix."
+        norm(f"l{i}.norm1", W)
+        if l["type"] == "latent_attention":
+            H, R = m["heads"], m["kv_rank"]
+            put(p + "q", H * (m["dim"] + m["rot_dim"]), W, std=3 * W ** -0.5)
+            put(p + "dkv", R + m["rot_dim"], W, std=2 * W ** -0.5)
+            put(p + "dkv.norm", R, std=0.2, mean=1.0)
+            put(p + "uk", H * m["dim"], R)
+            put(p + "uv", H * m["vdim"], R)
+            put(p + "sink", H, std=1.0, mean=1.5)
+            put(p + "o", W, H * m["vdim"], std=2 * (H * m["vdim"]) ** -0.5)
+        else:
+            H, Hk, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            ra, rg = d // 2 + 3, dv // 2 + 1
+            for x, n in (("q", Hk * d), ("k", Hk * d), ("v", H * dv)):
+                put(p + x, n, W, std=2 * W ** -0.5)
+                put(p + x + ".conv", n, m["conv"], std=m["conv"] ** -0.5)
+            put(p + "b", H, W, std=2 * W ** -0.5)
+            put(p + "A_log", H, std=0.7)
+            put(p + "norm", dv, std=0.2, mean=1.0)
+            put(p + "a1", ra, W)
+            put(p + "a2", H * d, ra)
+            put(p + "dt_bias", H * d, std=1.5, mean=-3.0)
+            put(p + "g1", rg, W)
+            put(p + "g2", H * dv, rg)
+            put(p + "o", W, H * dv, std=2 * (H * dv) ** -0.5)
+        if l["mlp"]:
+            ff = l["mlp"]["ff"]
+            norm(f"l{i}.norm2", W)
+            put(f"l{i}.mlp.gate", ff, W, std=2 * W ** -0.5)
+            put(f"l{i}.mlp.up", ff, W)
+            put(f"l{i}.mlp.down", W, ff, std=2 * ff ** -0.5)
+    norm("final.norm", W)
+    put("head", V, W)
+    return out
+
+
+def save_checkpoint(path, cfg, tensors) -> str:
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    names, head, data = sorted(tensors), {}, b""
+    kinds = {torch.bfloat16: "BF16", torch.float32: "F32", torch.int32: "I32"}
+    for n in names:
+        t = tensors[n].contiguous()
+        raw = t.reshape(-1).view(torch.uint8).numpy().tobytes()
+        head[n] = {"dtype": kinds[t.dtype], "shape": list(t.shape),
+                   "data_offsets": [len(data), len(data) + len(raw)]}
+        data += raw
+    blob = json.dumps(head).encode()
+    with open(os.path.join(path, "model.safetensors"), "wb") as f:
+        f.write(struct.pack("<Q", len(blob)) + blob + data)
+    return str(path)
+
+
+def tokens(cfg, n, seed):
+    g = torch.Generator().manual_seed(1000 + seed)
+    return torch.randint(0, cfg["vocab"], (n,), generator=g).tolist()
+
+
+def row_errors(got, want):
+    """RMS of each row's difference (mean taken off) over the RMS of all of ``want``."""
+    d = got.double().cpu() - want.double().cpu()
+    d = d - d.mean(-1, keepdim=True)
+    return d.pow(2).mean(-1).sqrt() / want.double().std()
