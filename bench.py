@@ -209,8 +209,87 @@ def self_launch(n: int) -> int:
     return rc if rc else (0 if any(ln.startswith("{") for ln in out.splitlines()) else 1)
 
 
+# ------------------------------------------------------------------ design comparison
+# Layer stacks of equal parameter count at two widths: three pairs of Ralesun layers (latent
+# attention + feed-forward, then a bare delta-rule layer) against four Llama-shaped layers.
+DESIGN_SIZES = {2048: (16, 4, 7168), 4096: (32, 8, 14336)}  # width -> heads, kv heads, ff
+DESIGN_VOCAB = 32000
+
+
+def design_configs(width: int) -> dict:
+    from drtc_amd.models.config import ChannelDelta, HybridConfig, LatentAttention, Layer, ModelConfig
+
+    H, Hk, ff = DESIGN_SIZES[width]
+    att = LatentAttention(H, 128, 64, 128, 512, 192 ** -0.5, 1024, 500000.0, 64)
+    return {
+        "ralesun": HybridConfig(f"ralesun-{width}", DESIGN_VOCAB, width,
+                                (Layer(att, ff), Layer(ChannelDelta(H, H, 128, 128, 4, 128, 128))) * 3),
+        "llama": ModelConfig(f"llama-{width}", DESIGN_VOCAB, width, ff, 4, H, Hk, 128)}
+
+
+def design_bench(args) -> None:
+    """Prefill and decode throughput of the Ralesun design beside Llama-shaped layers of equal
+    size (random weights), GPU time only; one JSON line per (width, family, case)."""
+    dev = torch.device("cuda", 0)
+    for width in map(int, args.design_widths.split(",")):
+        for fam, cfg in design_configs(width).items():
+            if fam not in args.design_families.split(","):
+                continue
+            model = build_model(cfg, dev, seed=1, full_then_shard=False)
+            base = {"bench": "design", "width": width, "family": fam, "layers": cfg.num_layers,
+                    "params_m": round(cfg.num_params() / 1e6), "dtype": "bf16",
+                    "data": "random tokens, random-init weights"}
+            g = torch.Generator().manual_seed(0)
+
+            def prompts(n, length):
+                return torch.randint(0, DESIGN_VOCAB, (n, length), generator=g).tolist()
+
+            if "prefill" in args.design_phases:
+                for n, length in ((64, 256), (16, 1024), (4, 4096)):
+                    eng = LLMEngine(model, max_batch=n, max_model_len=length + 32,
+                                    num_blocks=n * (length // 32 + 1) + 2)
+                    reqs = [eng.add_request(Request(p, SamplingParams.greedy(2))) for p in prompts(n, length)]
+                    with eng.lock:
+                        eng._admit(n * length)
+                    st = eng._stage_prefill([(r, r.prompt_ids, 0) for r in reqs],
+                                            eng.ctx[:0].astype("int64"), eng.last[:0])
+                    for _ in range(args.warmup + 2):
+                        model.forward_prefill(st["ids"], st["meta"], eng.kv)
+                    e0, e1 = (torch.cuda.Event(enable_timing=True) for _ in range(2))
+                    iters = 4 * args.steps
+                    e0.record()
+                    for _ in range(iters):
+                        model.forward_prefill(st["ids"], st["meta"], eng.kv)
+                    e1.record()
+                    torch.cuda.synchronize()
+                    ms = e0.elapsed_time(e1) / iters
+                    print(json.dumps({**base, "phase": "prefill", "sequences": n, "length": length,
+                                      "ms": round(ms, 3), "tokens_per_s": round(1000 * n * length / ms)}),
+                          flush=True)
+                    del eng, st
+            if "decode" in args.design_phases:
+                for B, ctx in ((16, 1024), (256, 1024), (64, 4096)):
+                    eng = LLMEngine(model, max_batch=B, max_model_len=ctx + 64,
+                                    num_blocks=B * (ctx // 32 + 3) + 2, max_prefill_tokens=B * ctx)
+                    eng.runner.time_gpu = True
+                    eng.generate(prompts(B, ctx), SamplingParams.greedy(12 + 8 * args.steps, ignore_eos=True))
+                    ms = statistics.median(eng.runner.gpu_ms[8:])
+                    print(json.dumps({**base, "phase": "decode", "sequences": B, "context": ctx,
+                                      "ms": round(ms, 3), "tokens_per_s": round(1000 * B / ms)}),
+                          flush=True)
+                    del eng
+            del model
+            torch.cuda.empty_cache()
+
+
 def main() -> None:
     ap = argparse.ArgumentParser()
+    ap.add_argument("--design", action="store_true",
+                    help="instead of the serving workload: prefill / decode throughput of the "
+                         "Ralesun design beside Llama-shaped layers of equal size")
+    ap.add_argument("--design-widths", default="2048,4096")
+    ap.add_argument("--design-families", default="ralesun,llama")
+    ap.add_argument("--design-phases", default="prefill,decode")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
@@ -243,6 +322,8 @@ def main() -> None:
                     help="prompt-token budget of a mixed prefill+decode step")
     ap.add_argument("--no-mixed", action="store_true", help="strict prefill-first scheduling")
     args = ap.parse_args()
+    if args.design:
+        return design_bench(args)
     if "WORLD_SIZE" not in os.environ and args.gpus > 1:
         sys.exit(self_launch(args.gpus))
     if int(os.environ.get("WORLD_SIZE", "1")) != args.gpus:

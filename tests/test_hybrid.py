@@ -396,8 +396,9 @@ def feed_all(eng, toks, cuts):
 def agree(got, want, dtype):
     e = row_errors(got, want)
     assert not torch.isnan(e).any()
-    limit = tol(dtype, 2e-4, 0.1)
-    assert e.max() <= limit, (int(e.argmax()), float(e.max()))
+    # a few positions amplify bf16 rounding (a short read-out, divided by its own size)
+    assert e.max() <= tol(dtype, 2e-4, 0.2), (int(e.argmax()), float(e.max()))
+    assert (e > 0.1).sum() <= max(1, e.numel() // 50)
 
 
 @on
@@ -530,11 +531,12 @@ def _mutations():
 @pytest.mark.parametrize("mistake", list(_mutations()))
 def test_mistakes_show(mistake):
     """The tests' models and tolerances can tell: each mistake, planted in the oracle, moves
-    some logits by more than the loosest limit."""
+    some logits by more than the loosest limit, several by more than half of it."""
     cfg, w = case("mixed")
     toks = tokens(cfg, 150, 1)
     got = O.forward(*_mutations()[mistake](cfg, w), toks)[0]
-    assert row_errors(got, expected("mixed", toks)).max() > 0.1
+    e = row_errors(got, expected("mixed", toks))
+    assert e.max() > 0.2 and (e > 0.1).sum() > 3
 
 
 # ------------------------------------------------------------------ scheduler, sampler, command line
