@@ -247,7 +247,7 @@ def design_bench(args) -> None:
             if "prefill" in args.design_phases:
                 for n, length in ((64, 256), (16, 1024), (4, 4096)):
                     eng = LLMEngine(model, max_batch=n, max_model_len=length + 32,
-                                    num_blocks=n * (length // 32 + 1) + 2)
+                                    num_blocks=n * (length // 32 + 2) * 9 // 8 + 2)
                     reqs = [eng.add_request(Request(p, SamplingParams.greedy(2))) for p in prompts(n, length)]
                     with eng.lock:
                         eng._admit(n * length)
@@ -270,7 +270,7 @@ def design_bench(args) -> None:
             if "decode" in args.design_phases:
                 for B, ctx in ((16, 1024), (256, 1024), (64, 4096)):
                     eng = LLMEngine(model, max_batch=B, max_model_len=ctx + 64,
-                                    num_blocks=B * (ctx // 32 + 3) + 2, max_prefill_tokens=B * ctx)
+                                    num_blocks=B * (ctx // 32 + 4) * 9 // 8 + 2, max_prefill_tokens=B * ctx)
                     eng.runner.time_gpu = True
                     eng.generate(prompts(B, ctx), SamplingParams.greedy(12 + 8 * args.steps, ignore_eos=True))
                     ms = statistics.median(eng.runner.gpu_ms[8:])

@@ -38,60 +38,122 @@ DRTC_DEVICE bf16x8 zero8() {
 }
 
 // ------------------------------------------------------------------ per-token preparation
-template <class T>
+// One workgroup per token.  V: elements a thread moves at once (8, or 2 where the sizes or the
+// rows do not align); pairs never straddle a vector.
+template <class T, int V>
+DRTC_DEVICE void lat_load(float (&v)[V], const T* p) {
+  if constexpr (V == 8) load8(v, p);
+  else {
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = to_f32(p[j]);
+  }
+}
+template <class T, int V>
+DRTC_DEVICE void lat_store(T* p, const float (&v)[V]) {
+  if constexpr (V == 8) store8(p, v);
+  else {
+#pragma unroll
+    for (int j = 0; j < V; ++j) p[j] = from_f32<T>(v[j]);
+  }
+}
+
+template <class T, int V>
 __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrepArgs a) {
   __shared__ float red[16];
   const int row = blockIdx.x, tid = threadIdx.x;
   T* pr = (T*)a.proj + (int64_t)row * a.ldp;
   const T* kv = pr + a.off_kv;
-  float ss = 0.f;
-  for (int i = tid; i < a.R; i += 256) {
-    const float x = to_f32(kv[i]);
-    ss += x * x;
+  const int half = a.rot_dims >> 1;
+  const float* cs = a.cos_sin + (int64_t)a.positions[row] * a.rot_dims;
+  // V elements of a rotated part from element i on
+  auto turn = [&](const T* src, T* dst, int i) {
+    float x[V];
+    lat_load<T, V>(x, src + i);
+#pragma unroll
+    for (int j = 0; j < V; j += 2) {
+      const int k = (i + j) >> 1;
+      if (k < half) {
+        const float u = x[j], v = x[j + 1], c = cs[k], s = cs[half + k];
+        x[j] = u * c - v * s;
+        x[j + 1] = v * c + u * s;
+      }
+    }
+    lat_store<T, V>(dst + i, x);
+  };
+  // queries: in place, or into the latent-space query rows
+  const int dq = a.dim + a.rot;
+  if (a.qa) {
+    const int tail = (a.LW - a.R) / V, own = a.rot / V;
+    for (int k = tid; k < a.H * tail; k += 256) {
+      const int h = k / tail, i = k - h * tail;
+      T* d = (T*)a.qa + ((int64_t)row * a.H + h) * a.LW + a.R;
+      if (i < own) turn(pr + h * dq + a.dim, d, i * V);
+      else {
+#pragma unroll
+        for (int j = 0; j < V; ++j) d[i * V + j] = from_f32<T>(0.f);
+      }
+    }
+  } else {
+    const int per = (a.rot_dims + V - 1) / V;
+    for (int k = tid; k < a.H * per; k += 256) {
+      const int h = k / per;
+      T* q = pr + h * dq + a.dim;
+      turn(q, q, (k - h * per) * V);
+    }
   }
-  const float rinv = 1.f / sqrtf(block_sum(ss, red) / (float)a.R + a.eps);
   const int64_t slot = a.slots ? a.slots[row] : -1;
   T* lat = a.lat ? (T*)a.lat + (int64_t)row * a.LW : nullptr;
   T* cache = a.cache && slot >= 0 ? (T*)a.cache + slot * a.LW : nullptr;
-  auto put = [&](int i, T v) {
-    if (lat) lat[i] = v;
-    if (cache) cache[i] = v;
-  };
-  for (int i = tid; i < a.R; i += 256) put(i, from_f32<T>(to_f32(kv[i]) * rinv * a.norm_w[i]));
-  const int half = a.rot_dims >> 1;
-  const float* cs = a.cos_sin + (int64_t)a.positions[row] * a.rot_dims;
-  for (int i = tid; i < half; i += 256) {
-    const float u = to_f32(kv[a.R + 2 * i]), v = to_f32(kv[a.R + 2 * i + 1]);
-    put(a.R + 2 * i, from_f32<T>(u * cs[i] - v * cs[half + i]));
-    put(a.R + 2 * i + 1, from_f32<T>(v * cs[i] + u * cs[half + i]));
+  float ss = 0.f;
+  for (int i = tid * V; i < a.R; i += 256 * V) {
+    float x[V];
+    lat_load<T, V>(x, kv + i);
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss += x[j] * x[j];
   }
-  for (int i = a.R + a.rot_dims + tid; i < a.LW; i += 256)
-    put(i, i < a.R + a.rot ? kv[i] : from_f32<T>(0.f));
-  // queries: in place, or into the latent-space query rows
-  const int dq = a.dim + a.rot;
-  for (int k = tid; k < a.H * half; k += 256) {
-    const int h = k / half, i = k - h * half;
-    T* q = pr + h * dq + a.dim + 2 * i;
-    T* d = a.qa ? (T*)a.qa + ((int64_t)row * a.H + h) * a.LW + a.R + 2 * i : q;
-    const float u = to_f32(q[0]), v = to_f32(q[1]);
-    d[0] = from_f32<T>(u * cs[i] - v * cs[half + i]);
-    d[1] = from_f32<T>(v * cs[i] + u * cs[half + i]);
-  }
-  if (a.qa) {
-    const int tail = a.LW - a.R - a.rot_dims;
-    for (int k = tid; k < a.H * tail; k += 256) {
-      const int h = k / tail, i = a.rot_dims + (k - h * tail);
-      ((T*)a.qa)[((int64_t)row * a.H + h) * a.LW + a.R + i] =
-          i < a.rot ? pr[h * dq + a.dim + i] : from_f32<T>(0.f);
+  const float rinv = 1.f / sqrtf(block_sum(ss, red) / (float)a.R + a.eps);
+  for (int i = tid * V; i < a.LW; i += 256 * V) {
+    float x[V];
+    if (i < a.R) {
+      lat_load<T, V>(x, kv + i);
+#pragma unroll
+      for (int j = 0; j < V; ++j) x[j] *= rinv * a.norm_w[i + j];
+    } else if (i < a.R + a.rot) {
+      lat_load<T, V>(x, kv + i);
+#pragma unroll
+      for (int j = 0; j < V; j += 2) {
+        const int k = (i + j - a.R) >> 1;
+        if (k < half) {
+          const float u = x[j], v = x[j + 1], c = cs[k], s = cs[half + k];
+          x[j] = u * c - v * s;
+          x[j + 1] = v * c + u * s;
+        }
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < V; ++j) x[j] = 0.f;
     }
+    if (lat) lat_store<T, V>(lat + i, x);
+    if (cache) lat_store<T, V>(cache + i, x);
   }
+}
+
+template <class T>
+static void lat_prep_t(const LatentPrepArgs& a, hipStream_t st) {
+  if (a.R % 8 == 0 && a.rot % 8 == 0 && a.dim % 8 == 0 && a.ldp % 8 == 0 && a.off_kv % 8 == 0 &&
+      a.LW % 8 == 0)
+    latent_prep_kernel<T, 8><<<dim3(a.rows), dim3(256), 0, st>>>(a);
+  else
+    latent_prep_kernel<T, 2><<<dim3(a.rows), dim3(256), 0, st>>>(a);
 }
 
 int launch_latent_prep(int f32, const LatentPrepArgs& a, hipStream_t st) {
   if (a.rows == 0) return 0;
-  if (a.rot_dims > a.rot || a.rot_dims % 2 || a.R + a.rot > a.LW) return -1;
-  if (f32) latent_prep_kernel<float><<<dim3(a.rows), dim3(256), 0, st>>>(a);
-  else latent_prep_kernel<bf16_t><<<dim3(a.rows), dim3(256), 0, st>>>(a);
+  if (a.rot_dims > a.rot || a.rot_dims % 2 || a.R + a.rot > a.LW || a.R % 2 || a.rot % 2 ||
+      a.LW % 2)
+    return -1;
+  if (f32) lat_prep_t<float>(a, st);
+  else lat_prep_t<bf16_t>(a, st);
   return (int)hipGetLastError();
 }
 
@@ -212,27 +274,31 @@ __global__ __launch_bounds__(256) void latent_decode_any_kernel(LatentDecodeArgs
 }
 
 // ------------------------------------------------------------------ prompt portions on MFMA
-// Workgroup: 4 waves, QF x 16 query rows each, one head.  K tile [64 keys][DKP] (per-head part,
-// then the shared rotated part) and V tile [64][DVP] double-buffered in LDS; the next tile's
-// global loads are in flight during this tile's MFMAs.  S^T = K Q^T, so its accumulators are
-// the P^T operand of O^T = V^T P^T without lane movement.
+// Workgroup: NW waves, QF x 16 query rows each, one head.  K tile [64 keys][DKP] (per-head part,
+// then the shared rotated part) and V tile [64][DVP] in LDS, NB buffers; the next tile's global
+// loads are in flight during this tile's MFMAs.  S^T = K Q^T, so its accumulators are the P^T
+// operand of O^T = V^T P^T without lane movement.  QF = 2 halves the LDS reads per MFMA; NB = 1
+// then leaves room for a second workgroup per CU, whose MFMAs run under this one's softmax.
 constexpr int kLK = 64;
 
-template <int DKP, int DVP>
+template <int DKP, int DVP, int NB>
 struct LatLds {
   static constexpr int KROW = DKP + 8;
   static constexpr int VROW = DVP + 16;
   static constexpr int K_ELEMS = kLK * KROW;
   static constexpr int BUF = K_ELEMS + kLK * VROW;
-  static constexpr size_t BYTES = (size_t)2 * BUF * 2;
+  static constexpr size_t BYTES = (size_t)NB * BUF * 2;
 };
 
-template <int DKP, int DVP, int QF>
-__global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a) {
-  using L = LatLds<DKP, DVP>;
+template <int DKP, int DVP, int QF, int NW, int NB>
+__global__ __launch_bounds__(64 * NW, NB == 1 ? 2 : 1) void latent_prefill_kernel(
+    LatentPrefillArgs a) {
+  using L = LatLds<DKP, DVP, NB>;
+  constexpr int NTHR = 64 * NW;
   constexpr int KS = DKP / 32, NT = DVP / 16;
-  constexpr int NK = kLK * (DKP / 8) / 256, NV = kLK * (DVP / 8) / 256;
-  constexpr int QT = 64 * QF;
+  constexpr int NK = kLK * (DKP / 8) / NTHR, NV = kLK * (DVP / 8) / NTHR;
+  constexpr int QT = 16 * NW * QF;
+  static_assert(NK * NTHR == kLK * (DKP / 8) && NV * NTHR == kLK * (DVP / 8), "staging split");
   extern __shared__ __attribute__((aligned(16))) bf16_t lat_lds[];
 
   const int seq = a.tile_seq[blockIdx.x], q0 = a.tile_q0[blockIdx.x], h = blockIdx.y;
@@ -253,7 +319,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a
   auto issue = [&](int k0) {
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const int v = threadIdx.x + i * 256;
+      const int v = threadIdx.x + i * NTHR;
       const int key = v / (DKP / 8), c = (v % (DKP / 8)) * 8;
       bf16x8 x = zero8();
       if (k0 + key < k_hi) {
@@ -264,7 +330,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int v = threadIdx.x + i * 256;
+      const int v = threadIdx.x + i * NTHR;
       const int key = v / (DVP / 8), c = (v % (DVP / 8)) * 8;
       bf16x8 x = zero8();
       if (k0 + key < k_hi && c < a.vdim)
@@ -275,12 +341,12 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a
   auto commit = [&](bf16_t* kb) {
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const int v = threadIdx.x + i * 256;
+      const int v = threadIdx.x + i * NTHR;
       store_bf16x8(kb + (v / (DKP / 8)) * L::KROW + (v % (DKP / 8)) * 8, kr[i]);
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int v = threadIdx.x + i * 256;
+      const int v = threadIdx.x + i * NTHR;
       store_bf16x8(kb + L::K_ELEMS + (v / (DVP / 8)) * L::VROW + (v % (DVP / 8)) * 8, vr[i]);
     }
   };
@@ -299,7 +365,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a
     }
   }
   f32x4 o[QF][NT];
-  float m[QF], lsum[QF];
+  float m[QF], lsum[QF];  // m: running maximum of the unscaled scores
 #pragma unroll
   for (int f = 0; f < QF; ++f) {
     m[f] = kNegBig;
@@ -314,7 +380,8 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a
   for (int kt = t_lo; kt < t_hi; ++kt) {
     bf16_t* kb = lat_lds + buf * L::BUF;
     const bf16_t* vb = kb + L::K_ELEMS;
-    buf ^= 1;
+    if constexpr (NB == 1) __syncthreads();
+    else buf ^= 1;
     commit(kb);
     __syncthreads();
     if (kt + 1 < t_hi) issue((kt + 1) * kLK);
@@ -336,45 +403,59 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a
         for (int f = 0; f < QF; ++f) sc[f][st] = mfma16(kf, qf[f][s], sc[f][st]);
       }
     }
+    if (!whole) {
+#pragma unroll
+      for (int f = 0; f < QF; ++f) {
+        const int qpos = ctx + qw + 16 * f + col;
+#pragma unroll
+        for (int st = 0; st < 4; ++st)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int key = k0 + 16 * st + 4 * g + r;
+            if (key > qpos || key <= qpos - win) sc[f][st][r] = kNegBig;
+          }
+      }
+    }
     bf16x8 pf[QF][2];
     float alpha[QF];
+    bool moved = false;
 #pragma unroll
     for (int f = 0; f < QF; ++f) {
-      const int qpos = ctx + qw + 16 * f + col;
       float bmax = kNegBig;
 #pragma unroll
       for (int st = 0; st < 4; ++st)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int key = k0 + 16 * st + 4 * g + r;
-          const bool ok = whole || (key <= qpos && key > qpos - win);
-          sc[f][st][r] = ok ? sc[f][st][r] * sl2 : kNegBig;
-          bmax = fmaxf(bmax, sc[f][st][r]);
-        }
+        for (int r = 0; r < 4; ++r) bmax = fmaxf(bmax, sc[f][st][r]);
       bmax = fmaxf(bmax, __shfl_xor(bmax, 16, 64));
       bmax = fmaxf(bmax, __shfl_xor(bmax, 32, 64));
       const float m_new = fmaxf(m[f], bmax);
-      alpha[f] = fast_exp2(m[f] - m_new);
+      alpha[f] = fast_exp2((m[f] - m_new) * sl2);
+      moved |= m_new > m[f];
       m[f] = m_new;
-      // a row with no key in any tile so far keeps m = kNegBig and p = 1 here; the first
-      // tile with one of its keys scales that away (alpha = 0)
+      // a row with no key in any tile so far: offset 0, so that its p are 0 (kNegBig minus a
+      // rounded product of itself would not be)
+      const float off = m_new > 0.5f * kNegBig ? m_new * sl2 : 0.f;
       float psum = 0.f;
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float pa = fast_exp2(sc[f][2 * ks][r] - m_new);
-          const float pb = fast_exp2(sc[f][2 * ks + 1][r] - m_new);
+          const float pa = fast_exp2(sc[f][2 * ks][r] * sl2 - off);
+          const float pb = fast_exp2(sc[f][2 * ks + 1][r] * sl2 - off);
           psum += pa + pb;
           pf[f][ks][r] = f2bf(pa);
           pf[f][ks][4 + r] = f2bf(pb);
         }
       lsum[f] = lsum[f] * alpha[f] + psum;
     }
+    if (__any(moved)) {
+#pragma unroll
+      for (int f = 0; f < QF; ++f)
+#pragma unroll
+        for (int i = 0; i < NT; ++i) o[f][i] *= alpha[f];
+    }
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
-#pragma unroll
-      for (int f = 0; f < QF; ++f) o[f][i] *= alpha[f];
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
         const bf16x4 lo = lat_read_tr16(vb + tr_off + 32 * ks * L::VROW + 16 * i);
@@ -392,7 +473,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a
     float l = lsum[f];
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
-    if (a.sink) l += fast_exp2(a.sink[h] * kLog2e - m[f]);
+    if (a.sink) l += fast_exp2(a.sink[h] * kLog2e - m[f] * sl2);
     const int qr = qw + 16 * f + col;
     if (qr < n) {
       const float inv = 1.f / l;
@@ -411,19 +492,19 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(LatentPrefillArgs a
   }
 }
 
-template <int DKP, int DVP, int QF>
-static void lat_prefill_go(const LatentPrefillArgs& a, hipStream_t st) {
-  latent_prefill_kernel<DKP, DVP, QF><<<dim3(a.ntiles, a.H), dim3(256), LatLds<DKP, DVP>::BYTES,
-                                         st>>>(a);
+template <int DKP, int DVP, int QF, int NW, int NB>
+static int lat_prefill_go(const LatentPrefillArgs& a, hipStream_t st) {
+  latent_prefill_kernel<DKP, DVP, QF, NW, NB>
+      <<<dim3(a.ntiles, a.H), dim3(64 * NW), LatLds<DKP, DVP, NB>::BYTES, st>>>(a);
+  return 0;
 }
 template <int DKP, int DVP>
 static int lat_prefill_q(const LatentPrefillArgs& a, hipStream_t st) {
   if constexpr (DKP <= 192 && DVP <= 128) {
-    if (a.qtile == 128) { lat_prefill_go<DKP, DVP, 2>(a, st); return 0; }
+    if (a.qtile == 256) return lat_prefill_go<DKP, DVP, 2, 8, 2>(a, st);
+    if (a.qtile == 128) return lat_prefill_go<DKP, DVP, 2, 4, 1>(a, st);
   }
-  if (a.qtile != 64) return -1;
-  lat_prefill_go<DKP, DVP, 1>(a, st);
-  return 0;
+  return a.qtile == 64 ? lat_prefill_go<DKP, DVP, 1, 4, 2>(a, st) : -1;
 }
 template <int DKP>
 static int lat_prefill_v(const LatentPrefillArgs& a, hipStream_t st) {
@@ -456,11 +537,15 @@ int launch_latent_prefill(int f32, const LatentPrefillArgs& a, hipStream_t st) {
 // Workgroup: NH head tiles of 16 x ND slices of the output dims, one wave each; grid
 // (sequence, group of 16 NH heads, split of the window).  Every wave of a head tile computes
 // the tile's scores (they are cheap beside the block's HBM time) and accumulates its slice of
-// O^T = C^T P^T.  RT: the latent size in units of 64 (rounded up to 1, 2, 4, 8).
-template <int RT, int NH, int ND>
-__global__ __launch_bounds__(64 * NH * ND) void latent_decode_kernel(LatentDecodeArgs a) {
+// O^T = C^T P^T.  RT: the latent size in units of 64 (rounded up to 1, 2, 4, 8).  KSX: the
+// exact number of 32-column steps of a cache row with R = 64 RT (branch-free products, loads
+// batched ahead of them); 0: both at run time.
+constexpr int kLatPad = 8;  // row padding: 16 rows of one b128 column start on distinct banks
+
+template <int RT, int NH, int ND, int KSX>
+__global__ __launch_bounds__(64 * NH * ND, 2) void latent_decode_kernel(LatentDecodeArgs a) {
   constexpr int NTHR = 64 * NH * ND;
-  constexpr int KSM = 2 * RT + 2;             // 32-column steps of a cache row, at most
+  constexpr int KSM = KSX ? KSX : 2 * RT + 2;  // 32-column steps of a cache row, at most
   constexpr int NTW = 4 * RT / ND;            // output tiles of 16 dims per wave
   constexpr int NVM = (4 * 32 * KSM + NTHR - 1) / NTHR;
   extern __shared__ __attribute__((aligned(16))) bf16_t lat_lds[];
@@ -469,7 +554,7 @@ __global__ __launch_bounds__(64 * NH * ND) void latent_decode_kernel(LatentDecod
   const int hw = w / ND, dw = w % ND;
   const int col = lane & 15, g = lane >> 4;
   const int h = (blockIdx.y * NH + hw) * 16 + col;
-  const int LW = a.LW, R = a.R, ks = LW / 32, row_l = LW + 16, tile_l = kLB * row_l;
+  const int LW = KSX ? 32 * KSX : a.LW, R = KSX ? 64 * RT : a.R, ks = LW / 32, row_l = LW + kLatPad, tile_l = kLB * row_l;
   const int ctx = a.context_lens[b];
   if (ctx <= 0) {
     if (sp == 0 && h < a.H)
@@ -529,15 +614,21 @@ __global__ __launch_bounds__(64 * NH * ND) void latent_decode_kernel(LatentDecod
     commit(kb);
     __syncthreads();
     if (t + 1 < te) issue(t + 1);
+    // four chains (token half x step parity) hide the MFMA latency
+    f32x4 part[2][2];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) part[i >> 1][i & 1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < KSM; ++s)
+      if (KSX || s < ks) {
+#pragma unroll
+        for (int h2 = 0; h2 < 2; ++h2)
+          part[h2][s & 1] = mfma16(load_bf16x8(kb + (16 * h2 + col) * row_l + 32 * s + 8 * g),
+                                   qf[s], part[h2][s & 1]);
+      }
     f32x4 sc[2];
 #pragma unroll
-    for (int h2 = 0; h2 < 2; ++h2) {
-      sc[h2] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int s = 0; s < KSM; ++s)
-        if (s < ks)
-          sc[h2] = mfma16(load_bf16x8(kb + (16 * h2 + col) * row_l + 32 * s + 8 * g), qf[s], sc[h2]);
-    }
+    for (int h2 = 0; h2 < 2; ++h2) sc[h2] = part[h2][0] + part[h2][1];
     float bmax = kNegBig;
 #pragma unroll
     for (int h2 = 0; h2 < 2; ++h2)
@@ -551,6 +642,7 @@ __global__ __launch_bounds__(64 * NH * ND) void latent_decode_kernel(LatentDecod
     bmax = fmaxf(bmax, __shfl_xor(bmax, 32, 64));
     const float m_new = fmaxf(m, bmax);  // every tile of a split holds a visible token
     const float alpha = fast_exp2(m - m_new);
+    const bool moved = __any(m_new > m);
     m = m_new;
     bf16x8 pf;
     float psum = 0.f;
@@ -562,15 +654,18 @@ __global__ __launch_bounds__(64 * NH * ND) void latent_decode_kernel(LatentDecod
       pf[4 + r] = f2bf(pb);
     }
     lsum = lsum * alpha + psum;
+    if (moved) {
+#pragma unroll
+      for (int i = 0; i < NTW; ++i) o[i] *= alpha;
+    }
 #pragma unroll
     for (int i = 0; i < NTW; ++i) {
-      if (16 * (NTW * dw + i) < R) {
+      if (KSX || 16 * (NTW * dw + i) < R) {
         const bf16x4 x = lat_read_tr16(kb + tr_off + 16 * i);
         const bf16x4 y = lat_read_tr16(kb + tr_off + 16 * row_l + 16 * i);
         bf16x8 vf;
 #pragma unroll
         for (int j = 0; j < 4; ++j) { vf[j] = x[j]; vf[4 + j] = y[j]; }
-        o[i] *= alpha;
         o[i] = mfma16(vf, pf, o[i]);
       }
     }
@@ -636,9 +731,19 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(LatentDecodeArgs a) {
 
 template <int RT, int NH, int ND>
 static void lat_decode_go(const LatentDecodeArgs& a, hipStream_t st) {
-  const size_t lds = (size_t)2 * kLB * (a.LW + 16) * 2;
-  latent_decode_kernel<RT, NH, ND>
-      <<<dim3(a.B, (a.H + 16 * NH - 1) / (16 * NH), a.nsplits), dim3(64 * NH * ND), lds, st>>>(a);
+  const size_t lds = (size_t)2 * kLB * (a.LW + kLatPad) * 2;
+  const dim3 grid(a.B, (a.H + 16 * NH - 1) / (16 * NH), a.nsplits), block(64 * NH * ND);
+  if constexpr (RT >= 4) {
+    if (a.R == 64 * RT && a.LW == 32 * (2 * RT + 2)) {
+      latent_decode_kernel<RT, NH, ND, 2 * RT + 2><<<grid, block, lds, st>>>(a);
+      return;
+    }
+    if (a.R == 64 * RT && a.LW == 32 * (2 * RT + 1)) {
+      latent_decode_kernel<RT, NH, ND, 2 * RT + 1><<<grid, block, lds, st>>>(a);
+      return;
+    }
+  }
+  latent_decode_kernel<RT, NH, ND, 0><<<grid, block, lds, st>>>(a);
 }
 template <int RT>
 static void lat_decode_h(const LatentDecodeArgs& a, hipStream_t st) {
@@ -669,40 +774,67 @@ int launch_latent_decode(int f32, const LatentDecodeArgs& a, hipStream_t st) {
 // y[b, h, :] = W[h] x[b, h, :], W [H, N, K].  MFMA: 16 output dims per wave, 64 batch rows per
 // workgroup sharing each weight fragment; operands straight from global memory (the weights
 // are read once per 64 rows and stay in L2).
+// WHOLE: K % 128 == 0 - four steps' loads ahead of their products.
+template <int NBT, bool WHOLE>
 __global__ __launch_bounds__(256) void head_gemm_kernel(
     bf16_t* __restrict__ y, const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, int B,
     int N, int K, int64_t yb, int64_t yh, int64_t xb, int64_t xh) {
-  const int h = blockIdx.z, b0 = blockIdx.y * 64;
+  const int h = blockIdx.z, b0 = blockIdx.y * 16 * NBT;
   const int wv = wave_id_uniform(), lane = threadIdx.x & 63;
   const int col = lane & 15, g = lane >> 4;
   const int n0 = (blockIdx.x * 4 + wv) * 16;
   if (n0 >= N) return;
   const bf16_t* wr = w + ((int64_t)h * N + min(n0 + col, N - 1)) * K;
-  const int nbt = min(4, (B - b0 + 15) / 16);
-  const bf16_t* xr[4];
+  const bf16_t* xr[NBT];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) xr[i] = x + (int64_t)min(b0 + 16 * i + col, B - 1) * xb + h * xh;
-  f32x4 acc[4];
+  for (int i = 0; i < NBT; ++i) xr[i] = x + (int64_t)min(b0 + 16 * i + col, B - 1) * xb + h * xh;
+  f32x4 acc[NBT];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) acc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  for (int k = 0; k < K; k += 32) {
-    const int c = k + 8 * g;
-    const bool in = c < K;
-    const bf16x8 wf = in ? load_bf16x8(wr + c) : zero8();
+  for (int i = 0; i < NBT; ++i) acc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  if constexpr (WHOLE) {
+    for (int k = 0; k < K; k += 128) {
+      bf16x8 wf[4], xf[4][NBT];
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (i < nbt) acc[i] = mfma16(wf, in ? load_bf16x8(xr[i] + c) : zero8(), acc[i]);
+      for (int s = 0; s < 4; ++s) {
+        wf[s] = load_bf16x8(wr + k + 32 * s + 8 * g);
+#pragma unroll
+        for (int i = 0; i < NBT; ++i) xf[s][i] = load_bf16x8(xr[i] + k + 32 * s + 8 * g);
+      }
+#pragma unroll
+      for (int s = 0; s < 4; ++s)
+#pragma unroll
+        for (int i = 0; i < NBT; ++i) acc[i] = mfma16(wf[s], xf[s][i], acc[i]);
+    }
+  } else {
+    for (int k = 0; k < K; k += 32) {
+      const int c = k + 8 * g;
+      const bool in = c < K;
+      const bf16x8 wf = in ? load_bf16x8(wr + c) : zero8();
+#pragma unroll
+      for (int i = 0; i < NBT; ++i)
+        acc[i] = mfma16(wf, in ? load_bf16x8(xr[i] + c) : zero8(), acc[i]);
+    }
   }
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (int i = 0; i < NBT; ++i) {
     const int b = b0 + 16 * i + col, n = n0 + 4 * g;
-    if (i < nbt && b < B && n < N) {
+    if (b < B && n < N) {
       bf16x4 v;
 #pragma unroll
       for (int r = 0; r < 4; ++r) v[r] = f2bf(acc[i][r]);
       *reinterpret_cast<bf16x4*>(y + b * yb + h * yh + n) = v;
     }
   }
+}
+
+template <int NBT>
+static void head_gemm_go(bf16_t* y, const bf16_t* x, const bf16_t* w, int B, int H, int N, int K,
+                         int64_t yb, int64_t yh, int64_t xb, int64_t xh, hipStream_t st) {
+  const dim3 grid((N + 63) / 64, (B + 16 * NBT - 1) / (16 * NBT), H);
+  if (K % 128 == 0)
+    head_gemm_kernel<NBT, true><<<grid, dim3(256), 0, st>>>(y, x, w, B, N, K, yb, yh, xb, xh);
+  else
+    head_gemm_kernel<NBT, false><<<grid, dim3(256), 0, st>>>(y, x, w, B, N, K, yb, yh, xb, xh);
 }
 
 template <class T>
@@ -723,8 +855,10 @@ int launch_head_gemm(int f32, void* y, const void* x, const void* w, int B, int 
   if (B == 0) return 0;
   if (!f32 && K % 8 == 0 && N % 4 == 0 && yb % 4 == 0 && yh % 4 == 0 && xb % 8 == 0 &&
       xh % 8 == 0) {
-    head_gemm_kernel<<<dim3((N + 63) / 64, (B + 63) / 64, H), dim3(256), 0, st>>>(
-        (bf16_t*)y, (const bf16_t*)x, (const bf16_t*)w, B, N, K, yb, yh, xb, xh);
+    const bf16_t *xx = (const bf16_t*)x, *ww = (const bf16_t*)w;
+    if (B <= 16) head_gemm_go<1>((bf16_t*)y, xx, ww, B, H, N, K, yb, yh, xb, xh, st);
+    else if (B <= 32) head_gemm_go<2>((bf16_t*)y, xx, ww, B, H, N, K, yb, yh, xb, xh, st);
+    else head_gemm_go<4>((bf16_t*)y, xx, ww, B, H, N, K, yb, yh, xb, xh, st);
   } else {
     const dim3 grid(B, H, (N + 255) / 256);
     if (f32)
@@ -738,16 +872,18 @@ int launch_head_gemm(int f32, void* y, const void* x, const void* w, int B, int 
 }
 
 // dynamic LDS above 64 KB
+template <int DKP, int DVP, int QF, int NW, int NB>
+static int lat_prefill_attr() {
+  return (int)hipFuncSetAttribute((const void*)latent_prefill_kernel<DKP, DVP, QF, NW, NB>,
+                                  hipFuncAttributeMaxDynamicSharedMemorySize,
+                                  (int)LatLds<DKP, DVP, NB>::BYTES);
+}
 template <int DKP, int DVP>
 static int lat_prefill_lds() {
-  int e = (int)hipFuncSetAttribute((const void*)latent_prefill_kernel<DKP, DVP, 1>,
-                                   hipFuncAttributeMaxDynamicSharedMemorySize,
-                                   (int)LatLds<DKP, DVP>::BYTES);
+  int e = lat_prefill_attr<DKP, DVP, 1, 4, 2>();
   if constexpr (DKP <= 192 && DVP <= 128) {
-    if (!e)
-      e = (int)hipFuncSetAttribute((const void*)latent_prefill_kernel<DKP, DVP, 2>,
-                                   hipFuncAttributeMaxDynamicSharedMemorySize,
-                                   (int)LatLds<DKP, DVP>::BYTES);
+    if (!e) e = lat_prefill_attr<DKP, DVP, 2, 8, 2>();
+    if (!e) e = lat_prefill_attr<DKP, DVP, 2, 4, 1>();
   }
   return e;
 }
@@ -758,11 +894,18 @@ static int lat_prefill_lds_v() {
   if (!e) e = lat_prefill_lds<DKP, 256>();
   return e;
 }
+template <int NH, int ND, int KSX>
+static int lat_decode_attr() {
+  return (int)hipFuncSetAttribute((const void*)latent_decode_kernel<8, NH, ND, KSX>,
+                                  hipFuncAttributeMaxDynamicSharedMemorySize,
+                                  2 * kLB * (18 * 32 + kLatPad) * 2);
+}
 template <int NH, int ND>
 static int lat_decode_lds() {
-  return (int)hipFuncSetAttribute((const void*)latent_decode_kernel<8, NH, ND>,
-                                  hipFuncAttributeMaxDynamicSharedMemorySize,
-                                  2 * kLB * (18 * 32 + 16) * 2);
+  int e = lat_decode_attr<NH, ND, 0>();
+  if (!e) e = lat_decode_attr<NH, ND, 17>();
+  if (!e) e = lat_decode_attr<NH, ND, 18>();
+  return e;
 }
 int configure_latent() {
   int e = lat_prefill_lds_v<64>();

@@ -46,6 +46,12 @@ DRTC_DEVICE float quad_sum(float v) {
   v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xF, 0xF, true));
   return v;
 }
+// Sum over aligned groups of 8 lanes: the quad, then its mirror image in the half row.
+DRTC_DEVICE float sum8(float v) {
+  v = quad_sum(v);
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x141, 0xF, 0xF, true));
+  return v;
+}
 // Sum over aligned groups of 16 lanes.
 DRTC_DEVICE float sum16(float v) {
 #pragma unroll

@@ -138,6 +138,8 @@ class LatentAttention:
     def __post_init__(self):
         if self.rot_dims % 2 or self.rot_dims > self.rot_dim:
             raise ValueError(f"rotated dims {self.rot_dims} of a {self.rot_dim}-wide part")
+        if not self.scale > 0:
+            raise ValueError("scores need a positive scale")
         if self.window is not None and self.window < 1:
             raise ValueError("a window holds at least the token itself")
         if self.kv_rank > 1024 or self.vdim > 1024:

@@ -123,19 +123,14 @@ def _token_ref(w: DeltaWeights, x, beta_in, decay, gate, S):
     return (o * torch.sigmoid(gate.float()).view(w.heads, w.vdim)).flatten()
 
 
-def scan_columns_per_lane(portions: int, heads: int, vdim: int) -> int:
-    """State columns a lane of the scan holds: 1 gives the shortest token-to-token path, 4 the
-    fewest LDS reads per state element - worth it once the portions alone fill the chip."""
-    waves = portions * heads * -(-vdim // 16)
-    return 1 if waves <= 2048 else 2 if waves <= 8192 else 4
-
-
 def delta_scan(proj: torch.Tensor, off_b: int, conv: torch.Tensor, w: DeltaWeights,
                ring: torch.Tensor, state: torch.Tensor, decay: torch.Tensor, gate: torch.Tensor,
-               p: Portions, columns: int | None = None) -> torch.Tensor:
+               p: Portions, columns: int = 0) -> torch.Tensor:
     """The recurrence over packed portions, each continuing its slot's state (from zero at
     position 0), then output norm and gate -> [rows, heads * vdim].  Leaves the state and the
-    ring as of each portion's last token.  Rows in no portion are not written."""
+    ring as of each portion's last token.  Rows in no portion are not written.  ``columns`` 0:
+    chunks of 8 tokens on the fp32 MFMA where the sizes allow it; 2 / 4: token by token, with
+    that many state columns to a lane."""
     rows = p.row_state.numel()
     out = torch.empty((rows, w.heads * w.vdim), dtype=proj.dtype, device=proj.device)
     if not on_gpu(proj):
@@ -161,8 +156,7 @@ def delta_scan(proj: torch.Tensor, off_b: int, conv: torch.Tensor, w: DeltaWeigh
     a.update(conv=conv.data_ptr(), seg_row=p.seg_row.data_ptr(), seg_len=p.seg_len.data_ptr(),
              seg_pos=p.seg_pos.data_ptr(), seg_state=p.seg_state.data_ptr(), nseg=n)
     check(hipk().delta_scan(int(proj.dtype == torch.float32), a,
-                            columns or scan_columns_per_lane(n, w.heads, w.vdim),
-                            stream_ptr(proj)), "delta_scan")
+                            columns, stream_ptr(proj)), "delta_scan")
     return out
 
 

@@ -126,9 +126,14 @@ def window_reach(start: int, window: int | None) -> int:
 
 
 def latent_qtile(max_len: int, dim: int, rot_dim: int, vdim: int) -> int:
-    """Query rows per workgroup: two 16-row fragments a wave where the sizes leave registers
-    for them and the portions are long enough to fill the tiles."""
-    return 128 if max_len > 256 and dim + rot_dim <= 192 and vdim <= 128 else 64
+    """Query rows per workgroup (64: one 16-row fragment a wave; 128 / 256: two, where the sizes
+    leave registers for them), by the longest portion."""
+    if dim + rot_dim > 192 or vdim > 128 or max_len <= 64:
+        return 64
+    return 128 if max_len < QTILE_256_MIN else 256
+
+
+QTILE_256_MIN = 192
 
 
 def portion_tiles(cu: list[int], qtile: int) -> tuple[list[int], list[int]]:
@@ -203,7 +208,7 @@ def _latent_prefill_ref(q, kv, voff, lat, kv_rank, heads, dim, rot_dim, vdim, q_
 
 # ------------------------------------------------------------------ decode rows
 def latent_decode_splits(batch: int, heads: int, window: int | None, max_blocks: int,
-                         target_wgs: int = 1024) -> tuple[int, int]:
+                         target_wgs: int = 256) -> tuple[int, int]:
     """(cache blocks per split, splits): static, so that a decode step can be captured.  Splits
     fill the chip when the batch alone does not; at least 4 blocks each."""
     blocks = max_blocks if window is None else min(max_blocks, (window + KV_BLOCK - 2) // KV_BLOCK + 1)

@@ -195,12 +195,13 @@ def test_latent_decode_attention(target, H, R, rot):
             if j >= 0:
                 row = c2[bt[b, j // 32], j % 32]
                 row[:R + rot] = (q2[b, 0, :R + rot].float() * 4).to(dt)
-        for parts in (1024, 1):
+        for parts in (4, 1):
             ws = None
             if dev == "cuda":
                 ws = ops.LatentDecodeWorkspace(B, H, R, window, nb, dev)
-                if parts == 1:
-                    ws.per, ws.splits = nb, 1
+                ws.per, ws.splits = -(-nb // parts), parts
+                ws.part_o = torch.empty(B, H, parts, R, device=dev)
+                ws.part_ml = torch.empty(B, H, parts, 2, device=dev)
             out = ops.latent_decode_attention(q2.to(dev), c2.to(dev), R, bt.to(dev),
                                               torch.tensor(ctx, dtype=torch.int32, device=dev),
                                               window, 0.11, sink.to(dev), ws)
@@ -274,7 +275,7 @@ DELTA_SHAPES = [(4, 2, 16, 24, 3), (2, 2, 128, 128, 4), (3, 1, 72, 136, 2), (2, 
 
 @on
 @pytest.mark.parametrize("shape", DELTA_SHAPES, ids=str)
-@pytest.mark.parametrize("columns", [1, 2, 4])
+@pytest.mark.parametrize("columns", [0, 2, 4])
 def test_delta_rule(target, shape, columns):
     """Packed whole sequences, then the same cut into portions and single decoded tokens, in
     state slots that hold another sequence's leftovers."""
