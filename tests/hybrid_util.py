@@ -37,6 +37,8 @@ CONFIGS = {
     # large latents and heads, more heads than a decode workgroup, long rows of state
     "large": config(128, 256, latent(70, 64, 64, 128, 448, 90), delta(2, 1, 160, 300, 1),
                     latent(17, 128, 64, 136, 512, 64), delta(2, 2, 128, 128, 4)),
+    # projections wide enough for the prefill GEMM tiles
+    "tiles": config(256, 256, latent(16, 64, 64, 64, 192, 300, ff=512), delta(12, 12, 64, 64, 4, ff=256)),
     # windows of one and two tokens, a window larger than any prompt
     "narrow": config(96, 64, latent(2, 16, 8, 16, 32, 1), latent(2, 16, 8, 16, 32, 2),
                      delta(1, 1, 8, 8, 2), latent(2, 32, 32, 64, 40, 5000, ff=64)),

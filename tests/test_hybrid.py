@@ -510,6 +510,28 @@ def test_long_decoding(target):
     agree(feed_all(engine("mixed", target), toks, [start, 1]), expected("mixed", toks), target[1])
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", [F32, BF16], ids=["f32", "bf16"])
+def test_prefill_sized_steps(dtype):
+    """Steps of more than a thousand rows (the prefill GEMMs, 256-row query tiles, portions far
+    into a prompt) beside decode rows."""
+    cfg, _ = case("tiles")
+    a, b, c = (tokens(cfg, n, n) for n in (1500, 1210, 40))
+    ea, eb, ec = (expected("tiles", t) for t in (a, b, c))
+    eng = engine("tiles", ("cuda", dtype), max_len=1536)
+    ra, rb, rc = Request([]), Request([]), Request([])
+    got = eng.feed([(ra, a[:700], list(range(700))), (rb, b[:520], list(range(520))), (rc, c[:39], [38])])
+    agree(got[0], ea[:700], dtype)
+    agree(got[1], eb[:520], dtype)
+    got = eng.feed([(rc, c[39:], [0]), (rb, b[520:1200], list(range(680))), (ra, a[700:1400], list(range(700)))])
+    agree(got[0], ec[39:], dtype)
+    agree(got[1], eb[520:1200], dtype)
+    agree(got[2], ea[700:1400], dtype)
+    got = [eng.feed([(ra, [a[1400 + i]], [0]), (rb, [b[1200 + i]], [0])]) for i in range(10)]
+    agree(torch.cat([g[0] for g in got]), ea[1400:1410], dtype)
+    agree(torch.cat([g[1] for g in got]), eb[1200:], dtype)
+
+
 def _mutations():
     def layers(f):
         return lambda c, w: ({**c, "layers": [f(json.loads(json.dumps(l))) for l in c["layers"]]}, w)
