@@ -707,6 +707,23 @@ def test_registered_preset_serves(target):
     assert abs(RALESUN_2B.num_params() / 2.9e9 - 1) < 0.3
 
 
+def test_service_backend_from_checkpoint_folder(tmp_path):
+    """The LLM service's --model takes a checkpoint folder; text in, text out."""
+    from argparse import Namespace
+
+    from drtc_amd.llm.server import build_backend
+
+    cfg, w = case("mixed")
+    path = save_checkpoint(tmp_path / "m", cfg, w)
+    backend = build_backend(Namespace(backend="engine", model=path, max_batch=2, max_model_len=128,
+                                      no_graphs=True, tp=1, gpus=1, in_process=True))
+    try:
+        out = backend.generate(["hello there", "ok"], SamplingParams.greedy(5, ignore_eos=True))
+        assert len(out) == 2 and all(isinstance(t, str) for t in out)
+    finally:
+        backend.close()
+
+
 def test_limits_are_errors():
     eng = engine("mixed", ("cpu", F32), max_len=64)
     r = Request([])
