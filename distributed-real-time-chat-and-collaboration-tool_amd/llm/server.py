@@ -297,14 +297,16 @@ def _stop_once(stop: threading.Event) -> None:
     """SIGTERM: start the ordered shutdown; further SIGTERMs are ignored (CPython restores
     the default - terminate - action for Python-level handlers during finalization, so a
     repeated SIGTERM from a supervisor would otherwise kill the exiting process)."""
-    stop.set()
     signal.signal(signal.SIGTERM, signal.SIG_IGN)
+    # set from a thread: this handler may interrupt the main thread inside stop.wait() or a
+    # first handler's set(), which hold the event's (non-reentrant) lock
+    threading.Thread(target=stop.set, daemon=True).start()
 
 
 def main(argv=None):
     # installed first: a SIGTERM while the engines load still ends the service in order
     stop = threading.Event()
-    signal.signal(signal.SIGINT, lambda *a: stop.set())
+    signal.signal(signal.SIGINT, lambda *a: threading.Thread(target=stop.set, daemon=True).start())
     signal.signal(signal.SIGTERM, lambda *a: _stop_once(stop))
     ap = argparse.ArgumentParser(description="drtc_amd LLM service (on-GPU inference)")
     ap.add_argument("--port", type=int, default=50055)

@@ -79,7 +79,7 @@ def serve(cfg: NodeConfig, block: bool = True, bind: str = "[::]",
 
 def _install_stop_handlers() -> threading.Event:
     stop = threading.Event()
-    signal.signal(signal.SIGINT, lambda *a: stop.set())
+    signal.signal(signal.SIGINT, lambda *a: threading.Thread(target=stop.set, daemon=True).start())
     signal.signal(signal.SIGTERM, lambda *a: _stop_once(stop))
     return stop
 
@@ -88,8 +88,10 @@ def _stop_once(stop: threading.Event) -> None:
     """SIGTERM: start the ordered shutdown; further SIGTERMs are ignored (CPython restores
     the default - terminate - action for Python-level handlers during finalization, so a
     repeated SIGTERM from a supervisor would otherwise kill the exiting process)."""
-    stop.set()
     signal.signal(signal.SIGTERM, signal.SIG_IGN)
+    # set from a thread: this handler may interrupt the main thread inside stop.wait() or a
+    # first handler's set(), which hold the event's (non-reentrant) lock
+    threading.Thread(target=stop.set, daemon=True).start()
 
 
 def main(argv=None) -> None:

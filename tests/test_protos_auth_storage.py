@@ -17,7 +17,7 @@ from drtc_amd.raft.storage import NativeStorage, PickleStorage
 from drtc_amd.utils import auth, pickle_compat
 
 REF = "/root/reference"
-have_ref = pytest.mark.skipif(not os.path.isdir(REF), reason="reference checkout not mounted")
+have_ref = pytest.mark.skipif(not os.path.isdir(f"{REF}/generated"), reason="reference checkout not mounted")
 
 
 def _ref_fdp(name):
