@@ -91,8 +91,9 @@ PYBIND11_MODULE(_hipk, m) {
                   int k, int e_off, int e_local, int act, u64 ws, int64_t ws_bytes, int variant,
                   int gu_form, int dn_form, u64 slab, int64_t slab_bytes, u64 counters,
                   int n_counters, int logit_ts, int logit_es, int f32, int logits_f32, int groups,
-                  int keep, float limit, u64 st) {
-    const drtc::MoeOptions opt{f32, logits_f32, groups, keep, limit};
+                  int keep, float limit, u64 stream, u64 y, int ldy, int W, u64 st) {
+    const drtc::MoeOptions opt{f32, logits_f32, groups, keep, limit, P<float>(stream),
+                               P<const void>(y), ldy, W};
     return drtc::launch_moe(P<void>(out), P<const void>(x), P<const void>(logits),
                             P<const void>(w_gu), P<const void>(w_dn), T, H, I, E, k, e_off,
                             e_local, act, P<void>(ws), ws_bytes, variant, gu_form, dn_form,

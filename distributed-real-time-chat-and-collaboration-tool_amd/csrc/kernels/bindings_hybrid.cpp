@@ -47,9 +47,41 @@ drtc::GroupedAttnArgs grouped_args(const py::dict& d) {
   return a;
 }
 
+drtc::MemoryArgs memory_args(const py::dict& d) {
+  const Fields f{d};
+  drtc::MemoryArgs a{};
+  PTR(proj); VAL(ldp); VAL(off_k); VAL(off_v); VAL(off_g); VAL(off_i); VAL(off_f); VAL(H); VAL(dim);
+  VAL(vdim); VAL(q_scale); VAL(k_scale); PTR(cos_sin); VAL(rot_dims); PTR(log_decay); PTR(i_bias);
+  PTR(f_bias); VAL(cap); PTR(norm_w); VAL(silu); VAL(eps); PTR(state); PTR(nrm); PTR(top);
+  VAL(slices); PTR(out); VAL(ldo); PTR(seg_row); PTR(seg_len); PTR(seg_pos); PTR(seg_state);
+  VAL(nseg); PTR(positions); PTR(row_state); VAL(rows);
+  return a;
+}
+
 }  // namespace
 
 void bind_hybrid(py::module_& m) {
+  m.def("memory_scan", [](int f32, const py::dict& d, int plain, u64 st) {
+    return drtc::launch_memory_scan(f32, memory_args(d), plain, S(st));
+  });
+  m.def("memory_decode", [](int f32, const py::dict& d, u64 st) {
+    return drtc::launch_memory_decode(f32, memory_args(d), S(st));
+  });
+  m.def("side_norm", [](int f32, const py::dict& d, u64 st) {
+    const Fields f{d};
+    drtc::SideNormArgs a{};
+    PTR(out); VAL(ldo); PTR(h); PTR(y); VAL(ldy); PTR(yw); PTR(ids); PTR(embed); VAL(embed_scale);
+    PTR(w); VAL(W); VAL(eps); VAL(rows);
+    return drtc::launch_side_norm(f32, a, S(st));
+  });
+  m.def("stream_add", [](int f32, u64 out, u64 h, u64 y, int64_t ldy, int rows, int W, u64 st) {
+    return drtc::launch_stream_add(f32, P<void>(out), P<float>(h), P<void>(y), ldy, rows, W, S(st));
+  });
+  m.def("side_gate", [](int f32, u64 out, u64 z, u64 embed, int64_t lde, int off, u64 ids, int rows,
+                        int dim, u64 st) {
+    return drtc::launch_side_gate(f32, P<void>(out), P<void>(z), P<void>(embed), lde, off,
+                                  P<const int>(ids), rows, dim, S(st));
+  });
   m.def("group_rms", [](int f32, const py::dict& d, u64 st) {
     const Fields f{d};
     drtc::GroupRmsArgs a{};
@@ -102,6 +134,7 @@ void bind_hybrid(py::module_& m) {
     PTR(out); VAL(ldo); PTR(q); VAL(ldq); PTR(kv); VAL(ldkv); VAL(voff); PTR(lat); VAL(LW);
     VAL(R); VAL(H); VAL(dim); VAL(rot); VAL(vdim); PTR(q_cu); PTR(k_cu); PTR(ctx); PTR(tile_seq);
     PTR(tile_q0); VAL(ntiles); VAL(qtile); VAL(nseq); VAL(nq); VAL(window); VAL(scale); PTR(sink);
+    PTR(gate); VAL(ldg);
     return drtc::launch_latent_prefill(f32, a, S(st));
   });
   m.def("latent_decode", [](int f32, const py::dict& d, u64 st) {
@@ -109,7 +142,7 @@ void bind_hybrid(py::module_& m) {
     drtc::LatentDecodeArgs a{};
     PTR(out); PTR(part_o); PTR(part_ml); PTR(qa); PTR(cache); PTR(block_tables); VAL(bt_stride);
     PTR(context_lens); VAL(B); VAL(H); VAL(R); VAL(LW); VAL(window); VAL(tiles_per_split);
-    VAL(nsplits); VAL(scale); PTR(sink);
+    VAL(nsplits); VAL(scale); PTR(sink); PTR(gate); VAL(ldg);
     return drtc::launch_latent_decode(f32, a, S(st));
   });
   m.def("head_gemm", [](int f32, u64 y, u64 x, u64 w, int B, int H, int N, int K, int64_t yb,

@@ -20,6 +20,8 @@ int configure_kernels() {
   if (e) return e;
   e = configure_grouped_decode();
   if (e) return e;
+  e = configure_memory();
+  if (e) return e;
   return configure_gemm_xd();
 }
 }  // namespace drtc

@@ -1008,8 +1008,8 @@ int launch_gemm_w4_grouped(void* c, const void* a, const void* b, const int* grp
                            int epi, int up_off, int group_m, int ksplit, int64_t c_split,
                            float limit, hipStream_t st) {
   const bool glu = epi == W4_SILU || epi == W4_GELU || epi == W4_CLAMP;
-  if (epi != W4_STORE && !glu) return -1;
-  if (ksplit < 1 || (glu && ksplit != 1)) return -1;  // a gated epilogue cannot be split
+  if (epi != W4_STORE && epi != W4_RELU2 && !glu) return -1;
+  if (ksplit < 1 || (epi != W4_STORE && ksplit != 1)) return -1;  // an activation cannot be split
   if (grp == nullptr || n_grp < 1 || max_rows < 1 || K % 64 || (K / 64) % ksplit ||
       K / 64 / ksplit < 2)
     return -1;
@@ -1047,6 +1047,7 @@ int launch_gemm_w4_grouped(void* c, const void* a, const void* b, const int* grp
     case W4_STORE: return w4_launch_grouped<W4_STORE>(p, nwg, st);
     case W4_SILU: return w4_launch_grouped<W4_SILU>(p, nwg, st);
     case W4_CLAMP: return w4_launch_grouped<W4_CLAMP>(p, nwg, st);
+    case W4_RELU2: return w4_launch_grouped<W4_RELU2>(p, nwg, st);
     default: return w4_launch_grouped<W4_GELU>(p, nwg, st);
   }
 }
@@ -1059,6 +1060,7 @@ int64_t gemm_w4_workspace_bytes(int64_t M, int64_t N, int splitk) {
 int configure_gemm_w4() {
   return w4_cfg<W4_STORE>() | w4_cfg<W4_RESIDUAL>() | w4_cfg<W4_SILU>() | w4_cfg<W4_GELU>() |
          w4_cfg_one<W4_RELU2, 0>() | w4_cfg_one<W4_RELU2, 40>() | w4_cfg_one<W4_RELU2, 56>() |
+         w4_cfg_one<W4_RELU2, 104>() | w4_cfg_one<W4_RELU2, 120>() |
          w4_cfg_one<W4_STORE, 104>() | w4_cfg_one<W4_SILU, 104>() | w4_cfg_one<W4_GELU, 104>() |
          w4_cfg_one<W4_CLAMP, 0>() | w4_cfg_one<W4_CLAMP, 40>() | w4_cfg_one<W4_CLAMP, 56>() |
          w4_cfg_one<W4_CLAMP, 104>() | w4_cfg_one<W4_CLAMP, 120>() |

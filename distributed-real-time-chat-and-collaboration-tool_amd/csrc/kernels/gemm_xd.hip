@@ -55,7 +55,7 @@ namespace {
 typedef __attribute__((address_space(3))) void* xd_lds_ptr;
 
 constexpr int kXdThreads = 256;
-enum { XD_STORE = 0, XD_RESIDUAL = 1, XD_SILU = 2, XD_GELU = 3, XD_CLAMP = 4 };
+enum { XD_STORE = 0, XD_RESIDUAL = 1, XD_SILU = 2, XD_GELU = 3, XD_CLAMP = 4, XD_RELU2 = 5 };
 template <int EPI>
 DRTC_DEVICE constexpr bool xd_glu() {
   return EPI == XD_SILU || EPI == XD_GELU || EPI == XD_CLAMP;
@@ -568,9 +568,15 @@ __global__ __launch_bounds__(kXdThreads, 1) void gemm_xd_kernel(XdParams p) {
 #pragma unroll
         for (int jj = 0; jj < JB; ++jj)
 #pragma unroll
-          for (int r = 0; r < 4; ++r)
+          for (int r = 0; r < 4; ++r) {
+            float x = v[jj][r];
+            if constexpr (EPI == XD_RELU2) {
+              x = fmaxf(x, 0.f);
+              x *= x;
+            }
             *reinterpret_cast<bf16_t*>(ep + (16 * i + 4 * g + r) * PITCH +
-                                       (16 * (j0 + jj) + l16) * 2) = f2bf(v[jj][r]);
+                                       (16 * (j0 + jj) + l16) * 2) = f2bf(x);
+          }
       }
     }
   }
@@ -618,7 +624,8 @@ int xd_launch(const XdParams& p, int epi, hipStream_t st) {
   }
 }
 
-// grouped mode: store (expert down projection) and the gated epilogues (expert gate_up)
+// grouped mode: store (expert down projection), the gated epilogues (expert gate_up) and the
+// squared relu (expert up)
 template <class C>
 int xd_launch_g(const XdParams& p, int epi, hipStream_t st) {
   switch (epi) {
@@ -626,6 +633,7 @@ int xd_launch_g(const XdParams& p, int epi, hipStream_t st) {
     case XD_SILU: return xd_launch_e<C, XD_SILU, true>(p, st);
     case XD_GELU: return xd_launch_e<C, XD_GELU, true>(p, st);
     case XD_CLAMP: return xd_launch_e<C, XD_CLAMP, true>(p, st);
+    case XD_RELU2: return xd_launch_e<C, XD_RELU2, true>(p, st);
     default: return -1;
   }
 }
@@ -649,7 +657,8 @@ int xd_cfg_g() {
   for (const void* f : {(const void*)gemm_xd_kernel<C, XD_STORE, true>,
                         (const void*)gemm_xd_kernel<C, XD_SILU, true>,
                         (const void*)gemm_xd_kernel<C, XD_GELU, true>,
-                        (const void*)gemm_xd_kernel<C, XD_CLAMP, true>})
+                        (const void*)gemm_xd_kernel<C, XD_CLAMP, true>,
+                        (const void*)gemm_xd_kernel<C, XD_RELU2, true>})
     e |= (int)hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, C::ALLOC);
   return e;
 }
@@ -792,8 +801,8 @@ int launch_gemm_xd_grouped(void* c, const void* a, const void* b, int a_rows, in
                            int n_counters, float limit, hipStream_t st) {
   const bool nt = (mt & 16) != 0;
   mt &= 15;
-  if (epi < XD_STORE || epi > XD_CLAMP || epi == XD_RESIDUAL) return -1;
-  const bool glu = epi != XD_STORE;
+  if (epi < XD_STORE || epi > XD_RELU2 || epi == XD_RESIDUAL) return -1;
+  const bool glu = epi != XD_STORE && epi != XD_RELU2;
   const int stages = xd_stages(mt, nf);
   if (stages == 0 || splitk < 1 || splitk > 8 || (glu && nf % 2)) return -1;
   if (lda % 8 || ldb % 8 || ldc % 8 || max_tiles < 1 || a_rows < 1) return -1;

@@ -1,7 +1,7 @@
 // Launchers of the kernels of models with mixed layer kinds (models/hybrid.py): Dynamic Tanh,
 // latent attention, gated delta rule; convolved layer norms, talking-heads attention, gated
-// average; norms in groups, grouped attention.  `f32` selects the activation type (0: bf16, 1:
-// fp32).  Same conventions as launchers.h.
+// average; norms in groups, grouped attention; matrix memories, the stream of joint layers.  `f32`
+// selects the activation type (0: bf16, 1: fp32).  Same conventions as launchers.h.
 #pragma once
 #include <hip/hip_runtime.h>
 #include <stdint.h>
@@ -17,7 +17,7 @@ int launch_act_glu_f32(float* out, const float* gu, int64_t T, int I, int gu_str
 
 // ---- latent_attention.hip
 struct LatentPrepArgs {
-  void* proj;             // [rows, ldp]: q heads at column 0 (stride dq), latent at off_kv
+  void* proj;             // [rows, ldp]: q heads at column 0 (stride dq), latent at off_kv (-1: queries only)
   int ldp, off_kv, H, dim, rot, rot_dims, R, LW;
   const float* norm_w;    // [R]
   float eps;
@@ -50,6 +50,8 @@ struct LatentPrefillArgs {
   int ntiles, qtile, nseq, nq, window;   // window 0: no limit
   float scale;
   const float* sink;      // [H] or null
+  const void* gate;       // [rows, ldg] gate inputs per head, or null
+  int ldg;
 };
 int launch_latent_prefill(int f32, const LatentPrefillArgs& a, hipStream_t st);
 
@@ -65,6 +67,8 @@ struct LatentDecodeArgs {
   int B, H, R, LW, window, tiles_per_split, nsplits;
   float scale;
   const float* sink;
+  const void* gate;       // [B, ldg] gate inputs per head, or null
+  int ldg;
 };
 int launch_latent_decode(int f32, const LatentDecodeArgs& a, hipStream_t st);
 int launch_head_gemm(int f32, void* y, const void* x, const void* w, int B, int H, int N, int K,
@@ -303,5 +307,61 @@ int configure_grouped();
 // ---- grouped_decode.hip
 int launch_grouped_decode(const GroupedAttnArgs& a, hipStream_t st);
 int configure_grouped_decode();
+
+// ---- memory_scan.hip
+struct MemoryArgs {
+  const void* proj;       // [rows, ldp]: query heads at column 0, keys, values, read-out gates and
+  int ldp, off_k, off_v, off_g, off_i, off_f;  // (log_decay null) input and forget gates behind
+  int H, dim, vdim;
+  float q_scale, k_scale;  // on queries, on keys (after the rotation)
+  const float* cos_sin;   // [positions, rot_dims]: cos | sin
+  int rot_dims;
+  const float* log_decay;  // [H], or null: gates
+  const float* i_bias;    // [H]
+  const float* f_bias;
+  float cap;
+  const float* norm_w;    // [H * vdim] or null
+  int silu;               // read-out gate: 1 silu, 0 sigmoid
+  float eps;
+  float* state;           // [slots, H, dim, vdim]
+  float* nrm;             // [slots, H, dim] (gates)
+  float* top;             // [slots, H, slices] running maximum (gates)
+  int slices;             // a head's columns are split over this many workgroups
+  void* out;              // [rows, ldo], head h at column h * vdim
+  int ldo;
+  const int* seg_row;     // prefill: one entry per portion
+  const int* seg_len;
+  const int* seg_pos;
+  const int* seg_state;
+  int nseg;
+  const int* positions;   // decode: one entry per row
+  const int* row_state;
+  int rows;
+};
+int launch_memory_scan(int f32, const MemoryArgs& a, int plain, hipStream_t st);
+int launch_memory_decode(int f32, const MemoryArgs& a, hipStream_t st);
+int configure_memory();
+
+// ---- norm_side.hip
+struct SideNormArgs {
+  void* out;              // [rows, ldo], columns beyond W zero
+  int ldo;
+  float* h;               // [rows, W] the residual stream, updated
+  const void* y;          // [rows, ldy] RMS-normed, times yw, added to it; or null
+  int ldy;
+  const float* yw;        // [W]
+  const int* ids;         // [rows]: the stream starts from embed rows times embed_scale instead
+  const void* embed;
+  float embed_scale;
+  const float* w;         // [W]
+  int W;
+  float eps;
+  int rows;
+};
+int launch_side_norm(int f32, const SideNormArgs& a, hipStream_t st);
+int launch_stream_add(int f32, void* out, float* h, const void* y, int64_t ldy, int rows, int W,
+                      hipStream_t st);
+int launch_side_gate(int f32, void* out, const void* z, const void* embed, int64_t lde, int off,
+                     const int* ids, int rows, int dim, hipStream_t st);
 
 }  // namespace drtc

@@ -1,5 +1,5 @@
 // Latent attention (gfx950): per-token key/value latents in a paged cache, a rotated key part
-// shared by all heads, sliding window, softmax sinks.
+// shared by all heads, sliding window, softmax sinks, sigmoid gates per head.
 //
 // Cache row of a token (LW elements, a multiple of 32):  [ latent R | rotated key r | 0 ... ]
 // 32 rows to a block.  A step runs
@@ -29,6 +29,11 @@ DRTC_DEVICE bf16x4 lat_read_tr16(const bf16_t* p) {
   lat_s16x4 v = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
       (__attribute__((address_space(3))) lat_s16x4*)(p));
   return __builtin_bit_cast(bf16x4, v);
+}
+// Factor of a head's output: 1, or the sigmoid of its gate input.
+template <class T>
+DRTC_DEVICE float head_gate(const void* gate, int64_t at) {
+  return gate ? 1.f / (1.f + expf(-to_f32(((const T*)gate)[at]))) : 1.f;
 }
 DRTC_DEVICE bf16x8 zero8() {
   bf16x8 z;
@@ -101,6 +106,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrepArgs a) {
       turn(q, q, (k - h * per) * V);
     }
   }
+  if (a.off_kv < 0) return;  // the latents are another layer's
   const int64_t slot = a.slots ? a.slots[row] : -1;
   T* lat = a.lat ? (T*)a.lat + (int64_t)row * a.LW : nullptr;
   T* cache = a.cache && slot >= 0 ? (T*)a.cache + slot * a.LW : nullptr;
@@ -140,8 +146,8 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrepArgs a) {
 
 template <class T>
 static void lat_prep_t(const LatentPrepArgs& a, hipStream_t st) {
-  if (a.R % 8 == 0 && a.rot % 8 == 0 && a.dim % 8 == 0 && a.ldp % 8 == 0 && a.off_kv % 8 == 0 &&
-      a.LW % 8 == 0)
+  if (a.R % 8 == 0 && a.rot % 8 == 0 && a.dim % 8 == 0 && a.ldp % 8 == 0 &&
+      (a.off_kv < 0 || a.off_kv % 8 == 0) && a.LW % 8 == 0)
     latent_prep_kernel<T, 8><<<dim3(a.rows), dim3(256), 0, st>>>(a);
   else
     latent_prep_kernel<T, 2><<<dim3(a.rows), dim3(256), 0, st>>>(a);
@@ -197,7 +203,8 @@ __global__ __launch_bounds__(256) void latent_prefill_any_kernel(LatentPrefillAr
   const T* q = (const T*)a.q + (int64_t)row * a.ldq + h * (a.dim + a.rot);
   const T* kv = (const T*)a.kv + (int64_t)k0 * a.ldkv;
   const T* lat = (const T*)a.lat + (int64_t)k0 * a.LW + a.R;
-  attend_any<T>(first, last + 1, a.vdim, a.sink != nullptr, a.sink ? a.sink[h] : 0.f, 1.f,
+  attend_any<T>(first, last + 1, a.vdim, a.sink != nullptr, a.sink ? a.sink[h] : 0.f,
+                head_gate<T>(a.gate, (int64_t)row * a.ldg + h),
                 (T*)a.out + (int64_t)row * a.ldo + h * a.vdim,
                 [&](int j) {
                   const T* k = kv + (int64_t)j * a.ldkv + h * a.dim;
@@ -226,7 +233,8 @@ __global__ __launch_bounds__(256) void latent_decode_any_kernel(LatentDecodeArgs
   const T* q = (const T*)a.qa + ((int64_t)b * a.H + h) * a.LW;
   const T* cache = (const T*)a.cache;
   auto row = [&](int j) { return cache + ((int64_t)bt[j / kLB] * kLB + j % kLB) * a.LW; };
-  attend_any<T>(first, ctx, a.R, a.sink != nullptr, a.sink ? a.sink[h] : 0.f, 1.f, out,
+  attend_any<T>(first, ctx, a.R, a.sink != nullptr, a.sink ? a.sink[h] : 0.f,
+                head_gate<T>(a.gate, (int64_t)b * a.ldg + h), out,
                 [&](int j) {
                   const T* k = row(j);
                   float s = 0.f;
@@ -439,7 +447,7 @@ __global__ __launch_bounds__(64 * NW, NB == 1 ? 2 : 1) void latent_prefill_kerne
     if (a.sink) l += fast_exp2(a.sink[h] * kLog2e - m[f] * sl2);
     const int qr = qw + 16 * f + col;
     if (qr < n) {
-      const float inv = 1.f / l;
+      const float inv = head_gate<bf16_t>(a.gate, (int64_t)(qb + qr) * a.ldg + h) / l;
       bf16_t* op = (bf16_t*)a.out + (int64_t)(qb + qr) * a.ldo + h * a.vdim;
 #pragma unroll
       for (int i = 0; i < NT; ++i) {
@@ -638,7 +646,7 @@ __global__ __launch_bounds__(64 * NH * ND, 2) void latent_decode_kernel(LatentDe
   if (h >= a.H) return;
   if (nparts == 1) {
     if (a.sink) lsum += fast_exp2(a.sink[h] * kLog2e - m);
-    const float inv = 1.f / lsum;
+    const float inv = head_gate<bf16_t>(a.gate, (int64_t)b * a.ldg + h) / lsum;
     bf16_t* op = (bf16_t*)a.out + ((int64_t)b * a.H + h) * R;
 #pragma unroll
     for (int i = 0; i < NTW; ++i) {
@@ -679,7 +687,7 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(LatentDecodeArgs a) {
   float l = a.sink ? fast_exp2(a.sink[h] * kLog2e - m) : 0.f;
   for (int p = 0; p < nparts; ++p)
     l += a.part_ml[2 * (pi + p) + 1] * fast_exp2(a.part_ml[2 * (pi + p)] - m);
-  const float inv = 1.f / l;
+  const float inv = head_gate<bf16_t>(a.gate, (int64_t)b * a.ldg + h) / l;
   for (int d = threadIdx.x * 4; d < a.R; d += 512) {
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
     for (int p = 0; p < nparts; ++p)

@@ -57,6 +57,12 @@ struct MoeOptions {
   int groups = 1;      // equal groups of neighbouring experts, of which a token may use `keep`
   int keep = 1;
   float limit = 0.f;   // act 2 (clamped): bound of the gate and up values
+  // a residual stream [T, W <= H] that the result and y [T, ldy] are added to; out is then the
+  // stream in the activation type [T, W] (fp32: unused)
+  float* stream = nullptr;
+  const void* y = nullptr;
+  int ldy = 0;
+  int W = 0;
 };
 // variant 0 / 1 / 2: the moe.hip grouped GEMMs; 3: gemm_xd grouped mode with xd forms gu_form
 // (gated gate_up) / dn_form (down), 0 = by rows per expert; slab / counters: the split-K

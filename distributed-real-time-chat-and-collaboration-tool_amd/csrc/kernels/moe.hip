@@ -11,9 +11,11 @@
 //                         with the gate|up activation fused in the epilogue: a
 //                         wave owns matching gate and up columns, so both MFMA
 //                         accumulators of an output element sit in one lane.
+//                         Experts without a gate: H[p] = relu(X[tok(p)] . Wu[e]^T)^2.
 //   moe_down_kernel       grouped GEMM  Z[p] = H[p] . Wd[e]^T
 //   moe_combine_kernel    out[t] = sum_j w[t,j] * Z[pos(t,j)]   (fp32, fixed order:
-//                         deterministic, no atomics)
+//                         deterministic, no atomics), or the same added to a 32-bit residual
+//                         stream together with another sublayer's output
 //
 // GEMM structure: 256-thread workgroup, 2x2 waves, 128-row tile; operands are
 // K-contiguous rows (activations gathered by token, weights [N][K]) loaded as
@@ -21,6 +23,7 @@
 // loop), 16 MFMA 16x16x32 per wave per k-step.
 #include "common.h"
 #include "launchers.h"
+#include "typed.h"
 
 #include <initializer_list>
 
@@ -305,8 +308,14 @@ __global__ __launch_bounds__(kMoeRouteWG) void moe_scatter_kernel(
 // MODE 0 (gate_up): B rows 0..63 = gate rows n0.., rows 64..127 = the
 //   matching up rows I+n0..; the epilogue writes act(gate) * up, 64 columns.
 // MODE 1 (down): B rows = output columns n0..n0+127.
+// MODE 2 (up without a gate): as MODE 1 over gathered rows; the epilogue writes relu(.)^2.
 typedef __attribute__((address_space(3))) void* lds_ptr_t;
 typedef __attribute__((address_space(1))) void* gbl_ptr_t;
+
+DRTC_DEVICE float relu2(float x) {
+  x = fmaxf(x, 0.f);
+  return x * x;
+}
 
 constexpr int kBK = 64;
 constexpr int kTileElems = 128 * kBK;  // one operand tile (16 KiB)
@@ -347,7 +356,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(
     const int r = 32 * wv + 8 * i + (lane >> 3);
     const int d = (lane & 7) ^ ((r >> 1) & 7);  // source chunk for this LDS slot
     const int rr = r < nr ? r : 0;
-    const int64_t arow = MODE == 0 ? (int64_t)sorted_tok[r0 + rr] : (int64_t)(r0 + rr);
+    const int64_t arow = MODE != 1 ? (int64_t)sorted_tok[r0 + rr] : (int64_t)(r0 + rr);
     asrc[i] = a + arow * K + 8 * d;
     const int wrow = MODE == 0 ? (r < 64 ? n0 + r : I + n0 + r - 64) : n0 + r;
     bsrc[i] = we + (int64_t)wrow * K + 8 * d;
@@ -434,7 +443,8 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(
         }
       } else {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) orow[n0 + 64 * wc + 16 * j + l16] = f2bf(acc[i][j][r]);
+        for (int j = 0; j < 4; ++j)
+          orow[n0 + 64 * wc + 16 * j + l16] = f2bf(MODE == 2 ? relu2(acc[i][j][r]) : acc[i][j][r]);
       }
     }
 }
@@ -495,7 +505,7 @@ __global__ __launch_bounds__(PipeCfg<BM>::NT, 1) void moe_gemm_pipe_kernel(
     const int d = (lane & 7) ^ ((r >> 1) & 7);
     if (r < BM) {
       const int rr = r < nr ? r : 0;
-      const int64_t arow = MODE == 0 ? (int64_t)sorted_tok[r0 + rr] : (int64_t)(r0 + rr);
+      const int64_t arow = MODE != 1 ? (int64_t)sorted_tok[r0 + rr] : (int64_t)(r0 + rr);
       src[i] = a + arow * K + 8 * d;
     } else {
       const int br = r - BM;
@@ -580,14 +590,15 @@ __global__ __launch_bounds__(PipeCfg<BM>::NT, 1) void moe_gemm_pipe_kernel(
         }
       } else {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) orow[n0 + 64 * wc + 16 * j + l16] = f2bf(acc[i][j][r]);
+        for (int j = 0; j < 4; ++j)
+          orow[n0 + 64 * wc + 16 * j + l16] = f2bf(MODE == 2 ? relu2(acc[i][j][r]) : acc[i][j][r]);
       }
     }
 }
 
 // ---------------------------------------------------------------- fp32
 // The same two products for fp32 operands of any size: 128 rows x 64 weight rows per workgroup,
-// 8 x 4 outputs per thread.  MODE 0: 32 gate rows and the 32 matching up rows.
+// 8 x 4 outputs per thread.  MODE 0: 32 gate rows and the 32 matching up rows; 2: up rows only.
 template <int MODE>
 __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
     float* __restrict__ out, const float* __restrict__ a, const float* __restrict__ w,
@@ -610,7 +621,7 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
       const int r = i / BK, c = i % BK;
       float v = 0.f;
       if (r < nr && k0 + c < K) {
-        const int64_t row = MODE == 0 ? sorted_tok[r0 + r] : r0 + r;
+        const int64_t row = MODE != 1 ? sorted_tok[r0 + r] : r0 + r;
         v = a[row * K + k0 + c];
       }
       As[c][r] = v;
@@ -662,7 +673,7 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int n = n0 + 4 * tx + j;
-        if (n < N) o[n] = acc[i][j];
+        if (n < N) o[n] = MODE == 2 ? relu2(acc[i][j]) : acc[i][j];
       }
     }
   }
@@ -679,6 +690,53 @@ __global__ __launch_bounds__(256) void moe_combine_f32_kernel(
       if (p >= lo && p < hi) s += topk_w[t * k + j] * z[(int64_t)p * H + c];
     }
     out[(int64_t)t * H + c] = s;
+  }
+}
+
+// As the combine kernels, added to the residual stream h [T, W] together with y; the first W of H
+// columns.  out (bf16): the stream after the add, or null.
+template <class T>
+__global__ __launch_bounds__(256) void moe_combine_stream_kernel(
+    bf16_t* __restrict__ out, float* __restrict__ h, const T* __restrict__ y, int64_t ldy,
+    const T* __restrict__ z, const T* __restrict__ z2, const float* __restrict__ topk_w,
+    const int* __restrict__ inv_pos, int W, int H, int k) {
+  const int t = blockIdx.x;
+  float* hr = h + (int64_t)t * W;
+  const T* yr = y + (int64_t)t * ldy;
+  if (W % 8 == 0 && ldy % 8 == 0) {
+    for (int c = threadIdx.x * 8; c < W; c += 256 * 8) {
+      float s[8], d[8];
+      load8(s, yr + c);
+      for (int j = 0; j < k; ++j) {
+        const int64_t p = inv_pos[t * k + j];
+        const float w = topk_w[t * k + j];
+        load8(d, z + p * H + c);
+        if (z2 != nullptr) {
+          float e[8];
+          load8(e, z2 + p * H + c);
+#pragma unroll
+          for (int q = 0; q < 8; ++q) d[q] += e[q];
+        }
+#pragma unroll
+        for (int q = 0; q < 8; ++q) s[q] += w * d[q];
+      }
+      load8(d, hr + c);
+#pragma unroll
+      for (int q = 0; q < 8; ++q) s[q] += d[q];
+      store8(hr + c, s);
+      if (out) store8(out + (int64_t)t * W + c, s);
+    }
+    return;
+  }
+  for (int c = threadIdx.x; c < W; c += 256) {
+    float s = to_f32(yr[c]);
+    for (int j = 0; j < k; ++j) {
+      const int64_t p = inv_pos[t * k + j];
+      s += topk_w[t * k + j] * (to_f32(z[p * H + c]) + (z2 ? to_f32(z2[p * H + c]) : 0.f));
+    }
+    s += hr[c];
+    hr[c] = s;
+    if (out) out[(int64_t)t * W + c] = f2bf(s);
   }
 }
 
@@ -750,15 +808,21 @@ int launch_moe(void* out, const void* x, const void* router_logits, const void* 
                int logit_es, const MoeOptions& opt, hipStream_t st) {
   if (T == 0) return 0;
   if (!((logit_ts == E && logit_es == 1) || (logit_ts == 1 && logit_es >= T))) return -1;
+  const bool glu = act != 3;  // 3: squared relu without a gate
   if (E > 256 || k > kMoeMaxK || k < 1 || k > E || e_off < 0 || e_local < 1 ||
-      e_off + e_local > E || act < 0 || act > 2)
+      e_off + e_local > E || act < 0 || act > 3)
     return -1;
-  if (!opt.f32 && (H % 128 != 0 || I % 64 != 0 || H % kBK != 0)) return -1;
+  if (!opt.f32 && (H % 128 != 0 || I % (glu ? 64 : 128) != 0)) return -1;
+  if (opt.stream && (opt.y == nullptr || opt.W < 1 || opt.W > H || opt.ldy < opt.W || e_off != 0 ||
+                     e_local != E))
+    return -1;
   if (opt.groups < 1 || opt.groups > kMoeMaxGroups || E % opt.groups || opt.keep < 1 ||
       opt.keep > opt.groups || k > opt.keep * (E / opt.groups))
     return -1;
   const int64_t esz = opt.f32 ? 4 : 2;
-  const int epi_gu = act == 2 ? 5 : 2 + act, epi_xd = act == 2 ? 4 : 2 + act;  // gemm_w4 / gemm_xd
+  // epilogues of gemm_w4 / gemm_xd
+  const int epi_gu = act == 3 ? 4 : act == 2 ? 5 : 2 + act, epi_xd = act == 3 ? 5 : 2 + act;
+  const int up_rows = glu ? 2 * I : I;
   if (opt.f32) variant = 0;
   const int P = T * k;
   // GEMM structure: 0 = 128-row 2-barrier (small tiles, decode), 1 = 128-row
@@ -774,7 +838,7 @@ int launch_moe(void* out, const void* x, const void* router_logits, const void* 
   if (auto_v) variant = rows_e >= kMoeW4Rows ? 4 : (rows_e >= 96 ? 3 : 1);
   if (variant > 4) return -1;
   // variant 4: the persistent GEMM's prologue stages two K tiles; the down reduction is I
-  if (variant == 4 && (H / 64 < 2 || I % 128 || I / 64 < 2 || H % 256)) {
+  if (variant == 4 && (H / 64 < 2 || I % (glu ? 128 : 256) || I / 64 < 2 || H % 256)) {
     if (!auto_v) return -1;
     variant = 3;
   }
@@ -792,7 +856,7 @@ int launch_moe(void* out, const void* x, const void* router_logits, const void* 
     if (gu_auto) {
       for (int f : rows_e >= 96 ? std::initializer_list<int>{281, 241} :
                                   std::initializer_list<int>{141})
-        if (moe_xd_ok(f, I, H, true)) { gu_form = f; break; }
+        if (moe_xd_ok(f, I, H, glu)) { gu_form = f; break; }
     }
     const int mt0 = (gu_form % 1000) / 100, bm0 = 128 * mt0;
     if (gu_auto && gu_form && gu_form < 1000 && rows_e <= bm0) gu_form += 1000;
@@ -810,7 +874,7 @@ int launch_moe(void* out, const void* x, const void* router_logits, const void* 
       }
       if (dn_form && rows_e <= bm0) dn_form += 1000;
     }
-    const bool ok = gu_form && dn_form && moe_xd_ok(gu_form, I, H, true) &&
+    const bool ok = gu_form && dn_form && moe_xd_ok(gu_form, I, H, glu) &&
                     moe_xd_ok(dn_form, H, I, false) &&
                     (gu_form % 1000) / 100 == (dn_form % 1000) / 100;  // one tile table
     if (!ok) {
@@ -865,14 +929,21 @@ int launch_moe(void* out, const void* x, const void* router_logits, const void* 
                      variant == 4 ? grp_off : (int*)nullptr);
   hipLaunchKernelGGL(moe_scatter_kernel, dim3(G), dim3(kMoeRouteWG), 0, st, (const float*)topk_w,
                      (const int*)wg_base, T, E, k, sorted_tok, sorted_w, inv_pos);
-  const dim3 g_gu((I / 64) * max_tiles), g_dn((H / 128) * max_tiles);
+  const dim3 g_gu((I / (glu ? 64 : 128)) * max_tiles), g_dn((H / 128) * max_tiles);
   if (opt.f32) {
-    moe_gemm_f32_kernel<0><<<dim3((I + 31) / 32, max_tiles), dim3(256), 0, st>>>(
+    const dim3 g_up(glu ? (I + 31) / 32 : (I + 63) / 64, max_tiles);
+    (glu ? moe_gemm_f32_kernel<0> : moe_gemm_f32_kernel<2>)<<<g_up, dim3(256), 0, st>>>(
         (float*)hbuf, (const float*)x, (const float*)w_gu, sorted_tok, t_e, t_r0, t_n, n_tiles, H,
         I, act, opt.limit);
     moe_gemm_f32_kernel<1><<<dim3((H + 63) / 64, max_tiles), dim3(256), 0, st>>>(
         (float*)zbuf, (const float*)hbuf, (const float*)w_dn, sorted_tok, t_e, t_r0, t_n, n_tiles,
         I, H, 0, 0.f);
+    if (opt.stream) {
+      moe_combine_stream_kernel<float><<<dim3(T), dim3(256), 0, st>>>(
+          nullptr, opt.stream, (const float*)opt.y, opt.ldy, (const float*)zbuf, nullptr, topk_w,
+          inv_pos, opt.W, H, k);
+      return (int)hipGetLastError();
+    }
     moe_combine_f32_kernel<<<dim3(T), dim3(256), 0, st>>>((float*)out, (const float*)zbuf, topk_w,
                                                           inv_pos, local_range, H, k);
     return (int)hipGetLastError();
@@ -883,7 +954,8 @@ int launch_moe(void* out, const void* x, const void* router_logits, const void* 
     hipLaunchKernelGGL(moe_gather_kernel, dim3(min(P, 8192)), dim3(256), 0, st, xs,
                        (const bf16_t*)x, sorted_tok, local_range, P, H);
     int e = launch_gemm_w4_grouped(hbuf, xs, w_gu, grp_off, e_local, P, I, H, H, H, I,
-                                   2ll * I * H, epi_gu, I, g_moe_gm_gu, 1, 0, opt.limit, st);
+                                   (int64_t)up_rows * H, epi_gu, glu ? I : 0, g_moe_gm_gu, 1, 0,
+                                   opt.limit, st);
     if (e) return e;
     if (dn_form) {
       // down on gemm_xd's grouped split-K forms over the 256-row tile table (few rows per
@@ -903,7 +975,7 @@ int launch_moe(void* out, const void* x, const void* router_logits, const void* 
     int mt, nf, sk, e;
     moe_xd_form(gu_form, mt, nf, sk);
     e = launch_gemm_xd_grouped(hbuf, x, w_gu, T, I, H, H, H, I, epi_xd, mt, nf, sk, max_tiles,
-                               t_r0, t_n, t_e, n_tiles, sorted_tok, 2ll * I * H, slab,
+                               t_r0, t_n, t_e, n_tiles, sorted_tok, (int64_t)up_rows * H, slab,
                                slab_bytes, counters, n_counters, opt.limit, st);
     if (e) return e;
     moe_xd_form(dn_form, mt, nf, sk);
@@ -912,28 +984,36 @@ int launch_moe(void* out, const void* x, const void* router_logits, const void* 
                                slab_bytes, counters, n_counters, 0.f, st);
     if (e) return e;
   } else if (variant == 0) {
-    hipLaunchKernelGGL(moe_gemm_kernel<0>, g_gu, dim3(256), 0, st, hbuf, (const bf16_t*)x,
-                       (const bf16_t*)w_gu, sorted_tok, t_e, t_r0, t_n, n_tiles, H, 2 * I, I, I,
-                       max_tiles, act, opt.limit);
+    hipLaunchKernelGGL((glu ? moe_gemm_kernel<0> : moe_gemm_kernel<2>), g_gu, dim3(256), 0, st, hbuf,
+                       (const bf16_t*)x, (const bf16_t*)w_gu, sorted_tok, t_e, t_r0, t_n, n_tiles, H,
+                       up_rows, I, I, max_tiles, act, opt.limit);
     hipLaunchKernelGGL(moe_gemm_kernel<1>, g_dn, dim3(256), 0, st, zbuf, (const bf16_t*)hbuf,
                        (const bf16_t*)w_dn, sorted_tok, t_e, t_r0, t_n, n_tiles, I, H, I, H,
                        max_tiles, 0, 0.f);
   } else if (variant == 1) {
     using Cf = PipeCfg<128>;
-    hipLaunchKernelGGL((moe_gemm_pipe_kernel<128, 0>), g_gu, dim3(Cf::NT), Cf::LDS_BYTES, st, hbuf,
-                       (const bf16_t*)x, (const bf16_t*)w_gu, sorted_tok, t_e, t_r0, t_n, n_tiles, H,
-                       2 * I, I, I, max_tiles, act, opt.limit);
+    hipLaunchKernelGGL((glu ? moe_gemm_pipe_kernel<128, 0> : moe_gemm_pipe_kernel<128, 2>), g_gu,
+                       dim3(Cf::NT), Cf::LDS_BYTES, st, hbuf, (const bf16_t*)x, (const bf16_t*)w_gu,
+                       sorted_tok, t_e, t_r0, t_n, n_tiles, H, up_rows, I, I, max_tiles, act,
+                       opt.limit);
     hipLaunchKernelGGL((moe_gemm_pipe_kernel<128, 1>), g_dn, dim3(Cf::NT), Cf::LDS_BYTES, st, zbuf,
                        (const bf16_t*)hbuf, (const bf16_t*)w_dn, sorted_tok, t_e, t_r0, t_n,
                        n_tiles, I, H, I, H, max_tiles, 0, 0.f);
   } else {
     using Cf = PipeCfg<256>;
-    hipLaunchKernelGGL((moe_gemm_pipe_kernel<256, 0>), g_gu, dim3(Cf::NT), Cf::LDS_BYTES, st, hbuf,
-                       (const bf16_t*)x, (const bf16_t*)w_gu, sorted_tok, t_e, t_r0, t_n, n_tiles, H,
-                       2 * I, I, I, max_tiles, act, opt.limit);
+    hipLaunchKernelGGL((glu ? moe_gemm_pipe_kernel<256, 0> : moe_gemm_pipe_kernel<256, 2>), g_gu,
+                       dim3(Cf::NT), Cf::LDS_BYTES, st, hbuf, (const bf16_t*)x, (const bf16_t*)w_gu,
+                       sorted_tok, t_e, t_r0, t_n, n_tiles, H, up_rows, I, I, max_tiles, act,
+                       opt.limit);
     hipLaunchKernelGGL((moe_gemm_pipe_kernel<256, 1>), g_dn, dim3(Cf::NT), Cf::LDS_BYTES, st, zbuf,
                        (const bf16_t*)hbuf, (const bf16_t*)w_dn, sorted_tok, t_e, t_r0, t_n,
                        n_tiles, I, H, I, H, max_tiles, 0, 0.f);
+  }
+  if (opt.stream) {
+    moe_combine_stream_kernel<bf16_t><<<dim3(T), dim3(256), 0, st>>>(
+        (bf16_t*)out, opt.stream, (const bf16_t*)opt.y, opt.ldy, zbuf,
+        dn_split ? (const bf16_t*)zbuf2 : nullptr, topk_w, inv_pos, opt.W, H, k);
+    return (int)hipGetLastError();
   }
   hipLaunchKernelGGL(moe_combine_kernel, dim3(T), dim3(256), 0, st, (bf16_t*)out, zbuf,
                      dn_split ? (const bf16_t*)zbuf2 : nullptr, topk_w, inv_pos, local_range, T, H,
@@ -952,9 +1032,13 @@ int configure_moe() {
                                 hipFuncAttributeMaxDynamicSharedMemorySize, PipeCfg<128>::LDS_BYTES);
   e |= (int)hipFuncSetAttribute((const void*)moe_gemm_pipe_kernel<128, 1>,
                                 hipFuncAttributeMaxDynamicSharedMemorySize, PipeCfg<128>::LDS_BYTES);
+  e |= (int)hipFuncSetAttribute((const void*)moe_gemm_pipe_kernel<128, 2>,
+                                hipFuncAttributeMaxDynamicSharedMemorySize, PipeCfg<128>::LDS_BYTES);
   e |= (int)hipFuncSetAttribute((const void*)moe_gemm_pipe_kernel<256, 0>,
                                 hipFuncAttributeMaxDynamicSharedMemorySize, PipeCfg<256>::LDS_BYTES);
   e |= (int)hipFuncSetAttribute((const void*)moe_gemm_pipe_kernel<256, 1>,
+                                hipFuncAttributeMaxDynamicSharedMemorySize, PipeCfg<256>::LDS_BYTES);
+  e |= (int)hipFuncSetAttribute((const void*)moe_gemm_pipe_kernel<256, 2>,
                                 hipFuncAttributeMaxDynamicSharedMemorySize, PipeCfg<256>::LDS_BYTES);
   return e;
 }

@@ -16,9 +16,9 @@ from __future__ import annotations
 
 import torch
 
-from ..ops import KV_BLOCK, latent_width, pad8, talk_cache_shapes
+from ..ops import KV_BLOCK, latent_width, memory_slices, pad8, talk_cache_shapes
 from ..models.config import (GatedAverage, GroupedAttention, HybridConfig, Layer, LatentAttention,
-                             ModelConfig, TalkingAttention)
+                             MatrixMemory, ModelConfig, Retention, TalkingAttention)
 from .block_allocator import BlockAllocator
 
 
@@ -116,7 +116,14 @@ def _layer_parts(l: Layer, dtype) -> tuple[list, list]:
     state slot."""
     m, f32 = l.mixer, torch.float32
     if isinstance(m, LatentAttention):
+        if m.kv_from is not None:  # nothing of its own
+            return [], []
         return [((KV_BLOCK, latent_width(m.kv_rank, m.rot_dim)), dtype)], []
+    if isinstance(m, Retention):
+        return [], [((m.heads, m.dim, m.vdim), f32)]
+    if isinstance(m, MatrixMemory):
+        n = memory_slices(m.vdim)
+        return [], [((m.heads, m.dim, m.vdim), f32), ((m.heads, n, m.dim), f32), ((m.heads, n), f32)]
     if isinstance(m, TalkingAttention):
         return [(s, dtype) for s in talk_cache_shapes(m.kv_heads, m.dim, m.vdim)], []
     if isinstance(m, GroupedAttention):
@@ -143,6 +150,7 @@ class HybridCache:
     state slots - one per live sequence - for its recurrent layers and convolved inputs.
 
       latent layer    [num_blocks, 32, latent_width]                      (ops/latent.py)
+                      a layer with kv_from: the very tensor of the layer it reads
       talking layer   keys, values [num_blocks, ...]                      (ops/talking.py)
                       and the plane [num_blocks, heads, 32] of scores all such layers share
       grouped layer   keys, values as a talking layer's; ring [slots, taps - 1, channels] of
@@ -150,6 +158,9 @@ class HybridCache:
       delta layer     ring  [slots, taps, channels]       last convolution inputs
                       state [slots, heads, dim, vdim]     fp32
       average layer   state [slots, channels]             fp32
+      retention layer state [slots, heads, dim, vdim]     fp32            (ops/memory.py)
+      memory layer    state as a retention layer's; normaliser [slots, heads, slices, dim] and
+                      running maximum [slots, heads, slices] of each column slice    fp32
       rings           [slots, sublayers, taps - 1, W]     convolved inputs, per layer
 
     Blocks come from ``allocator`` (block 0 is the padding target), slots from ``states``.
@@ -173,7 +184,8 @@ class HybridCache:
             ts = [new(self.num_blocks, *p) for p in block] + [new(self.num_slots, *p) for p in slot]
             if isinstance(l.mixer, TalkingAttention):
                 ts.append(self.plane)
-            self.layers.append(ts[0] if len(ts) == 1 else tuple(ts))
+            j = getattr(l.mixer, "kv_from", None)
+            self.layers.append(self.layers[j] if j is not None else ts[0] if len(ts) == 1 else tuple(ts))
             ring = _ring_part(cfg, l)
             self.rings.append(new(self.num_slots, ring, dtype) if ring else None)
         self.allocator = BlockAllocator(self.num_blocks, reserved=1)
@@ -187,7 +199,8 @@ class HybridCache:
 
     @property
     def bytes(self) -> int:
-        ts = [t for l in self.layers for t in (l if isinstance(l, tuple) else (l,))] + self.rings
+        ts = [t for c, l in zip(self.layers, self.cfg.layers) if getattr(l.mixer, "kv_from", None) is None
+              for t in (c if isinstance(c, tuple) else (c,))] + self.rings
         ts = [t for t in ts if t is not None and t is not self.plane]
         return sum(t.numel() * t.element_size() for t in ts + ([self.plane] if self.plane is not None else []))
 

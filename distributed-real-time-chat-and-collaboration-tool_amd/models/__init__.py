@@ -1,6 +1,7 @@
 """Model zoo: Llama-3 (8B/70B), Gemma-2B, Mixtral-8x7B (random-init bf16), and the designs with layers
 of mixed kinds, Ralesun (latent attention + gated delta rule), Mebalorn (talking-heads attention +
-minGRU) and Nurilorn (capped attention with convolved projections + routed experts): random-init
+minGRU), Nurilorn (capped attention with convolved projections + routed experts) and Garesun
+(retention, matrix memory and attention over shared latents beside routed experts): random-init
 presets and checkpoint folders."""
 from __future__ import annotations
 
@@ -8,10 +9,10 @@ import os
 
 
 from .checkpoint import read_safetensors
-from .config import (GEMMA_2B, LLAMA3_8B, LLAMA3_70B, MEBALORN_2B, MEBALORN_8B, MIXTRAL_8X7B,
+from .config import (GARESUN_5B, GARESUN_24B, GEMMA_2B, LLAMA3_8B, LLAMA3_70B, MEBALORN_2B, MEBALORN_8B, MIXTRAL_8X7B,
                      NURILORN_5B, NURILORN_24B, RALESUN_2B, RALESUN_8B, REGISTRY, TINY_GEMMA,
-                     TINY_LLAMA, TINY_MEBALORN, TINY_MIXTRAL, TINY_NURILORN, TINY_RALESUN, HybridConfig, ModelConfig, config_from_dict,
-                     get_config, load_config)
+                     TINY_GARESUN, TINY_LLAMA, TINY_MEBALORN, TINY_MIXTRAL, TINY_NURILORN, TINY_RALESUN,
+                     HybridConfig, ModelConfig, config_from_dict, get_config, load_config)
 from .hybrid import HybridLM
 from .transformer import DecodeMeta, PrefillMeta, TransformerLM
 
@@ -36,7 +37,7 @@ def load_model(name: str, device="cpu", *, max_position: int | None = None, **kw
     return build_model(cfg, device, tensors=tensors, **kw)
 
 
-__all__ = ["GEMMA_2B", "LLAMA3_8B", "LLAMA3_70B", "MEBALORN_2B", "MEBALORN_8B", "MIXTRAL_8X7B",
+__all__ = ["GARESUN_5B", "GARESUN_24B", "TINY_GARESUN", "GEMMA_2B", "LLAMA3_8B", "LLAMA3_70B", "MEBALORN_2B", "MEBALORN_8B", "MIXTRAL_8X7B",
            "NURILORN_5B", "NURILORN_24B", "RALESUN_2B", "RALESUN_8B", "REGISTRY", "TINY_GEMMA",
            "TINY_LLAMA", "TINY_MEBALORN", "TINY_MIXTRAL", "TINY_NURILORN", "TINY_RALESUN", "HybridConfig",
            "HybridLM", "ModelConfig", "build_model", "config_from_dict", "get_config",

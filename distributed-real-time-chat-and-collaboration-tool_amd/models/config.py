@@ -10,9 +10,10 @@ plus tiny variants of each for CPU tests.
 :class:`HybridConfig` describes models whose layers differ (mixer kind, sizes, window, with or
 without a feed-forward): the Ralesun design, latent attention and channel-wise gated delta-rule
 mixers one after the other with their feed-forward; the Mebalorn design, talking-heads attention
-and minGRU mixers beside it; and the Nurilorn design, attention with convolved projections and
-capped scores, followed by a clamped feed-forward or routed experts.  Their checkpoints carry a config.json, parsed by
-:func:`config_from_dict`.
+and minGRU mixers beside it; the Nurilorn design, attention with convolved projections and
+capped scores, followed by a clamped feed-forward or routed experts; and the Garesun design,
+retention, matrix memory and latent attention with shared latents beside squared-relu experts.
+Their checkpoints carry a config.json, parsed by :func:`config_from_dict`.
 """
 from __future__ import annotations
 
@@ -126,7 +127,8 @@ TINY_MIXTRAL = ModelConfig(
 class LatentAttention:
     """Attention over per-token latents: heads of ``dim`` unrotated + ``rot_dim`` rotated query
     dims, values of ``vdim``, latents of ``kv_rank``; ``window`` tokens visible (None: all);
-    the first ``rot_dims`` rotated dims turned in interleaved pairs; a softmax sink per head."""
+    the first ``rot_dims`` rotated dims turned in interleaved pairs; a softmax sink and a sigmoid
+    gate per head.  ``kv_from``: attends to that layer's cached latents instead of its own."""
     heads: int
     dim: int
     rot_dim: int
@@ -137,10 +139,14 @@ class LatentAttention:
     rot_base: float
     rot_dims: int
     sink: bool = True
+    gate: bool = False
+    kv_from: int | None = None
 
     def __post_init__(self):
         if self.rot_dims % 2 or self.rot_dims > self.rot_dim:
             raise ValueError(f"rotated dims {self.rot_dims} of a {self.rot_dim}-wide part")
+        if self.kv_rank % 2 or self.rot_dim % 2:
+            raise ValueError("latent attention kernels take even latents and rotated parts")
         if not self.scale > 0:
             raise ValueError("scores need a positive scale")
         if self.window is not None and self.window < 1:
@@ -210,6 +216,45 @@ class GatedAverage:
     def __post_init__(self):
         if self.width < 1:
             raise ValueError("a recurrence needs channels")
+
+
+def _check_memory(m) -> None:
+    if m.heads < 1 or not 1 <= m.dim <= 256 or not 1 <= m.vdim <= 1024:
+        raise ValueError("matrix memories take keys up to 256 and values up to 1024 wide")
+
+
+@dataclass(frozen=True)
+class Retention:
+    """Linear attention with a fixed ``decay`` per head; the first ``rot_dims`` dims of queries and
+    keys turned in pairs half of them apart."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple[float, ...]
+    rot_base: float = 10000.0
+    rot_dims: int = 0
+
+    def __post_init__(self):
+        _check_memory(self)
+        if len(self.decay) != self.heads or not all(0 < x <= 1 for x in self.decay):
+            raise ValueError("retention takes a decay above 0 and up to 1 for each head")
+        if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.dim:
+            raise ValueError(f"rotated dims {self.rot_dims} of a {self.dim}-wide head")
+
+
+@dataclass(frozen=True)
+class MatrixMemory:
+    """mLSTM: linear attention with exponential input and sigmoid forget gates per head and token,
+    both capped at +-``gate_cap`` in the logarithm, read out against a normaliser."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+    def __post_init__(self):
+        _check_memory(self)
+        if not self.gate_cap > 0:
+            raise ValueError("gates are capped at a positive number")
 
 
 @dataclass(frozen=True)
@@ -283,10 +328,12 @@ class Experts:
 
 @dataclass(frozen=True)
 class Layer:
-    mixer: LatentAttention | ChannelDelta | TalkingAttention | GatedAverage | GroupedAttention
+    mixer: LatentAttention | ChannelDelta | TalkingAttention | GatedAverage | GroupedAttention | \
+        Retention | MatrixMemory
     ff: int | None = None  # feed-forward size; None: the layer is its mixer alone
     limit: float = 0.0     # bound of the clamped activation
     experts: Experts | None = None  # the feed-forward is this mixture, ``ff`` each expert's size
+    shared: int | None = None  # size of the expert that every token uses beside them
 
 
 @dataclass(frozen=True)
@@ -302,11 +349,12 @@ class HybridConfig:
     eos_token_id: int = 2
     init_std: float = 0.02
     prefill_chunk: int = 16384
-    # the layers' structure: "serial" (norm, mixer, norm, gated feed-forward) or "parallel" (mixer
-    # and squared-relu feed-forward on two layer norms of the same stream)
+    # the layers' structure: "serial" (norm, mixer, norm, gated feed-forward), "parallel" (mixer
+    # and squared-relu feed-forward on two layer norms of the same stream) or "joint" (both on one
+    # layer norm)
     block: str = "serial"
     # serial: "dyt" (Dynamic Tanh) or "group_rms" (RMS norms of norm_groups parts of a row, factors
-    # per column on what a sublayer adds)
+    # per column on what a sublayer adds); joint: "layer" (layer norms without bias)
     norm: str = "dyt"
     norm_groups: int = 1
     embed_scale: float = 1.0
@@ -315,25 +363,32 @@ class HybridConfig:
     conv_taps: int = 1                    # parallel: causal convolution added to sublayer inputs
     sinusoids: bool = False               # sinusoidal positions added to the embedding
     logit_softcap: float | None = None
+    side_dim: int = 0                     # joint: size of a token's own input to each layer
 
     def __post_init__(self):
-        if self.block not in ("serial", "parallel"):
+        if self.block not in ("serial", "parallel", "joint"):
             raise ValueError(f"unknown layer structure {self.block!r}")
-        if self.block == "serial" and (self.conv_taps != 1 or self.sinusoids or self.logit_softcap):
-            raise ValueError("serial layers have no convolved inputs, sinusoids or logit cap")
-        if self.norm not in ("dyt", "group_rms"):
+        if self.block != "parallel" and (self.conv_taps != 1 or self.sinusoids or self.logit_softcap):
+            raise ValueError("convolved inputs, sinusoids and a logit cap come with parallel layers")
+        if self.norm not in ("dyt", "group_rms", "layer"):
             raise ValueError(f"unknown norm {self.norm!r}")
-        if self.norm == "dyt" and (self.norm_groups, self.embed_scale, self.residual_mult,
-                                   self.logit_scale) != (1, 1.0, 1.0, 1.0):
+        if (self.norm == "layer") != (self.block == "joint"):
+            raise ValueError("joint layers, and only they, have layer norms without bias")
+        if self.norm != "group_rms" and (self.norm_groups, self.residual_mult,
+                                         self.logit_scale) != (1, 1.0, 1.0):
             raise ValueError("groups and scales come with norms in groups")
+        if self.norm == "dyt" and self.embed_scale != 1.0:
+            raise ValueError("an embedding scale comes with norms in groups and layer norms")
+        self._check_joint()
         if self.norm == "group_rms":
             if self.block != "serial" or self.norm_groups < 1 or \
                     self.hidden_size % self.norm_groups or self.hidden_size + self.norm_groups > 16384:
                 raise ValueError("norms in groups take equal parts of serial rows up to 16K columns")
         if self.act == "clamped" and any(l.ff and not l.limit > 0 for l in self.layers):
             raise ValueError("the clamped activation needs a positive limit")
-        if any(l.experts and not (l.ff and self.norm == "group_rms") for l in self.layers):
-            raise ValueError("experts are feed-forwards of layers with norms in groups")
+        if any(l.experts and not (l.ff and self.norm != "dyt" and self.block != "parallel")
+               for l in self.layers):
+            raise ValueError("experts are feed-forwards of layers with norms in groups, or joint ones")
         if len({l.mixer.kv_heads * l.mixer.vdim for l in self.layers
                 if isinstance(l.mixer, GroupedAttention) and l.mixer.v_mix}) > 1:
             raise ValueError("layers that mix values need values of one size")
@@ -348,6 +403,25 @@ class HybridConfig:
 
     is_moe = False
     tie_embeddings = False
+
+    def _check_joint(self) -> None:
+        joint = self.block == "joint"
+        if not joint and (self.side_dim or any(l.shared for l in self.layers)):
+            raise ValueError("side inputs and shared experts come with joint layers")
+        if joint and (self.act != "relu2" or self.hidden_size > 16384 or self.side_dim < 0):
+            raise ValueError("joint layers take squared-relu feed-forwards and rows up to 16K columns")
+        if any(l.shared and not l.experts for l in self.layers):
+            raise ValueError("a shared expert stands beside others")
+        for i, m in enumerate(l.mixer for l in self.layers):
+            if not joint and (isinstance(m, (Retention, MatrixMemory))
+                              or isinstance(m, LatentAttention) and (m.gate or m.kv_from is not None)):
+                raise ValueError("matrix memories, head gates and shared latents come with joint layers")
+            if isinstance(m, LatentAttention) and m.kv_from is not None:
+                s = self.layers[m.kv_from].mixer if 0 <= m.kv_from < i else None
+                if not isinstance(s, LatentAttention) or s.kv_from is not None or \
+                        (s.kv_rank, s.rot_dim, s.rot_dims, s.rot_base) != \
+                        (m.kv_rank, m.rot_dim, m.rot_dims, m.rot_base):
+                    raise ValueError(f"layer {i} cannot read the latents of layer {m.kv_from}")
 
     @property
     def num_layers(self) -> int:
@@ -368,6 +442,8 @@ class HybridConfig:
     def num_params(self) -> int:
         if self.norm == "group_rms":
             return self._num_params_scaled()
+        if self.block == "joint":
+            return self._num_params_joint()
         W, n = self.hidden_size, 2 * self.vocab_size * self.hidden_size + 2 * self.hidden_size
         serial = self.block == "serial"
         for l in self.layers:
@@ -398,6 +474,24 @@ class HybridConfig:
             n += m.channels * m.conv
             if l.ff:
                 n += 3 * W * l.ff * (l.experts.count if l.experts else 1) + 2 * W
+                n += W * l.experts.count if l.experts else 0
+        return n
+
+    def _num_params_joint(self) -> int:
+        W, side = self.hidden_size, self.side_dim
+        n = W + self.vocab_size * (2 * W + self.num_layers * side)
+        for l in self.layers:
+            m = l.mixer
+            if isinstance(m, LatentAttention):
+                n += W * m.heads * (m.dim + m.rot_dim + m.vdim + m.gate) + m.kv_rank * m.heads * (m.dim + m.vdim)
+                n += (m.heads if m.sink else 0)
+                n += 0 if m.kv_from is not None else W * (m.kv_rank + m.rot_dim) + m.kv_rank
+            else:
+                n += W * m.heads * (2 * m.dim + 3 * m.vdim)
+                n += m.heads * (2 * W + 2 + m.vdim) if isinstance(m, MatrixMemory) else 0
+            n += W + (W * (2 * side + 1) if side else 0)
+            if l.ff:
+                n += 2 * W * (l.ff * (l.experts.count if l.experts else 1) + (l.shared or 0))
                 n += W * l.experts.count if l.experts else 0
         return n
 
@@ -478,8 +572,40 @@ def _nurilorn(d: dict, name: str) -> HybridConfig:
                         logit_scale=float(d["logit_scale"]))
 
 
+def _garesun(d: dict, name: str) -> HybridConfig:
+    layers = []
+    for e in d["layers"]:
+        m = e["mixer"]
+        rot = m.get("rot") or {"base": 10000.0, "dims": 0}
+        if e["type"] == "latent_attention":
+            mixer = LatentAttention(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"],
+                                    float(m["scale"]), None, float(rot["base"]), rot["dims"],
+                                    sink=False, gate=True, kv_from=m.get("kv_from"))
+        elif e["type"] == "retention":
+            mixer = Retention(m["heads"], m["dim"], m["vdim"], tuple(map(float, m["decay"])),
+                              float(rot["base"]), rot["dims"])
+        elif e["type"] == "mlstm":
+            mixer = MatrixMemory(m["heads"], m["dim"], m["vdim"], float(m["gate_cap"]))
+        else:
+            raise ValueError(f"unknown layer type {e['type']!r}")
+        mlp = e["mlp"]
+        if mlp is None:
+            layers.append(Layer(mixer))
+        elif mlp["kind"] == "moe":
+            r, shared = mlp["router"], mlp.get("shared")
+            layers.append(Layer(mixer, mlp["expert"]["ff"], experts=Experts(r["experts"], r["top"]),
+                                shared=shared["ff"] if shared else None))
+        else:
+            raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+    return HybridConfig(name, d["vocab"], d["width"], tuple(layers), float(d["norm"]["eps"]),
+                        act="relu2", max_position=d.get("max_position", 32768), bos_token_id=0,
+                        eos_token_id=-1, block="joint", norm="layer",
+                        embed_scale=float(d["embedding"]["scale"]), side_dim=d["token_side"]["dim"])
+
+
 # checkpoint configuration ("architecture" key) -> parser
-ARCHITECTURES = {"Ralesun": _ralesun, "Mebalorn": _mebalorn, "Nurilorn": _nurilorn}
+ARCHITECTURES = {"Ralesun": _ralesun, "Mebalorn": _mebalorn, "Nurilorn": _nurilorn,
+                 "Garesun": _garesun}
 
 
 def config_from_dict(d: dict, name: str = "") -> HybridConfig:
@@ -572,10 +698,50 @@ TINY_NURILORN = _scaled("tiny-nurilorn", 160, (
           Experts(6, 2, 3, 2))), vocab=384, norm_groups=4, embed_scale=4.0, max_position=1024,
     init_std=0.06)
 
+def _joint(name: str, width: int, layers: tuple, side: int, vocab: int = 128256, **kw) -> HybridConfig:
+    return HybridConfig(name, vocab, width, layers, act="relu2", block="joint", norm="layer",
+                        embed_scale=4.0, side_dim=side, **kw)
+
+
+def retention_decays(heads: int) -> tuple[float, ...]:
+    """Spans from 32 tokens to thousands, one per head."""
+    return tuple(1 - 2.0 ** (-5 - 7 * h / max(heads - 1, 1)) for h in range(heads))
+
+
+def _memories(blocks: int, heads: int, ff: int, experts: Experts) -> tuple:
+    """Blocks of matrix memory, latent attention, retention, and an attention that reads the same
+    latents; a shared expert twice as wide as the others."""
+    out = []
+    for b in range(blocks):
+        att = LatentAttention(heads, 128, 64, 128, 512, 192 ** -0.5, None, 500000.0, 64, False, True)
+        for m in (MatrixMemory(heads, 128, 128, 15.0), att,
+                  Retention(heads, 128, 128, retention_decays(heads), 500000.0, 128),
+                  dataclasses.replace(att, kv_from=4 * b + 1)):
+            out.append(Layer(m, ff, experts=experts, shared=2 * ff))
+    return tuple(out)
+
+
+# Llama's head sizes; a token's four routed experts and its shared one together as many parameters
+# as its feed-forward.
+GARESUN_24B = _joint("garesun-24b", 4096, _memories(8, 32, 3584, Experts(20, 4)), 256,
+                     bos_token_id=128000, eos_token_id=128001)
+
+GARESUN_5B = _joint("garesun-5b", 2048, _memories(6, 16, 1792, Experts(20, 4)), 128,
+                    bos_token_id=128000, eos_token_id=128001)
+
+TINY_GARESUN = _joint("tiny-garesun", 160, (
+    Layer(LatentAttention(3, 24, 8, 40, 48, 0.2, None, 10000.0, 8, False, True), 72,
+          experts=Experts(6, 2), shared=104),
+    Layer(Retention(2, 48, 32, (0.9, 0.99), 5000.0, 32)),
+    Layer(MatrixMemory(3, 16, 40, 10.0), 40, experts=Experts(5, 3)),
+    Layer(LatentAttention(5, 16, 8, 24, 48, 0.25, None, 10000.0, 8, False, True, kv_from=0), 56,
+          experts=Experts(8, 1), shared=48)), 24, vocab=384, max_position=1024, init_std=0.06)
+
 REGISTRY = {c.name: c for c in (LLAMA3_8B, LLAMA3_70B, GEMMA_2B, MIXTRAL_8X7B,
                                 TINY_LLAMA, TINY_GEMMA, TINY_MIXTRAL, RALESUN_8B, RALESUN_2B,
                                 TINY_RALESUN, MEBALORN_8B, MEBALORN_2B, TINY_MEBALORN,
-                                NURILORN_24B, NURILORN_5B, TINY_NURILORN)}
+                                NURILORN_24B, NURILORN_5B, TINY_NURILORN,
+                                GARESUN_24B, GARESUN_5B, TINY_GARESUN)}
 
 
 def get_config(name: str) -> ModelConfig | HybridConfig:

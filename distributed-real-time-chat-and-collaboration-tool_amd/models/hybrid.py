@@ -8,6 +8,9 @@ structure.
   parallel  two layer norms of one stream, each followed by a causal convolution -> mixer and
             squared-relu feed-forward -> one add (the Mebalorn design: talking-heads attention and
             minGRU, sinusoidal positions, capped logits)
+  joint     one layer norm -> mixer, squared-relu experts and a shared one -> one add, then a gated
+            input of the token to this layer -> norm -> add (the Garesun design: retention, matrix
+            memory, latent attention whose latents several layers may share)
 
 Same interface as :class:`~.transformer.TransformerLM` towards the engine (packed prefill with
 decode rows appended, static-shaped decode, the cache it needs), so scheduler, decode graphs
@@ -19,8 +22,8 @@ and sampler serve it unchanged.  Differences the engine sees:
 
 In bf16 the residual stream, norms, angles, scores, attention weights, decays, step sizes, gates of
 a recurrence and its state are 32-bit; projections and activations bf16.  With dtype float32
-everything is.  In a parallel layer mixer and feed-forward write the columns of ONE operand of ONE
-output projection, so their sum is formed in its fp32 accumulators.
+everything is.  In a parallel or joint layer mixer and (shared) feed-forward write the columns of ONE
+operand of ONE output projection, so their sum is formed in its fp32 accumulators.
 """
 from __future__ import annotations
 
@@ -47,6 +50,12 @@ class Dyt:
 
 @dataclass
 class GroupNorm:
+    w: torch.Tensor
+
+
+@dataclass
+class PlainNorm:
+    """Layer norm without bias."""
     w: torch.Tensor
 
 
@@ -126,7 +135,9 @@ class HybridLM:
         return W if self.dtype == torch.float32 else pad_to(W, 128)
 
     def _expert_ff(self, ff: int) -> int:
-        return ff if self.dtype == torch.float32 else pad_to(ff, 64)
+        if self.dtype == torch.float32:
+            return ff
+        return pad_to(ff, 128 if self.cfg.block == "joint" else 64)
 
     def _norm(self, src, name: str, conv: str | None = None):
         W, t = self.cfg.hidden_size, self.cfg.conv_taps
@@ -134,6 +145,8 @@ class HybridLM:
             w = self.f32(src.take(name, W))
             # the logits' factor rides on the last norm's weights
             return GroupNorm(w * self.cfg.logit_scale if name == "final.norm" else w)
+        if self.cfg.norm == "layer":
+            return PlainNorm(self.f32(src.take(name, W)))
         w, b = src.take(name, W), src.take(name + ".b", W)
         if self.cfg.block == "serial":
             return Dyt(self.f32(w), self.f32(b), float(src.take(name + ".alpha")))
@@ -148,7 +161,11 @@ class HybridLM:
         self.turns = ops.sinusoid_turns(W, self.device) if cfg.sinusoids else None
         scaled = cfg.norm == "group_rms"
         self.layers = []
-        for i, l in enumerate(cfg.layers):
+        for i, l in enumerate(cfg.layers if cfg.block == "joint" else ()):
+            self.layers.append(self._load_joint(src, i, l))
+        if cfg.side_dim:
+            self.side_embed = lin(src.take("side.embed", cfg.vocab_size, cfg.num_layers * cfg.side_dim))
+        for i, l in enumerate(cfg.layers if cfg.block != "joint" else ()):
             p, q = f"l{i}.", f"l{i}.mlp."
             mixer = MIXERS[type(l.mixer)](l.mixer, p + "mix.", src, self)
             L: dict = {"norm1": self._norm(src, p + "norm1", p + "canon1"), "mixer": mixer}
@@ -180,14 +197,40 @@ class HybridLM:
         self.lm_head = lin(src.take("head", cfg.vocab_size, W))
         src.finish()
 
+    def _load_joint(self, src, i: int, l) -> dict:
+        cfg, lin, W = self.cfg, self.lin, self.cfg.hidden_size
+        p, q = f"l{i}.", f"l{i}.mlp."
+        mixer = MIXERS[type(l.mixer)](l.mixer, p + "mix.", src, self)
+        L: dict = {"norm1": self._norm(src, p + "norm1"), "mixer": mixer}
+        # the feed-forward every token uses writes behind the mixer: [mixer | feed-forward] columns
+        # of one output projection
+        name, ff = (q + "shared.", l.shared) if l.experts else (q, l.ff)
+        off, ffp = pad_to(mixer.width), pad_to(ff or 0)
+        L["out"] = self.embed.new_zeros(W, off + ffp)
+        L["out"][:, :mixer.width] = mixer.o
+        mixer.o = None
+        if ff:
+            L["up"] = self.embed.new_zeros(ffp, W)
+            L["up"][:ff] = lin(src.take(name + "up", ff, W))
+            L["out"][:, off:off + ff] = lin(src.take(name + "down", W, ff))
+        if l.experts:
+            self._load_experts(src, q, l, L)
+        if cfg.side_dim:
+            L["side_gate"] = lin(src.take(p + "side.gate", cfg.side_dim, W))
+            L["side_proj"] = lin(src.take(p + "side.proj", W, cfg.side_dim))
+            L["side_norm"] = self.f32(src.take(p + "side.norm", W))
+        return L
+
     def _load_experts(self, src, q: str, l, L: dict) -> None:
         W, ff, n = self.cfg.hidden_size, l.ff, l.experts.count
         Wp, fp = self._moe_width, self._expert_ff(ff)
-        new = self.embed.new_zeros
-        L["experts_in"], L["experts_out"] = new(n, 2 * fp, Wp), new(n, Wp, fp)
+        new, gated = self.embed.new_zeros, self.cfg.act != "relu2"
+        L["experts_in"], L["experts_out"] = new(n, (1 + gated) * fp, Wp), new(n, Wp, fp)
         for e in range(n):
-            L["experts_in"][e, :ff, :W] = self.lin(src.take(f"{q}e{e}.gate", ff, W))
-            L["experts_in"][e, fp:fp + ff, :W] = self.lin(src.take(f"{q}e{e}.up", ff, W))
+            if gated:
+                L["experts_in"][e, :ff, :W] = self.lin(src.take(f"{q}e{e}.gate", ff, W))
+            up = fp if gated else 0
+            L["experts_in"][e, up:up + ff, :W] = self.lin(src.take(f"{q}e{e}.up", ff, W))
             L["experts_out"][e, :W, :ff] = self.lin(src.take(f"{q}e{e}.down", W, ff))
         L["router"] = new(n, Wp)
         L["router"][:, :W] = self.lin(src.take(q + "router", n, W))
@@ -197,10 +240,11 @@ class HybridLM:
             return [t for t in vars(n).values() if isinstance(t, torch.Tensor)]
 
         ts = [self.embed, self.lm_head, *norm(self.final)]
+        ts += [self.side_embed] if self.cfg.side_dim else []
         for L in self.layers:
             for v in L.values():
                 ts += [v] if isinstance(v, torch.Tensor) else \
-                    norm(v) if isinstance(v, (Dyt, GroupNorm, ops.LayerNorm)) else v.operands()
+                    norm(v) if isinstance(v, (Dyt, GroupNorm, PlainNorm, ops.LayerNorm)) else v.operands()
         return sum(t.numel() * t.element_size() for t in ts)
 
     # ------------------------------------------------------------ engine hooks
@@ -359,11 +403,11 @@ class HybridLM:
                              embed=self.embed, embed_scale=cfg.embed_scale, width=width,
                              dtype=self.dtype)
 
-    def _experts(self, L: dict, l, x: torch.Tensor) -> torch.Tensor:
+    def _experts(self, L: dict, l, x: torch.Tensor, **kw) -> torch.Tensor:
         e = l.experts
         return ops.fused_moe(x, ops.router_logits_f32(x, L["router"]), L["experts_in"],
                              L["experts_out"], e.top, self.cfg.act, e.count, workspace=self.moe_ws,
-                             groups=e.groups, keep=e.keep, limit=l.limit)
+                             groups=e.groups, keep=e.keep, limit=l.limit, **kw)
 
     def _parallel(self, ids: torch.Tensor, mix, rows: torch.Tensor | None, positions, kv,
                   **where) -> torch.Tensor:
@@ -395,6 +439,36 @@ class HybridLM:
         logits = ops.linear(x, self.lm_head)
         return ops.softcap_(logits, cfg.logit_softcap) if cfg.logit_softcap else logits
 
+    def _joint(self, ids: torch.Tensor, mix, rows: torch.Tensor | None) -> torch.Tensor:
+        """As _serial: one norm for both sublayers, one add, then the token's input to the layer."""
+        cfg, dt, eps, W = self.cfg, self.dtype, self.cfg.norm_eps, self.cfg.hidden_size
+        h = torch.empty((ids.shape[0], W), dtype=torch.float32, device=self.device)
+        z, zn, last = None, None, len(self.layers) - 1
+        for i, (l, L) in enumerate(zip(cfg.layers, self.layers)):
+            first = {"ids": ids, "embed": self.embed, "embed_scale": cfg.embed_scale} if i == 0 else {}
+            wide = ops.side_norm(h, L["norm1"].w, eps, z, zn, dtype=dt,
+                                 width=self._moe_width if l.experts else None, **first)
+            x, mw, off = wide[:, :W], L["mixer"].width, pad_to(L["mixer"].width)
+            a = torch.empty((ids.shape[0], L["out"].shape[1]), dtype=dt, device=self.device)
+            if off > mw:
+                a[:, mw:off].zero_()
+            mix(i, L["mixer"], x, a[:, :mw])
+            if i == last and rows is not None:
+                ids, h, a, wide = (t.index_select(0, rows) for t in (ids, h, a, wide))
+                x = wide[:, :W]
+            if "up" in L:
+                ops.squared_relu(x, L["up"], a[:, off:])
+            y = ops.linear(a, L["out"])
+            if l.experts:
+                x = self._experts(L, l, wide, stream=h, y=y)
+            else:
+                x = ops.stream_add(h, y)
+            z = zn = None
+            if cfg.side_dim:
+                g = ops.side_gate(ops.linear(x, L["side_gate"]), self.side_embed, ids, i)
+                z, zn = ops.linear(g, L["side_proj"]), L["side_norm"]
+        return ops.linear(ops.side_norm(h, self.final.w, eps, z, zn, dtype=dt), self.lm_head)
+
     def forward_prefill(self, ids: torch.Tensor, meta: PrefillMeta, kv) -> torch.Tensor:
         """Packed prompt portions, optionally with decode rows appended; logits of the rows in
         ``meta.last_idx``."""
@@ -403,8 +477,8 @@ class HybridLM:
         def mix(i, mixer, x, out=None):
             return mixer.prefill(x, meta, kv[i], out, carry)
 
-        if self.cfg.block == "serial":
-            return self._serial(ids, mix, meta.last_idx)
+        if self.cfg.block != "parallel":
+            return (self._joint if self.cfg.block == "joint" else self._serial)(ids, mix, meta.last_idx)
         step: HybridStep = meta.extra
         return self._parallel(ids, mix, meta.last_idx, meta.positions, kv, portions=step.portions,
                               tiles=step.conv_tiles)
@@ -417,8 +491,8 @@ class HybridLM:
         def mix(i, mixer, x, out=None):
             return mixer.decode(x, meta, kv[i], out, carry)
 
-        if self.cfg.block == "serial":
-            return self._serial(ids, mix, None)
+        if self.cfg.block != "parallel":
+            return (self._joint if self.cfg.block == "joint" else self._serial)(ids, mix, None)
         return self._parallel(ids, mix, None, meta.positions, kv, row_state=meta.state)
 
     # ------------------------------------------------------------ reference
@@ -493,6 +567,8 @@ class _RandomTensors:
             t = torch.randn(*shape, **kw) * (1.0 if leaf == "sink" else 0.05)
             if name.endswith(".mix.z.b"):  # gates from a few tokens to thousands
                 t = t * 40 - 3
+            elif name.endswith(".mix.f.b"):
+                t = t * 20 + 5
         elif leaf in ("uk", "uv", "a2", "g2"):
             t = torch.randn(*shape, **kw) * shape[1] ** -0.5
         elif leaf == "embed":

@@ -5,11 +5,13 @@ A mixer reads its (normed) input through ONE fused projection whose sections sta
 8 columns, and writes ``width`` columns - of a buffer of its own, or (``out``) of a wider operand -
 that the output projection ``o`` [hidden, width] consumes:
 
-  latent attention   [queries | latent, key part]
+  latent attention   [queries | latent, key part | head gates]
   delta rule         [q | k | v | beta | decay rank | gate rank]
   talking heads      [queries | keys | values], heads padded to multiples of 8
   gated average      [gate | candidate | read-out gate]
   grouped attention  [queries | keys | values | head gates], heads padded to multiples of 8
+  retention          [q | k | v | read-out gate]
+  matrix memory      [q | k | v | read-out gate | input gates | forget gates]
 
 ``carry``: a dict that lives as long as the step, for what layers hand to later ones.
 """
@@ -18,8 +20,8 @@ from __future__ import annotations
 import torch
 
 from .. import ops
-from .config import (ChannelDelta, GatedAverage, GroupedAttention, LatentAttention,
-                     TalkingAttention)
+from .config import (ChannelDelta, GatedAverage, GroupedAttention, LatentAttention, MatrixMemory,
+                     Retention, TalkingAttention)
 
 
 def pad_to(n: int, m: int = 8) -> int:
@@ -67,7 +69,7 @@ class Mixer:
             ts += [v] if isinstance(v, torch.Tensor) else \
                 [t for t in vars(v).values() if isinstance(t, torch.Tensor)] \
                 if isinstance(v, (ops.DeltaWeights, ops.TalkWeights, ops.AverageWeights,
-                                  ops.GroupedWeights)) else []
+                                  ops.GroupedWeights, ops.MemoryWeights)) else []
         return ts
 
     def _out(self, x, out) -> torch.Tensor:
@@ -78,10 +80,18 @@ class LatentMixer(Mixer):
     def __init__(self, m: LatentAttention, p: str, src, model):
         W, lin, f32 = model.cfg.hidden_size, model.lin, model.f32
         self.m, self.eps, self.rope = m, model.cfg.norm_eps, model.rope(m.rot_base, m.rot_dims)
-        w, offs = fused_rows([src.take(p + "q", m.heads * (m.dim + m.rot_dim), W),
-                              src.take(p + "dkv", m.kv_rank + m.rot_dim, W)])
-        self.proj, self.off_kv = lin(w), offs[1]
-        self.c_norm = f32(src.take(p + "dkv.norm", m.kv_rank))
+        # whose latents are read: this layer's own, or another's
+        self.source = int(p[1:p.index(".")]) if m.kv_from is None else m.kv_from
+        own = m.kv_from is None
+        sections = [src.take(p + "q", m.heads * (m.dim + m.rot_dim), W)]
+        if own:
+            sections.append(src.take(p + "dkv", m.kv_rank + m.rot_dim, W))
+        if m.gate:
+            sections.append(src.take(p + "g", m.heads, W))
+        w, offs = fused_rows(sections)
+        self.proj, self.off_kv = lin(w), offs[1] if own else None
+        self.off_g = offs[-1] if m.gate else None
+        self.c_norm = f32(src.take(p + "dkv.norm", m.kv_rank)) if own else None
         uk = src.take(p + "uk", m.heads * m.dim, m.kv_rank)
         uv = src.take(p + "uv", m.heads * m.vdim, m.kv_rank)
         w, offs = fused_rows([uk, uv])
@@ -97,6 +107,9 @@ class LatentMixer(Mixer):
     def operands(self):
         return [t for t in super().operands() if t is not self.uv and t is not self.rope]
 
+    def _gate(self, proj):
+        return None if self.off_g is None else proj[:, self.off_g:self.off_g + self.m.heads]
+
     def _decode(self, proj, positions, slots, cache, dm, out) -> None:
         """One token per row of ``proj``, in the latent space -> out [rows, heads * vdim]."""
         m = self.m
@@ -108,34 +121,46 @@ class LatentMixer(Mixer):
         ops.head_linear(proj[:, :m.heads * dq].unflatten(1, (m.heads, dq)), self.uk_t, out=qa)
         o = ops.latent_decode_attention(qa, cache, m.kv_rank, dm.block_tables, dm.context_lens,
                                         m.window, m.scale, self.sink,
-                                        dm.workspace[m.heads, m.kv_rank, m.window])
-        ops.head_linear(o, self.uv, out=out.view(B, m.heads, m.vdim))
+                                        dm.workspace[m.heads, m.kv_rank, m.window], self._gate(proj))
+        ops.head_linear(o, self.uv, out=out.unflatten(1, (m.heads, m.vdim)))
+
+    def _latents(self, proj, meta, cache, carry):
+        """Latent rows of the portions' keys; queries are rotated in place.  Layers that read the
+        same cache share them."""
+        m, step = self.m, meta.extra
+        keys, Tp = step.keys[m.window], meta.n_prefill
+        lat = proj.new_empty(Tp, cache.shape[-1]) if self.off_kv is not None else None
+        ops.latent_prep(proj[:Tp], self.off_kv, m.heads, m.dim, m.rot_dim, m.rot_dims, m.kv_rank,
+                        self.c_norm, self.eps, self.rope, meta.positions, meta.slots, cache, lat=lat)
+        if lat is not None:
+            carry["latents", self.source] = lat
+        if keys.slots is None:
+            return carry["latents", self.source]
+        if (self.source, m.window) not in carry:
+            carry[self.source, m.window] = ops.latent_gather(cache, keys.slots)
+        return carry[self.source, m.window]
 
     def prefill(self, x, meta, cache, out=None, carry=None):
         m, step = self.m, meta.extra
         proj = ops.linear(x, self.proj)
         R, Tp, T = x.shape[0], meta.n_prefill, step.q_host[-1]
-        a = x.new_empty(R, self.width)
-        lat = proj.new_empty(Tp, cache.shape[-1])
-        ops.latent_prep(proj[:Tp], self.off_kv, m.heads, m.dim, m.rot_dim, m.rot_dims, m.kv_rank,
-                        self.c_norm, self.eps, self.rope, meta.positions, meta.slots, cache, lat=lat)
-        keys = step.keys[m.window]
-        if keys.slots is not None:
-            lat = ops.latent_gather(cache, keys.slots)
+        a = self._out(x, out)
+        lat = self._latents(proj, meta, cache, carry)
         up = ops.linear(lat[:, :m.kv_rank], self.up)
         ops.latent_prefill_attention(proj, up, self.voff, lat, m.kv_rank, m.heads, m.dim,
-                                     m.rot_dim, m.vdim, step.q_cu, step.q_host, keys, step.tiles,
-                                     step.qtile, m.window, m.scale, self.sink, a)
+                                     m.rot_dim, m.vdim, step.q_cu, step.q_host, step.keys[m.window],
+                                     step.tiles, step.qtile, m.window, m.scale, self.sink, a,
+                                     self._gate(proj))
         if T < Tp:
             a[T:Tp].zero_()
         if Tp < R:
             self._decode(proj[Tp:], meta.positions[Tp:], meta.slots[Tp:], cache, meta.decode, a[Tp:])
-        return a if out is None else out.copy_(a)
+        return a
 
     def decode(self, x, meta, cache, out=None, carry=None):
-        a = x.new_empty(x.shape[0], self.width)
+        a = self._out(x, out)
         self._decode(ops.linear(x, self.proj), meta.positions, meta.slots, cache, meta, a)
-        return a if out is None else out.copy_(a)
+        return a
 
 
 class DeltaMixer(Mixer):
@@ -329,5 +354,59 @@ class GroupedMixer(Mixer):
         return a
 
 
-MIXERS = {LatentAttention: LatentMixer, ChannelDelta: DeltaMixer, TalkingAttention: TalkingMixer,
+class MemoryMixer(Mixer):
+    """Retention or matrix memory: a matrix state per head with one decay."""
+
+    def __init__(self, m: Retention | MatrixMemory, p: str, src, model):
+        W, lin, f32 = model.cfg.hidden_size, model.lin, model.f32
+        H, kd, vd = m.heads, m.heads * m.dim, m.heads * m.vdim
+        gated = isinstance(m, MatrixMemory)
+        sections = [src.take(p + x, n, W) for x, n in (("q", kd), ("k", kd), ("v", vd), ("g", vd))]
+        if gated:
+            sections += [src.take(p + x, H, W) for x in "if"]
+        w, offs = fused_rows(sections)
+        self.proj = lin(w)
+        kw = dict(heads=H, dim=m.dim, vdim=m.vdim, eps=model.cfg.norm_eps, off_k=offs[1], off_v=offs[2],
+                  off_g=offs[3])
+        if gated:
+            self.w = ops.MemoryWeights(
+                **kw, act="sigmoid", q_scale=m.dim ** -0.5, off_i=offs[4], off_f=offs[5],
+                i_bias=f32(src.take(p + "i.b", H)), f_bias=f32(src.take(p + "f.b", H)),
+                cap=m.gate_cap, norm=f32(src.take(p + "norm", vd)))
+        else:
+            self.w = ops.MemoryWeights(
+                **kw, act="silu", k_scale=m.dim ** -0.5, rot_dims=m.rot_dims,
+                rope=model.rope(m.rot_base, m.rot_dims) if m.rot_dims else None,
+                log_decay=f32(torch.tensor(m.decay, dtype=torch.float64).log()))
+        self.width = vd
+        self.o = lin(src.take(p + "o", W, vd))
+
+    def operands(self):
+        return [t for t in super().operands() if t is not self.w.rope]
+
+    @staticmethod
+    def _states(cache) -> tuple:
+        return cache if isinstance(cache, tuple) else (cache, None, None)
+
+    def prefill(self, x, meta, cache, out=None, carry=None):
+        step = meta.extra
+        a = self._out(x, out)
+        R, Tp, T = x.shape[0], meta.n_prefill, step.q_host[-1]
+        proj = ops.linear(x, self.proj)
+        ops.memory_scan(proj, self.w, self._states(cache), step.portions, a, len(step.q_host) - 1)
+        if T < Tp:
+            a[T:Tp].zero_()
+        if Tp < R:
+            ops.memory_decode(proj[Tp:], self.w, self._states(cache), meta.positions[Tp:],
+                              step.portions.row_state[Tp:], a[Tp:])
+        return a
+
+    def decode(self, x, meta, cache, out=None, carry=None):
+        a = self._out(x, out)
+        ops.memory_decode(ops.linear(x, self.proj), self.w, self._states(cache), meta.positions,
+                          meta.state, a)
+        return a
+
+
+MIXERS = {Retention: MemoryMixer, MatrixMemory: MemoryMixer, LatentAttention: LatentMixer, ChannelDelta: DeltaMixer, TalkingAttention: TalkingMixer,
           GatedAverage: AverageMixer, GroupedAttention: GroupedMixer}

@@ -10,7 +10,7 @@ import torch
 
 from ._ext import check, hipk, on_gpu, stream_ptr
 
-ACTS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
+ACTS = {"silu": 0, "gelu_tanh": 1, "clamped": 2, "relu2": 3}  # relu2: not gated (ops/moe.py)
 
 
 def act_glu_ref(gu: torch.Tensor, act: str = "silu", limit: float = 0.0) -> torch.Tensor:

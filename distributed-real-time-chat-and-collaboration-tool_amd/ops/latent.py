@@ -60,31 +60,33 @@ def rotate_pairs_ref(x: torch.Tensor, cs: torch.Tensor, dims: int) -> torch.Tens
 
 
 # ------------------------------------------------------------------ per-token preparation
-def latent_prep(proj: torch.Tensor, off_kv: int, heads: int, dim: int, rot_dim: int,
-                rot_dims: int, kv_rank: int, norm_w: torch.Tensor, eps: float,
+def latent_prep(proj: torch.Tensor, off_kv: int | None, heads: int, dim: int, rot_dim: int,
+                rot_dims: int, kv_rank: int, norm_w: torch.Tensor | None, eps: float,
                 cos_sin: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor | None,
                 cache: torch.Tensor | None, lat: torch.Tensor | None = None,
                 qa: torch.Tensor | None = None) -> None:
     """Rows of the fused projection [queries | latent, key part]: RMS-norm the latent, rotate
     the key part, write both to ``lat`` [rows, LW] and to the cache rows ``slots`` (-1: none).
     The queries' rotated parts go to ``qa`` [rows, heads, LW] at column kv_rank (zeros
-    behind), or are rotated in place."""
+    behind), or are rotated in place.  ``off_kv`` None: queries only."""
     rows = proj.shape[0]
+    own = off_kv is not None
     LW = (cache if cache is not None else lat if lat is not None else qa).shape[-1]
     dq = dim + rot_dim
     if not on_gpu(proj):
-        kv = proj[:, off_kv:off_kv + kv_rank + rot_dim]
         cs = cos_sin[positions[:rows].long()]
-        cf = kv[:, :kv_rank].float()
-        c = cf * torch.rsqrt(cf.pow(2).mean(-1, keepdim=True) + eps) * norm_w
-        full = proj.new_zeros(rows, LW)
-        full[:, :kv_rank] = c.to(proj.dtype)
-        full[:, kv_rank:kv_rank + rot_dim] = rotate_pairs_ref(kv[:, kv_rank:], cs, rot_dims)
-        if lat is not None:
-            lat.copy_(full)
-        if cache is not None and slots is not None:
-            ok = slots[:rows] >= 0
-            cache.view(-1, LW)[slots[:rows][ok]] = full[ok]
+        if own:
+            kv = proj[:, off_kv:off_kv + kv_rank + rot_dim]
+            cf = kv[:, :kv_rank].float()
+            c = cf * torch.rsqrt(cf.pow(2).mean(-1, keepdim=True) + eps) * norm_w
+            full = proj.new_zeros(rows, LW)
+            full[:, :kv_rank] = c.to(proj.dtype)
+            full[:, kv_rank:kv_rank + rot_dim] = rotate_pairs_ref(kv[:, kv_rank:], cs, rot_dims)
+            if lat is not None:
+                lat.copy_(full)
+            if cache is not None and slots is not None:
+                ok = slots[:rows] >= 0
+                cache.view(-1, LW)[slots[:rows][ok]] = full[ok]
         q = proj[:, :heads * dq].unflatten(1, (heads, dq))
         r = rotate_pairs_ref(q[..., dim:], cs, rot_dims)
         if qa is not None:
@@ -93,11 +95,13 @@ def latent_prep(proj: torch.Tensor, off_kv: int, heads: int, dim: int, rot_dim: 
         else:
             q[..., dim:] = r
         return
-    assert proj.dim() == 2 and proj.stride(1) == 1 and off_kv + kv_rank + rot_dim <= proj.shape[1]
-    assert heads * dq <= off_kv
+    assert proj.dim() == 2 and proj.stride(1) == 1
+    assert heads * dq <= (off_kv if own else proj.shape[1])
+    assert not own or off_kv + kv_rank + rot_dim <= proj.shape[1]
     assert positions.dtype == torch.int32 and positions.numel() >= rows
     assert cos_sin.dtype == torch.float32 and cos_sin.shape[1] == rot_dims
-    assert cos_sin.is_contiguous() and norm_w.dtype == torch.float32 and norm_w.numel() == kv_rank
+    assert cos_sin.is_contiguous()
+    assert not own or (norm_w.dtype == torch.float32 and norm_w.numel() == kv_rank)
     for t in (lat, cache, qa):
         assert t is None or (t.is_contiguous() and t.shape[-1] == LW and t.dtype == proj.dtype)
     assert lat is None or lat.shape[0] == rows
@@ -105,8 +109,8 @@ def latent_prep(proj: torch.Tensor, off_kv: int, heads: int, dim: int, rot_dim: 
     if cache is not None:
         assert slots is not None and slots.dtype == torch.int64 and slots.numel() >= rows
     check(hipk().latent_prep(int(proj.dtype == torch.float32), dict(
-        proj=proj.data_ptr(), ldp=proj.stride(0), off_kv=off_kv, H=heads, dim=dim, rot=rot_dim,
-        rot_dims=rot_dims, R=kv_rank, LW=LW, norm_w=norm_w.data_ptr(), eps=float(eps),
+        proj=proj.data_ptr(), ldp=proj.stride(0), off_kv=off_kv if own else -1, H=heads, dim=dim,
+        rot=rot_dim, rot_dims=rot_dims, R=kv_rank, LW=LW, norm_w=ptr(norm_w), eps=float(eps),
         cos_sin=cos_sin.data_ptr(), positions=positions.data_ptr(), slots=ptr(slots),
         lat=ptr(lat), cache=ptr(cache), qa=ptr(qa), rows=rows), stream_ptr(proj)), "latent_prep")
 
@@ -169,13 +173,15 @@ def latent_prefill_attention(q: torch.Tensor, kv: torch.Tensor, voff: int, lat: 
                              kv_rank: int, heads: int, dim: int, rot_dim: int, vdim: int,
                              q_cu: torch.Tensor, q_host: list, keys: PortionKeys,
                              tiles: tuple, qtile: int, window: int | None, scale: float,
-                             sink: torch.Tensor | None, out: torch.Tensor) -> torch.Tensor:
+                             sink: torch.Tensor | None, out: torch.Tensor,
+                             gate: torch.Tensor | None = None) -> torch.Tensor:
     """Causal windowed attention of packed prompt portions.  q rows: heads of [dim | rotated];
     kv rows: per-head keys [heads * dim], values from column ``voff``; lat rows: the shared
-    rotated key part from column kv_rank.  Writes out[:q_host[-1]] ([rows, heads * vdim])."""
+    rotated key part from column kv_rank.  ``gate`` [rows, heads]: outputs times its sigmoid.
+    Writes out[:q_host[-1]] ([rows, heads * vdim])."""
     if not on_gpu(q):
         return _latent_prefill_ref(q, kv, voff, lat, kv_rank, heads, dim, rot_dim, vdim, q_host,
-                                   keys, window, scale, sink, out)
+                                   keys, window, scale, sink, out, gate)
     n = len(q_host) - 1
     for t in (q, kv, lat, out):
         assert t.stride(1) == 1 and t.dtype == q.dtype and t.is_cuda
@@ -184,6 +190,7 @@ def latent_prefill_attention(q: torch.Tensor, kv: torch.Tensor, voff: int, lat: 
     assert kv.shape[1] >= voff + heads * vdim and out.shape[1] >= heads * vdim
     assert q.shape[1] >= heads * (dim + rot_dim) and lat.stride(0) == lat.shape[1]
     assert sink is None or (sink.dtype == torch.float32 and sink.numel() == heads)
+    _check_gate(gate, q, q_host[-1], heads)
     for t in (q_cu, keys.k_cu, keys.ctx, *tiles):
         assert t.dtype == torch.int32 and t.is_cuda
     assert q_cu.numel() == n + 1 and keys.k_cu.numel() == n + 1 and keys.ctx.numel() == n
@@ -193,8 +200,14 @@ def latent_prefill_attention(q: torch.Tensor, kv: torch.Tensor, voff: int, lat: 
         dim=dim, rot=rot_dim, vdim=vdim, q_cu=q_cu.data_ptr(), k_cu=keys.k_cu.data_ptr(),
         ctx=keys.ctx.data_ptr(), tile_seq=tiles[0].data_ptr(), tile_q0=tiles[1].data_ptr(),
         ntiles=tiles[0].numel(), qtile=qtile, nseq=n, nq=q_host[-1], window=window or 0,
-        scale=float(scale), sink=ptr(sink)), stream_ptr(q)), "latent_prefill")
+        scale=float(scale), sink=ptr(sink), gate=ptr(gate),
+        ldg=gate.stride(0) if gate is not None else 0), stream_ptr(q)), "latent_prefill")
     return out
+
+
+def _check_gate(gate, x, rows: int, heads: int) -> None:
+    assert gate is None or (gate.dtype == x.dtype and gate.stride(1) == 1 and gate.is_cuda
+                            and gate.shape[0] >= rows and gate.shape[1] == heads)
 
 
 def _sink_softmax_ref(sc: torch.Tensor, sink: torch.Tensor | None) -> torch.Tensor:
@@ -206,7 +219,7 @@ def _sink_softmax_ref(sc: torch.Tensor, sink: torch.Tensor | None) -> torch.Tens
 
 
 def _latent_prefill_ref(q, kv, voff, lat, kv_rank, heads, dim, rot_dim, vdim, q_host, keys,
-                        window, scale, sink, out):
+                        window, scale, sink, out, gate=None):
     dq = dim + rot_dim
     for s, ctx in enumerate(keys.ctx_host):
         a, b = q_host[s], q_host[s + 1]
@@ -220,7 +233,10 @@ def _latent_prefill_ref(q, kv, voff, lat, kv_rank, heads, dim, rot_dim, vdim, q_
         d = (torch.arange(b - a)[:, None] + ctx) - torch.arange(k1 - k0)[None, :]
         hide = d < 0 if window is None else (d < 0) | (d >= window)
         p = _sink_softmax_ref(sc.masked_fill(hide.to(sc.device), float("-inf")), sink)
-        out[a:b, :heads * vdim] = torch.einsum("hij,jhv->ihv", p, v).flatten(1).to(out.dtype)
+        o = torch.einsum("hij,jhv->ihv", p, v)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[a:b].float())[..., None]
+        out[a:b, :heads * vdim] = o.flatten(1).to(out.dtype)
     return out
 
 
@@ -253,10 +269,11 @@ class LatentDecodeWorkspace:
 def latent_decode_attention(qa: torch.Tensor, cache: torch.Tensor, kv_rank: int,
                             block_tables: torch.Tensor, context_lens: torch.Tensor,
                             window: int | None, scale: float, sink: torch.Tensor | None,
-                            workspace: LatentDecodeWorkspace | None = None) -> torch.Tensor:
+                            workspace: LatentDecodeWorkspace | None = None,
+                            gate: torch.Tensor | None = None) -> torch.Tensor:
     """One query per sequence in the latent space, qa [B, heads, LW], against the cache rows of
     its last ``window`` tokens (its own included: context_lens counts it).  Rows with context 0
-    give zeros.  Returns [B, heads, kv_rank]."""
+    give zeros.  ``gate`` [B, heads]: results times its sigmoid.  Returns [B, heads, kv_rank]."""
     B, H, LW = qa.shape
     if not on_gpu(qa):
         out = qa.new_zeros(B, H, kv_rank)
@@ -268,13 +285,17 @@ def latent_decode_attention(qa: torch.Tensor, cache: torch.Tensor, kv_rank: int,
             j = torch.arange(0 if window is None else max(0, n - window), n, device=qa.device)
             rows = flat[block_tables[b].long()[j // KV_BLOCK] * KV_BLOCK + j % KV_BLOCK].float()
             p = _sink_softmax_ref(qa[b].float() @ rows.T * scale, sink)
-            out[b] = (p @ rows[:, :kv_rank]).to(out.dtype)
+            o = p @ rows[:, :kv_rank]
+            if gate is not None:
+                o = o * torch.sigmoid(gate[b].float())[:, None]
+            out[b] = o.to(out.dtype)
         return out
     assert qa.is_contiguous() and cache.is_contiguous() and cache.shape[1:] == (KV_BLOCK, LW)
     assert cache.dtype == qa.dtype and block_tables.dtype == torch.int32
     assert block_tables.stride(1) == 1 and block_tables.shape[0] >= B
     assert context_lens.dtype == torch.int32 and context_lens.numel() >= B
     assert sink is None or (sink.dtype == torch.float32 and sink.numel() == H)
+    _check_gate(gate, qa, B, H)
     ws = workspace or LatentDecodeWorkspace(B, H, kv_rank, window, block_tables.shape[1], qa.device)
     assert ws.splits == 1 or (ws.part_o is not None and ws.part_o.shape[:2] == (B, H)
                               and ws.part_o.shape[3] == kv_rank)
@@ -284,7 +305,8 @@ def latent_decode_attention(qa: torch.Tensor, cache: torch.Tensor, kv_rank: int,
         cache=cache.data_ptr(), block_tables=block_tables.data_ptr(),
         bt_stride=block_tables.stride(0), context_lens=context_lens.data_ptr(), B=B, H=H,
         R=kv_rank, LW=LW, window=window or 0, tiles_per_split=ws.per, nsplits=ws.splits,
-        scale=float(scale), sink=ptr(sink)), stream_ptr(qa)), "latent_decode")
+        scale=float(scale), sink=ptr(sink), gate=ptr(gate),
+        ldg=gate.stride(0) if gate is not None else 0), stream_ptr(qa)), "latent_decode")
     return out
 
 

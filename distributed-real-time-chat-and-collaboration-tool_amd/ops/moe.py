@@ -59,7 +59,8 @@ def route_ref(router_logits: torch.Tensor, top_k: int, groups: int = 1, keep: in
 
 def fused_moe_ref(x: torch.Tensor, router_logits: torch.Tensor, w_gu: torch.Tensor,
                   w_dn: torch.Tensor, top_k: int, act: str = "silu", e_off: int = 0,
-                  groups: int = 1, keep: int = 1, limit: float = 0.0) -> torch.Tensor:
+                  groups: int = 1, keep: int = 1, limit: float = 0.0, stream: torch.Tensor | None = None,
+                  y: torch.Tensor | None = None) -> torch.Tensor:
     """fp32-accumulated PyTorch reference of :func:`fused_moe`."""
     topi, wts = route_ref(router_logits, top_k, groups, keep)
     out = torch.zeros(x.shape[0], x.shape[1], dtype=torch.float32, device=x.device)
@@ -68,9 +69,14 @@ def fused_moe_ref(x: torch.Tensor, router_logits: torch.Tensor, w_gu: torch.Tens
         if tok.numel() == 0:
             continue
         xe = x.index_select(0, tok).float()
-        h = act_glu_ref(xe @ w_gu[le].float().t(), act, limit).to(x.dtype).float()
+        h = xe @ w_gu[le].float().t()
+        h = h.relu().square() if act == "relu2" else act_glu_ref(h, act, limit)
+        h = h.to(x.dtype).float()
         ye = (h @ w_dn[le].float().t()).to(x.dtype).float()
         out.index_add_(0, tok, ye * wts[tok, slot].unsqueeze(1))
+    if stream is not None:
+        stream += out[:, :stream.shape[1]] + y.float()
+        return stream.to(x.dtype)
     return out.to(x.dtype)
 
 
@@ -145,16 +151,23 @@ def fused_moe(x: torch.Tensor, router_logits: torch.Tensor, w_gu: torch.Tensor,
               e_off: int = 0, workspace: torch.Tensor | None = None,
               out: torch.Tensor | None = None, variant: int | None = None,
               gu_form: int | None = None, dn_form: int | None = None, groups: int = 1,
-              keep: int = 1, limit: float = 0.0) -> torch.Tensor:
-    """y[t] = sum_j w[t,j] * down_e(act(gate_e x_t) * up_e x_t) over the top-k experts.
+              keep: int = 1, limit: float = 0.0, stream: torch.Tensor | None = None,
+              y: torch.Tensor | None = None) -> torch.Tensor:
+    """y[t] = sum_j w[t,j] * down_e(act(gate_e x_t) * up_e x_t) over the top-k experts; act
+    "relu2": down_e(relu(up_e x_t)^2), w_gu [E_local, I, H].
+
+    ``stream`` [T, W <= H] fp32: the result is added to it together with ``y`` [T, W], and the
+    stream is returned in x's type (itself in fp32).
 
     x [T, H] bf16 (H % 128 == 0, I % 64 == 0) or fp32 (any size); router_logits [T, E] bf16 or
     fp32, row-major or the transposed view of an [E, T] tensor (``router_logits(...,
-    contiguous=False)``); w_gu [E_local, 2I, H] ([gate | up] rows); w_dn [E_local, H, I].
+    contiguous=False)``); w_gu [E_local, 2I, H] ([gate | up] rows); w_dn [E_local, H, I] ("relu2"
+    in bf16: I % 128 == 0).
     ``groups`` / ``keep``: group-limited choice; ``limit``: bound of the clamped activation.
     """
     if not on_gpu(x):
-        r = fused_moe_ref(x, router_logits, w_gu, w_dn, top_k, act, e_off, groups, keep, limit)
+        r = fused_moe_ref(x, router_logits, w_gu, w_dn, top_k, act, e_off, groups, keep, limit,
+                          stream, y)
         if out is not None:
             out.copy_(r)
             return out
@@ -164,8 +177,8 @@ def fused_moe(x: torch.Tensor, router_logits: torch.Tensor, w_gu: torch.Tensor,
     # the round-4 per-expert hipBLASLt path for T >= 4096 measured slower at T = 8192,
     # 6.05 / 5.86 ms fused vs 6.25 / 5.95 ms, profiles/r4ah, r4ak)
     E = num_experts if num_experts is not None else router_logits.shape[1]
-    e_local, two_i, h2 = w_gu.shape
-    inter = two_i // 2
+    e_local, n_in, h2 = w_gu.shape
+    inter = n_in if act == "relu2" else n_in // 2
     f32 = x.dtype == torch.float32
     assert x.dtype == w_gu.dtype == w_dn.dtype and x.is_contiguous()
     assert f32 or x.dtype == torch.bfloat16
@@ -175,12 +188,19 @@ def fused_moe(x: torch.Tensor, router_logits: torch.Tensor, w_gu: torch.Tensor,
     assert (lts, les) == (E, 1) or (lts == 1 and les >= T), router_logits.stride()
     assert w_gu.is_contiguous() and w_dn.is_contiguous() and w_dn.shape == (e_local, H, inter)
     assert E <= 256 and 1 <= top_k <= min(MAX_TOP_K, E)
-    assert f32 or (H % 128 == 0 and inter % 64 == 0)
+    assert f32 or (H % 128 == 0 and inter % (128 if act == "relu2" else 64) == 0)
     assert 1 <= groups <= MAX_GROUPS and E % groups == 0 and 1 <= keep <= groups
     assert top_k <= keep * (E // groups)
-    if out is None:
+    W = H
+    if stream is not None:
+        W = stream.shape[1]
+        assert stream.shape == y.shape == (T, W) and W <= H and stream.is_contiguous()
+        assert stream.dtype == torch.float32 and y.dtype == x.dtype and y.stride(1) == 1
+        assert out is None and (e_off, e_local) == (0, E)
+        out = stream if f32 else x.new_empty(T, W)
+    elif out is None:
         out = torch.empty_like(x)
-    assert out.is_contiguous() and out.shape == x.shape
+    assert out.is_contiguous() and out.shape == (T, W)
     chunk = min(T, MOE_CHUNK) if T else 1
     need = workspace_bytes(chunk, H, inter, e_local, top_k, f32)
     if workspace is None or workspace.numel() < need:
@@ -207,7 +227,9 @@ def fused_moe(x: torch.Tensor, router_logits: torch.Tensor, w_gu: torch.Tensor,
                       slab.numel() * 4 if slab is not None else 0,
                       cnt.data_ptr() if cnt is not None else 0,
                       cnt.numel() if cnt is not None else 0, lts, les, int(f32),
-                      int(router_logits.dtype == torch.float32), groups, keep, float(limit), st),
-              "moe")
+                      int(router_logits.dtype == torch.float32), groups, keep, float(limit),
+                      0 if stream is None else stream[t0].data_ptr(),
+                      0 if stream is None else y[t0].data_ptr(),
+                      0 if stream is None else y.stride(0), W, st), "moe")
     return out
 

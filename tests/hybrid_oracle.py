@@ -6,6 +6,8 @@ no cache, no batching, no code shared with the package.  The tests compare the f
              norms, convolved sublayer inputs
   Nurilorn   attention with convolved projections, scaled rotation, capped scores, value mixing and
              head gates; clamped feed-forwards and routed experts, norms in groups, layer scales
+  Garesun    retention, matrix memory (mLSTM) and latent attention whose latents several layers may
+             share, beside squared-relu experts under one layer norm; per-layer token inputs
 
 Weights are a dict name -> tensor under the checkpoint's names, the configuration is the
 checkpoint's config.json as a dict.  Everything is computed in ``DT`` (float64 by default).
@@ -76,21 +78,39 @@ def sink_softmax(scores, ok, sink):
     return e / den
 
 
-def latent_attention(h, W, m, eps):
-    """h [n, width] -> [n, width]; W: this mixer's tensors without their prefix."""
-    n, H = h.shape[0], m["heads"]
-    d, r, dv, R = m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
-    pos = torch.arange(n)
-    q = (h @ W["q"].T).reshape(n, H, d + r)
-    qn, qr = q[..., :d], rotate_interleaved(q[..., d:], pos, m["rot"]["base"], m["rot"]["dims"])
+def latent_rows(h, W, m, eps):
+    """What a token leaves for later ones: its normed latent, the rotated key part of all heads."""
+    R = m["kv_rank"]
     kv = h @ W["dkv"].T
-    c = rms(kv[:, :R], eps) * W["dkv.norm"]
-    kr = rotate_interleaved(kv[:, R:], pos, m["rot"]["base"], m["rot"]["dims"])
+    return rms(kv[:, :R], eps) * W["dkv.norm"], \
+        rotate_interleaved(kv[:, R:], torch.arange(h.shape[0]), m["rot"]["base"], m["rot"]["dims"])
+
+
+def latent_read(h, W, m, rows, size, sink):
+    """Every head's output [n, H, vdim] over ``rows``."""
+    n, H = h.shape[0], m["heads"]
+    d, r, dv = m["dim"], m["rot_dim"], m["vdim"]
+    c, kr = rows
+    q = (h @ W["q"].T).reshape(n, H, d + r)
+    qn, qr = q[..., :d], rotate_interleaved(q[..., d:], torch.arange(n), m["rot"]["base"], m["rot"]["dims"])
     kn = (c @ W["uk"].T).reshape(n, H, d)
     v = (c @ W["uv"].T).reshape(n, H, dv)
     sc = (torch.einsum("ihd,jhd->hij", qn, kn) + torch.einsum("ihr,jr->hij", qr, kr)) * m["scale"]
-    p = sink_softmax(sc, window_mask(n, m["mask"]["size"]), W["sink"])
-    return torch.einsum("hij,jhv->ihv", p, v).reshape(n, H * dv) @ W["o"].T
+    p = sink_softmax(sc, window_mask(n, size), sink)
+    return torch.einsum("hij,jhv->ihv", p, v)
+
+
+def latent_attention(h, W, m, eps):
+    """h [n, width] -> [n, width]; W: this mixer's tensors without their prefix."""
+    o = latent_read(h, W, m, latent_rows(h, W, m, eps), m["mask"]["size"], W["sink"])
+    return o.flatten(1) @ W["o"].T
+
+
+def gated_latent_attention(h, W, m, eps, held):
+    """Without window and sink, a sigmoid gate per head; ``held``: another layer's rows, or None."""
+    rows = latent_rows(h, W, m, eps) if held is None else held
+    o = latent_read(h, W, m, rows, None, None) * torch.sigmoid(h @ W["g"].T)[:, :, None]
+    return o.flatten(1) @ W["o"].T, rows
 
 
 def causal_conv(x, w):
@@ -294,6 +314,84 @@ def experts(h, W, mlp):
                for e in range(w.shape[1]))
 
 
+def rotate_halves(x, positions, base, dims):
+    """x [T, heads, D]: components i and i + dims / 2 turned by position * base^(-2i / dims)."""
+    half = dims // 2
+    i = torch.arange(half, dtype=x.dtype)
+    a = positions.to(x.dtype)[:, None, None] * base ** (-2 * i / max(dims, 1))
+    u, v = x[..., :half], x[..., half:dims]
+    return torch.cat([u * torch.cos(a) - v * torch.sin(a), v * torch.cos(a) + u * torch.sin(a), x[..., dims:]], -1)
+
+
+def retention_scan(q, k, v, decay, S=None):
+    """S <- decay S + k v^T, o = S^T q; q, k [n, H, d], v [n, H, dv], decay [H]."""
+    S = q.new_zeros(q.shape[1], q.shape[2], v.shape[2]) if S is None else S
+    out = []
+    for t in range(q.shape[0]):
+        S = decay[:, None, None] * S + k[t][:, :, None] * v[t][:, None, :]
+        out.append(torch.einsum("hdv,hd->hv", S, q[t]))
+    return torch.stack(out), S
+
+
+def retention(h, W, m, eps):
+    n, H, d, dv = h.shape[0], m["heads"], m["dim"], m["vdim"]
+    pos, rot = torch.arange(n), m.get("rot") or {"base": 1.0, "dims": 0}
+    q = rotate_halves((h @ W["q"].T).reshape(n, H, d), pos, rot["base"], rot["dims"])
+    k = rotate_halves((h @ W["k"].T).reshape(n, H, d), pos, rot["base"], rot["dims"]) * d ** -0.5
+    o, _ = retention_scan(q, k, (h @ W["v"].T).reshape(n, H, dv), torch.tensor(m["decay"], dtype=h.dtype))
+    return (rms(o, eps).reshape(n, H * dv) * silu(h @ W["g"].T)) @ W["o"].T
+
+
+def memory_scan(q, k, v, i, f, state=None):
+    """Matrix memory with log gates i, f [n, H] and a running maximum from 0 -> every read-out, the
+    state (S, normaliser, maximum)."""
+    H, d, dv = q.shape[1], q.shape[2], v.shape[2]
+    S, N, top = state or (q.new_zeros(H, d, dv), q.new_zeros(H, d), q.new_zeros(H))
+    out = []
+    for t in range(q.shape[0]):
+        new = torch.maximum(f[t] + top, i[t])
+        keep, put = torch.exp(f[t] + top - new), torch.exp(i[t] - new)
+        S = keep[:, None, None] * S + put[:, None, None] * k[t][:, :, None] * v[t][:, None, :]
+        N = keep[:, None] * N + put[:, None] * k[t]
+        top = new
+        den = torch.maximum((N * q[t]).sum(-1).abs(), torch.exp(-top)) + 1e-6
+        out.append(torch.einsum("hdv,hd->hv", S, q[t]) / den[:, None])
+    return torch.stack(out), (S, N, top)
+
+
+def memory_gates(h, W, cap):
+    """Log input gate, log forget gate."""
+    i, f = (cap * torch.tanh((h @ W[x].T + W[x + ".b"]) / cap) for x in "if")
+    return i, -torch.logaddexp(-f, torch.zeros_like(f))
+
+
+def mlstm(h, W, m, eps):
+    n, H, d, dv = h.shape[0], m["heads"], m["dim"], m["vdim"]
+    q = (h @ W["q"].T).reshape(n, H, d) * d ** -0.5
+    o, _ = memory_scan(q, (h @ W["k"].T).reshape(n, H, d), (h @ W["v"].T).reshape(n, H, dv),
+                       *memory_gates(h, W, m["gate_cap"]))
+    return (rms(o, eps).reshape(n, H * dv) * W["norm"] * torch.sigmoid(h @ W["g"].T)) @ W["o"].T
+
+
+def relu2_experts(h, W, mlp):
+    """Squared-relu experts: softmax over the chosen logits; a shared one for every token."""
+    z = h @ W["router"].T
+    top = z.topk(mlp["router"]["top"], -1)
+    w = torch.zeros_like(z).scatter(1, top.indices, torch.softmax(top.values, -1))
+
+    def sub(p):
+        return {x: W[p + x] for x in ("up", "down")}
+
+    y = sum(w[:, e:e + 1] * relu2_mlp(h, sub(f"e{e}.")) for e in range(z.shape[1]))
+    return y + relu2_mlp(h, sub("shared.")) if mlp.get("shared") else y
+
+
+def token_side(x, e, W, eps):
+    """A token's own input to a layer, gated by the stream: what is added to it."""
+    y = (gelu_tanh(x @ W["gate"].T) * e) @ W["proj"].T
+    return rms(y, eps) * W["norm"]
+
+
 # ------------------------------------------------------------------ the models
 MIXERS = {"latent_attention": latent_attention, "channel_delta": channel_delta,
           "attention": talking_attention, "mingru": mingru}
@@ -304,6 +402,8 @@ def forward(cfg, weights, tokens, margins=None):
     list that takes every routed layer's ``route_margin``."""
     if cfg["architecture"] == "Nurilorn":
         return _nurilorn(cfg, weights, tokens, margins)
+    if cfg["architecture"] == "Garesun":
+        return _garesun(cfg, weights, tokens, margins)
     return {"Ralesun": _ralesun, "Mebalorn": _mebalorn}[cfg["architecture"]](cfg, weights, tokens)
 
 
@@ -334,6 +434,33 @@ def _nurilorn(cfg, weights, tokens, margins=None):
             x = x + mult * (y * W[p + "ls2"])
         stream.append(x)
     return norm("final.norm", x) @ W["head"].T * cfg["logit_scale"], torch.stack(stream)
+
+
+def _garesun(cfg, weights, tokens, margins=None):
+    W = {k: t.to(DT) for k, t in weights.items()}
+    eps, dim = cfg["norm"]["eps"], cfg["token_side"]["dim"]
+    toks = torch.as_tensor(list(tokens), dtype=torch.long)
+
+    def sub(prefix):
+        return {k[len(prefix):]: t for k, t in W.items() if k.startswith(prefix)}
+
+    x = W["embed"][toks] * cfg["embedding"]["scale"]
+    stream, rows = [], {}
+    for i, layer in enumerate(cfg["layers"]):
+        m, mix = layer["mixer"], sub(f"l{i}.mix.")
+        h = layer_norm(x, W[f"l{i}.norm1"], 0.0, eps)
+        if layer["type"] == "latent_attention":
+            y, rows[i] = gated_latent_attention(h, mix, m, eps, rows.get(m.get("kv_from")))
+        else:
+            y = {"retention": retention, "mlstm": mlstm}[layer["type"]](h, mix, m, eps)
+        if layer["mlp"] is not None:
+            if margins is not None:
+                margins.append(route_margin(h, W[f"l{i}.mlp.router"], layer["mlp"]["router"]))
+            y = y + relu2_experts(h, sub(f"l{i}.mlp."), layer["mlp"])
+        x = x + y
+        x = x + token_side(x, W["side.embed"][toks, i * dim:(i + 1) * dim], sub(f"l{i}.side."), eps)
+        stream.append(x)
+    return layer_norm(x, W["final.norm"], 0.0, eps) @ W["head"].T, torch.stack(stream)
 
 
 def _mebalorn(cfg, weights, tokens):
