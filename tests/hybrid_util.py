@@ -55,6 +55,38 @@ def scaled(vocab, width, *layers, eps=1e-5, groups=2, embed=3.0, mult=0.8, logit
             "embedding": {"scale": embed}, "residual_mult": mult, "logit_scale": logits, "layers": list(layers)}
 
 
+def _moe(ff, experts, top, shared):
+    if not ff:
+        return None
+    out = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    return {**out, "shared": {"ff": shared}} if shared else out
+
+
+def retention(heads, dim, vdim, rot=0, decay=None, base=10000.0, ff=None, experts=6, top=2, shared=None):
+    decay = decay or [1 - 2.0 ** (-1 - 7 * h / heads) for h in range(heads)]
+    return {"type": "retention", "mlp": _moe(ff, experts, top, shared),
+            "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": decay, "rot": {"base": base, "dims": rot}}}
+
+
+def mlstm(heads, dim, vdim, cap=9.0, ff=None, experts=6, top=2, shared=None):
+    return {"type": "mlstm", "mlp": _moe(ff, experts, top, shared),
+            "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "gate_cap": cap}}
+
+
+def gated_latent(heads, dim, rot, vdim, rank, kv_from=None, base=10000.0, scale=None, ff=None, experts=6, top=2,
+                 shared=None):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": rank,
+         "scale": scale or (dim + rot) ** -0.5, "rot": {"base": base, "dims": rot}}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "latent_attention", "mlp": _moe(ff, experts, top, shared), "mixer": m}
+
+
+def joint(vocab, width, *layers, eps=1e-5, embed=2.0, side=16):
+    return {"architecture": "Garesun", "vocab": vocab, "width": width, "norm": {"eps": eps},
+            "embedding": {"scale": embed}, "token_side": {"dim": side}, "layers": list(layers)}
+
+
 def parallel(vocab, width, *layers, eps=1e-5, taps=3, cap=12.0):
     return {"architecture": "Mebalorn", "vocab": vocab, "width": width, "norm": {"eps": eps},
             "canon": {"taps": taps}, "logit_softcap": cap, "layers": list(layers)}
@@ -120,6 +152,32 @@ CONFIGS = {
                            grouped(16, 8, 64, 64, 64, ff=256, experts=4, top=2, limit=1.0),
                            grouped(16, 4, 128, 128, 128, conv=4, ff=128, experts=16, top=4, groups=(4, 2), v_mix=False),
                            groups=4),
+    # --- one norm for mixer and experts, token inputs: every mixer with and without experts and shared
+    # experts, latents read by two layers and a second set of them
+    "memory": joint(320, 192, mlstm(2, 32, 48, ff=40, shared=72),
+                    gated_latent(5, 24, 8, 40, 48, base=500.0, ff=64, experts=5, top=3),
+                    retention(3, 48, 32, 32),
+                    gated_latent(3, 16, 8, 24, 48, kv_from=1, base=500.0, scale=0.25, ff=24, experts=4, top=2, shared=40),
+                    gated_latent(4, 32, 8, 32, 48, base=500.0),
+                    retention(2, 64, 72, 64, base=300.0, ff=32, experts=4, top=4),
+                    gated_latent(2, 24, 8, 56, 48, kv_from=4, base=500.0),
+                    gated_latent(6, 8, 8, 16, 48, kv_from=1, base=500.0, ff=48, experts=4, shared=16),
+                    mlstm(3, 16, 40, cap=4.0), side=24),
+    # the largest heads of the chunk kernel, columns over several workgroups, a rotation of a part
+    "memory-wide": joint(256, 512, mlstm(4, 128, 128, ff=128, experts=4), retention(2, 256, 200, 128, ff=72, experts=3, shared=64),
+                         gated_latent(20, 64, 32, 64, 160), mlstm(1, 144, 320, cap=15.0),
+                         gated_latent(17, 128, 32, 96, 160, kv_from=2, ff=64, experts=12, top=11),
+                         retention(1, 96, 400, 96), mlstm(2, 256, 256, cap=30.0), embed=1.0, side=64),
+    # sizes no vector path takes
+    "memory-odd": joint(203, 100, mlstm(3, 20, 17, ff=17, experts=3, top=3), retention(2, 12, 15, 6, ff=9, shared=11),
+                        gated_latent(2, 12, 6, 20, 52), gated_latent(3, 10, 6, 9, 52, kv_from=2, ff=21, experts=5),
+                        retention(3, 7, 30, 0, decay=[1.0, 0.2, 0.97]), mlstm(1, 130, 261, cap=5.0), side=19),
+    # projections and experts wide enough for the prefill GEMM tiles
+    "memory-tiles": joint(256, 256, mlstm(8, 64, 64, ff=256, experts=4, shared=256), gated_latent(16, 64, 64, 64, 192),
+                          retention(8, 128, 128, 128, ff=128, experts=8, top=4, shared=512),
+                          gated_latent(8, 128, 64, 128, 192, kv_from=1, ff=256, experts=4), side=32),
+    # recurrent layers only, one of everything
+    "memories": joint(96, 64, mlstm(1, 16, 24, ff=24, experts=1, top=1), retention(1, 8, 40, 8), side=20),
     # recurrent layers only
     "average": parallel(96, 64, mingru(24, ff=72), mingru(200), taps=4),
     "recurrent": config(96, 64, delta(2, 2, 24, 16, 4, ff=72), delta(4, 1, 16, 32, 3)),
@@ -139,7 +197,7 @@ def weights(cfg, seed=0):
 
     def norm(name, W):
         put(name, W, std=0.2, mean=1.0)
-        if scaled:
+        if scaled or side:
             return
         put(name + ".b", W, std=0.1)
         if cfg["architecture"] == "Mebalorn":
@@ -147,19 +205,39 @@ def weights(cfg, seed=0):
         out[name + ".alpha"] = (0.3 + 0.5 * torch.rand((), generator=g)).to(torch.bfloat16)
 
     V, W, scaled = cfg["vocab"], cfg["width"], cfg["architecture"] == "Nurilorn"
-    put("embed", V, W, std=0.5 if scaled else 1.5)
+    side = (cfg.get("token_side") or {}).get("dim")
+    put("embed", V, W, std=0.5 if scaled or side else 1.5)
+    if side:
+        put("side.embed", V, len(cfg["layers"]) * side, std=1.0)
     for i, l in enumerate(cfg["layers"]):
         m, p = l["mixer"], f"l{i}.mix."
         norm(f"l{i}.norm1", W)
         if l["type"] == "latent_attention":
             H, R = m["heads"], m["kv_rank"]
             put(p + "q", H * (m["dim"] + m["rot_dim"]), W, std=3 * W ** -0.5)
-            put(p + "dkv", R + m["rot_dim"], W, std=2 * W ** -0.5)
-            put(p + "dkv.norm", R, std=0.2, mean=1.0)
+            if "kv_from" not in m:
+                put(p + "dkv", R + m["rot_dim"], W, std=2 * W ** -0.5)
+                put(p + "dkv.norm", R, std=0.2, mean=1.0)
             put(p + "uk", H * m["dim"], R)
             put(p + "uv", H * m["vdim"], R)
-            put(p + "sink", H, std=1.0, mean=1.5)
+            if side:
+                put(p + "g", H, W, std=1.5 * W ** -0.5)
+            else:
+                put(p + "sink", H, std=1.0, mean=1.5)
             put(p + "o", W, H * m["vdim"], std=2 * (H * m["vdim"]) ** -0.5)
+        elif l["type"] in ("retention", "mlstm"):
+            H, d, dv = m["heads"], m["dim"], m["vdim"]
+            for x, n in (("q", H * d), ("k", H * d), ("v", H * dv), ("g", H * dv)):
+                put(p + x, n, W, std=1.5 * W ** -0.5)
+            # a token finds its own key: where one read nothing but it, a chance product near zero
+            # would leave the read-out's sign to rounding
+            out[p + "k"] = (0.7 * out[p + "k"].float() + 0.7 * out[p + "q"].float()).to(torch.bfloat16)
+            if l["type"] == "mlstm":
+                for x, mean in (("i", 1.0), ("f", 4.0)):
+                    put(p + x, H, W, std=2 * W ** -0.5)
+                    put(f"{p}{x}.b", H, std=1.5, mean=mean)
+                put(p + "norm", H * dv, std=0.2, mean=1.0)
+            put(p + "o", W, H * dv, std=2 * (H * dv) ** -0.5)
         elif scaled:
             H, G, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
             for x, n in (("q", H * d), ("k", G * d), ("v", G * dv)):
@@ -208,12 +286,16 @@ def weights(cfg, seed=0):
             put(p + "o", W, H * dv, std=2 * (H * dv) ** -0.5)
         if l["mlp"] and l["mlp"]["kind"] == "moe":
             ff, n = l["mlp"]["expert"]["ff"], l["mlp"]["router"]["experts"]
-            norm(f"l{i}.norm2", W)
-            put(f"l{i}.mlp.router", n, W, std=6 * W ** -0.5)
+            if not side:
+                norm(f"l{i}.norm2", W)
+            put(f"l{i}.mlp.router", n, W, std=(9 if side else 6) * W ** -0.5)
+            if l["mlp"].get("shared"):
+                put(f"l{i}.mlp.shared.up", l["mlp"]["shared"]["ff"], W)
+                put(f"l{i}.mlp.shared.down", W, l["mlp"]["shared"]["ff"])
             for e in range(n):
-                for x in ("gate", "up"):
+                for x in ("gate", "up")[bool(side):]:
                     put(f"l{i}.mlp.e{e}.{x}", ff, W, std=1.5 * W ** -0.5)
-                put(f"l{i}.mlp.e{e}.down", W, ff, std=1.2 * ff ** -0.5)
+                put(f"l{i}.mlp.e{e}.down", W, ff, std=(0.6 if side else 1.2) * ff ** -0.5)
         elif l["mlp"]:
             ff = l["mlp"]["ff"]
             norm(f"l{i}.norm2", W)
@@ -221,11 +303,15 @@ def weights(cfg, seed=0):
                 put(f"l{i}.mlp.gate", ff, W, std=2 * W ** -0.5)
             put(f"l{i}.mlp.up", ff, W)
             put(f"l{i}.mlp.down", W, ff, std=2 * ff ** -0.5)
+        if side:
+            put(f"l{i}.side.gate", side, W)
+            put(f"l{i}.side.proj", W, side)
+            put(f"l{i}.side.norm", W, std=0.2, mean=0.6)
         if cfg["architecture"] == "Mebalorn":
             for k in (1, 2) if l["mlp"] else (1,):
                 put(f"l{i}.canon{k}", W, cfg["canon"]["taps"], std=0.5)
     norm("final.norm", W)
-    put("head", V, W, std=(2 if scaled else 3 if "logit_softcap" in cfg else 1) * W ** -0.5)
+    put("head", V, W, std=(2 if scaled or side else 3 if "logit_softcap" in cfg else 1) * W ** -0.5)
     return out
 
 

@@ -1,5 +1,5 @@
 """Models of mixed layer kinds, and the mechanisms of the Ralesun design (those of the others:
-test_hybrid_parallel.py, test_hybrid_grouped.py), against the plain implementation in hybrid_oracle.py: every
+test_hybrid_parallel.py, test_hybrid_grouped.py, test_hybrid_joint.py), against the plain implementation in hybrid_oracle.py: every
 mechanism alone, then the model on the engine - portions, batches, reuse of pages and slots,
 long decoding, generation.  Each case runs on the CPU (fp32 op references) and, marked gpu, on
 the HIP kernels in fp32 and bf16."""
@@ -14,13 +14,13 @@ import pytest
 import torch
 
 import hybrid_oracle as O
-from hybrid_util import (CONFIGS, attention, config, delta, grouped, latent, mingru, parallel, row_errors,
-                         save_checkpoint, scaled, tokens, weights)
+from hybrid_util import (CONFIGS, attention, config, delta, gated_latent, grouped, joint, latent, mingru, mlstm,
+                         parallel, retention, row_errors, save_checkpoint, scaled, tokens, weights)
 
 from drtc_amd import ops
 from drtc_amd.engine import LLMEngine, Request, SamplingParams
-from drtc_amd.models import (MEBALORN_2B, NURILORN_5B, NURILORN_24B, RALESUN_2B, TINY_MEBALORN, TINY_NURILORN,
-                             TINY_RALESUN, HybridLM, build_model, config_from_dict, get_config, load_model)
+from drtc_amd.models import (GARESUN_5B, GARESUN_24B, MEBALORN_2B, NURILORN_5B, NURILORN_24B, RALESUN_2B,
+                             TINY_GARESUN, TINY_MEBALORN, TINY_NURILORN, TINY_RALESUN, HybridLM, build_model, config_from_dict, get_config, load_model)
 from drtc_amd.models.checkpoint import read_safetensors
 
 F32, BF16 = torch.float32, torch.bfloat16
@@ -446,7 +446,7 @@ def test_prompt_decode_and_portions(target, name):
 
 
 @on
-@pytest.mark.parametrize("name", ["mixed", "talking", "capped"])
+@pytest.mark.parametrize("name", ["mixed", "talking", "capped", "memory"])
 def test_stream_follows_the_oracle(target, name):
     """The residual stream after every layer (fp32)."""
     dev, dt = target
@@ -458,6 +458,8 @@ def test_stream_follows_the_oracle(target, name):
     for i in range(len(cfg["layers"])):
         c2 = dict(cfg, layers=cfg["layers"][:i + 1], vocab=cfg["width"])
         w2 = {k: v for k, v in w.items() if not k.startswith("l") or int(k[1:k.index(".")]) <= i}
+        if "side.embed" in w:
+            w2["side.embed"] = w["side.embed"][:cfg["width"], :(i + 1) * cfg["token_side"]["dim"]]
         w2["embed"] = w["embed"][:cfg["width"]]
         w2["head"] = torch.eye(cfg["width"]).to(BF16)
         t2 = [t % cfg["width"] for t in toks]
@@ -467,7 +469,8 @@ def test_stream_follows_the_oracle(target, name):
 
 @on
 @pytest.mark.parametrize("name", ["mixed", "wide", "odd", "talking", "talking-wide", "talking-odd", "talking-any",
-                                  "capped", "capped-wide", "capped-odd", "capped-any"])
+                                  "capped", "capped-wide", "capped-odd", "capped-any", "memory", "memory-wide",
+                                  "memory-odd"])
 def test_mixed_batches(target, name):
     """Portions beside single tokens of other requests, idle requests, unequal lengths, and
     pages and slots freed and taken again - from a pool that holds no more than the live
@@ -507,7 +510,7 @@ def test_mixed_batches(target, name):
 
 
 @on
-@pytest.mark.parametrize("name", ["mixed", "talking", "capped"])
+@pytest.mark.parametrize("name", ["mixed", "talking", "capped", "memory"])
 def test_unwanted_rows_still_count(target, name):
     """Steps nothing is asked of leave the same cache and state; wanted places come in order."""
     cfg, _ = case(name)
@@ -526,7 +529,7 @@ def test_unwanted_rows_still_count(target, name):
 
 
 @on
-@pytest.mark.parametrize("name", ["mixed", "talking", "capped"])
+@pytest.mark.parametrize("name", ["mixed", "talking", "capped", "memory"])
 def test_long_decoding(target, name):
     """Hundreds of decoded tokens: windows, splits and blocks pass over decoded tokens."""
     if target[0] == "cpu":
@@ -539,7 +542,8 @@ def test_long_decoding(target, name):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("name", ["tiles", "talking-tiles", "talking-wide", "capped-tiles", "capped-wide"])
+@pytest.mark.parametrize("name", ["tiles", "talking-tiles", "talking-wide", "capped-tiles", "capped-wide", "memory-tiles",
+                                  "memory-wide"])
 @pytest.mark.parametrize("dtype", [F32, BF16], ids=["f32", "bf16"])
 def test_prefill_sized_steps(dtype, name):
     """Steps of more than a thousand rows (the prefill GEMMs, 256-row query tiles, portions far
@@ -602,6 +606,15 @@ def _mutations():
             l["mlp"].get("expert", l["mlp"])["limit"] = 1e6
         return l
 
+    def own_read(l):  # the other set of latents
+        if l["mixer"].get("kv_from") == 1:
+            l["mixer"]["kv_from"] = 4
+        return l
+
+    def no_shared(l):
+        (l["mlp"] or {}).pop("shared", None)
+        return l
+
     return {("mixed", "window+1"): window(1), ("mixed", "window-1"): window(-1),
             ("mixed", "no sink"): swap(".sink", lambda t: t * 0 - 50),
             ("mixed", "no decay bias"): swap("dt_bias", lambda t: t * 0),
@@ -629,7 +642,24 @@ def _mutations():
             ("capped", "no layer scale"): swap(".ls2", lambda t: t * 0 + 1),
             ("capped", "residual not multiplied"): lambda c, w: ({**c, "residual_mult": 1.0}, w),
             ("capped", "experts of any group"): layers(no_groups),
-            ("capped", "no limit"): layers(no_limit)}
+            ("capped", "no limit"): layers(no_limit),
+            ("memory", "other latents"): lambda c, w: (dict(c, layers=[
+                own_read(json.loads(json.dumps(l))) if i == 7 else l for i, l in enumerate(c["layers"])]), w),
+            ("memory", "no shared experts"): layers(no_shared),
+            ("memory", "gates open"): swap(".mix.g", lambda t: t * 0),
+            ("memory", "input gates shut"): swap(".mix.i.b", lambda t: t - 3),
+            ("memory", "no input gate"): swap(".mix.i", lambda t: t * 0),
+            ("memory", "no forget bias"): swap(".mix.f.b", lambda t: t * 0),
+            ("memory", "forgets later"): swap(".mix.f.b", lambda t: t + 3),
+            ("memory", "loose cap"): mixer(lambda m: m.update(gate_cap=1e6) if "gate_cap" in m else None),
+            ("memory", "other decay"): mixer(lambda m: m.update(decay=m["decay"][::-1]) if "decay" in m else None),
+            ("memory", "no memory norm"): swap(".mix.norm", lambda t: t * 0 + 1),
+            ("memory", "rotation"): mixer(lambda m: m["rot"].update(base=50.0) if "decay" in m else None),
+            ("memory", "part unrotated"): mixer(lambda m: m["rot"].update(dims=32) if m["dim"] == 64 else None),
+            ("memory", "no latent norm"): swap(".dkv.norm", lambda t: t * 0 + 1),
+            ("memory", "no token inputs"): swap(".side.norm", lambda t: t * 0),
+            ("memory", "another layer's input"): swap("side.embed", lambda t: torch.roll(t, 24, 1)),
+            ("memory", "embedding unscaled"): lambda c, w: ({**c, "embedding": {"scale": 1.0}}, w)}
 
 
 @pytest.mark.parametrize("mistake", list(_mutations()), ids=": ".join)
@@ -653,7 +683,7 @@ def greedy_ok(name, prompt, out, slack):
 
 
 @on
-@pytest.mark.parametrize("name", ["mixed", "talking", "capped"])
+@pytest.mark.parametrize("name", ["mixed", "talking", "capped", "memory"])
 @pytest.mark.parametrize("how", ["whole", "portions", "preempted"])
 def test_greedy_generation(target, how, name):
     cfg, _ = case(name)
@@ -678,7 +708,7 @@ def test_greedy_generation(target, how, name):
 
 
 @on
-@pytest.mark.parametrize("name", ["mixed", "talking", "capped"])
+@pytest.mark.parametrize("name", ["mixed", "talking", "capped", "memory"])
 def test_generation_with_stops_and_aborts(target, name):
     """Pipelined decoding over a changing batch: stop tokens found a step late, aborts, slot
     moves; every output as alone."""
@@ -706,7 +736,7 @@ def test_generation_with_stops_and_aborts(target, name):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("name", ["mixed", "talking", "capped"])
+@pytest.mark.parametrize("name", ["mixed", "talking", "capped", "memory"])
 def test_graphs_match_eager(name):
     """Replays of a captured step - several, with eager work between - advance the recurrent
     state exactly once each."""
@@ -726,7 +756,7 @@ def test_graphs_match_eager(name):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
-@pytest.mark.parametrize("name", ["mixed", "talking", "capped"])
+@pytest.mark.parametrize("name", ["mixed", "talking", "capped", "memory"])
 def test_trace_run(tmp_path, dtype, name):
     """The command-line replay: files, order, reuse of the pool, exit status."""
     cfg, w = case(name)
@@ -782,7 +812,7 @@ def test_checkpoint_folder(tmp_path):
 
 
 @on
-@pytest.mark.parametrize("cfg", [TINY_RALESUN, TINY_MEBALORN, TINY_NURILORN], ids=lambda c: c.name)
+@pytest.mark.parametrize("cfg", [TINY_RALESUN, TINY_MEBALORN, TINY_NURILORN, TINY_GARESUN], ids=lambda c: c.name)
 def test_registered_preset_serves(target, cfg):
     dev, dt = target
     m = build_model(cfg, dev, seed=3, dtype=dt)
@@ -794,10 +824,11 @@ def test_registered_preset_serves(target, cfg):
     assert m.weight_bytes() >= cfg.num_params() * m.embed.element_size()
     assert abs(RALESUN_2B.num_params() / 2.9e9 - 1) < 0.3
     assert abs(MEBALORN_2B.num_params() / 1.8e9 - 1) < 0.1
+    assert abs(GARESUN_5B.num_params() / 5e9 - 1) < 0.2 and abs(GARESUN_24B.num_params() / 24e9 - 1) < 0.2
     assert abs(NURILORN_5B.num_params() / 5e9 - 1) < 0.1 and abs(NURILORN_24B.num_params() / 24e9 - 1) < 0.1
 
 
-@pytest.mark.parametrize("name", ["mixed", "talking", "capped"])
+@pytest.mark.parametrize("name", ["mixed", "talking", "capped", "memory"])
 def test_service_backend_from_checkpoint_folder(tmp_path, name):
     """The LLM service's --model takes a checkpoint folder; text in, text out."""
     from argparse import Namespace
@@ -840,7 +871,19 @@ def test_limits_are_errors():
                 scaled(16, 16, grouped(2, 2, 8, 8, 8, ff=8, experts=6, top=2, groups=(4, 1))),
                 scaled(16, 16, grouped(2, 2, 8, 8, 8, ff=8, experts=6, top=4, groups=(2, 1))),
                 scaled(16, 16, dict(grouped(2, 2, 8, 8, 8), type="other")),
-                scaled(16, 16, dict(grouped(2, 2, 8, 8, 8), mlp={"kind": "other"}))):
+                scaled(16, 16, dict(grouped(2, 2, 8, 8, 8), mlp={"kind": "other"})),
+                joint(16, 16, retention(2, 8, 8, decay=[0.5])), joint(16, 16, retention(1, 8, 8, decay=[1.5])),
+                joint(16, 16, retention(1, 8, 8, decay=[0.0])), joint(16, 16, retention(1, 8, 8, 10)),
+                joint(16, 16, retention(1, 300, 8)), joint(16, 16, mlstm(1, 8, 1100)),
+                joint(16, 16, mlstm(1, 8, 8, cap=0.0)), joint(16, 16, dict(mlstm(1, 8, 8), type="other")),
+                joint(16, 16, dict(mlstm(1, 8, 8), mlp={"kind": "other"})),
+                joint(16, 16, mlstm(1, 8, 8, ff=8, experts=4, top=5)),
+                joint(16, 16, gated_latent(1, 8, 8, 8, 8, kv_from=0)),
+                joint(16, 16, mlstm(1, 8, 8), gated_latent(1, 8, 8, 8, 8, kv_from=0)),
+                joint(16, 16, gated_latent(1, 8, 8, 8, 8), gated_latent(1, 8, 8, 8, 16, kv_from=0)),
+                joint(16, 16, gated_latent(1, 8, 8, 8, 8), gated_latent(1, 8, 8, 8, 8, base=5.0, kv_from=0)),
+                joint(16, 16, gated_latent(1, 8, 8, 8, 8), gated_latent(1, 8, 8, 8, 8, kv_from=0),
+                      gated_latent(1, 8, 8, 8, 8, kv_from=1))):
         with pytest.raises(ValueError):
             config_from_dict(bad)
     with pytest.raises(ValueError):
