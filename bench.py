@@ -26,6 +26,7 @@ are torchrun's and WORLD_SIZE must equal --gpus.
 from __future__ import annotations
 
 import argparse
+import dataclasses
 import json
 import os
 import statistics
@@ -215,15 +216,18 @@ def self_launch(n: int) -> int:
 # Mebalorn layers (minGRU, then talking-heads attention of Llama's head sizes, each beside a
 # two-matrix feed-forward of 1.5 times Llama's size).  Four Nurilorn layers (capped attention of
 # Llama's head sizes, 16 experts of a quarter of its feed-forward, 4 per token out of 2 of 4 groups)
-# against four Mixtral-shaped layers with as many experts of that size.
+# against four Mixtral-shaped layers with as many experts of that size.  Four Garesun layers (matrix
+# memory, latent attention, retention, attention over the same latents, each beside 20 experts of two
+# matrices, 4 per token, and a shared one of twice their size) have as many parameters as the latter,
+# and as many at work for a token.
 DESIGN_SIZES = {2048: (16, 4, 7168), 4096: (32, 8, 14336)}  # width -> heads, kv heads, ff
 DESIGN_VOCAB = 32000
 
 
 def design_configs(width: int) -> dict:
     from drtc_amd.models.config import (ChannelDelta, Experts, GatedAverage, GroupedAttention,
-                                        HybridConfig, LatentAttention, Layer, ModelConfig,
-                                        RotaryScaling, TalkingAttention)
+                                        HybridConfig, LatentAttention, Layer, MatrixMemory, ModelConfig,
+                                        Retention, RotaryScaling, TalkingAttention, retention_decays)
 
     H, Hk, ff = DESIGN_SIZES[width]
     att = LatentAttention(H, 128, 64, 128, 512, 192 ** -0.5, 1024, 500000.0, 64)
@@ -231,7 +235,13 @@ def design_configs(width: int) -> dict:
     talk = TalkingAttention(H, Hk, 128, 128, 128 ** -0.5)
     capped = GroupedAttention(H, Hk, 128, 128, 128 ** -0.5, 500000.0, 64,
                               RotaryScaling(4.0, 8192, 32.0, 1.0), 4, 30.0, True)
+    full = LatentAttention(H, 128, 64, 128, 512, 192 ** -0.5, None, 500000.0, 64, False, True)
+    shared = dataclasses.replace(full, kv_from=1)
+    memories = (MatrixMemory(H, 128, 128, 15.0), full, Retention(H, 128, 128, retention_decays(H), 500000.0, 128), shared)
     return {
+        "garesun": HybridConfig(f"garesun-{width}", DESIGN_VOCAB, width,
+                                tuple(Layer(m, ff // 4, experts=Experts(20, 4), shared=ff // 2) for m in memories),
+                                act="relu2", block="joint", norm="layer", embed_scale=4.0, side_dim=width // 16),
         "nurilorn": HybridConfig(f"nurilorn-{width}", DESIGN_VOCAB, width,
                                  (Layer(capped, ff // 4, 7.0, Experts(16, 4, 4, 2)),) * 4,
                                  act="clamped", norm="group_rms", norm_groups=8, embed_scale=16.0,
@@ -306,10 +316,10 @@ def main() -> None:
     ap = argparse.ArgumentParser()
     ap.add_argument("--design", action="store_true",
                     help="instead of the serving workload: prefill / decode throughput of the "
-                         "Nurilorn, Mebalorn and Ralesun designs beside Mixtral-shaped and "
+                         "Garesun, Nurilorn, Mebalorn and Ralesun designs beside Mixtral-shaped and "
                          "Llama-shaped layers of equal size")
     ap.add_argument("--design-widths", default="2048,4096")
-    ap.add_argument("--design-families", default="nurilorn,mixtral,mebalorn,ralesun,llama")
+    ap.add_argument("--design-families", default="garesun,nurilorn,mixtral,mebalorn,ralesun,llama")
     ap.add_argument("--design-phases", default="prefill,decode")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)
