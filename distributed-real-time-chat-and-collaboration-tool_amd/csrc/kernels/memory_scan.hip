@@ -141,8 +141,7 @@ __global__ __launch_bounds__(576) void memory_scan_kernel(MemoryArgs a) {
     float mm = m, da[CT], db[CT];
 #pragma unroll
     for (int t = 0; t < CT; ++t) {
-      if (t >= nt) break;
-      const float f = av[t], i = bv[t], mn = fmaxf(f + mm, i);
+      const float f = t < nt ? av[t] : 0.f, i = t < nt ? bv[t] : kNegBig, mn = fmaxf(f + mm, i);
       da[t] = expf(f + mm - mn);
       db[t] = expf(i - mn);
       mm = mn;
@@ -152,7 +151,7 @@ __global__ __launch_bounds__(576) void memory_scan_kernel(MemoryArgs a) {
     if (live) {
 #pragma unroll
       for (int t = 0; t < CT; ++t) {
-        if (t >= nt) break;
+        if (t >= nt) continue;
         float u[CPL], o[CPL];
 #pragma unroll
         for (int c = 0; c < CPL; ++c) {
@@ -236,10 +235,12 @@ __global__ __launch_bounds__(576) void memory_scan_kernel(MemoryArgs a) {
 // accumulator tiles.  Their layout (row 4 g + r of lane group g) is that of an A operand of S^T
 // whose k-step takes dims 4 g + r of two tiles, so S feeds O^T = S^T Q^T without lane movement,
 // split into two bf16 parts (16 significant bits).  K and V are read transposed from LDS; the
-// weights of the update go onto the V fragments in registers.
+// weights of the update go onto the V fragments in registers.  The scales of queries and keys ride
+// on the exponents and weights, so unrotated rows are staged as they are.
 constexpr int kMC = 64;
 
 typedef short mem_s16x4 __attribute__((ext_vector_type(4)));
+typedef unsigned int u32x2 __attribute__((ext_vector_type(2)));
 DRTC_DEVICE bf16x4 mem_read_tr16(const bf16_t* p) {
   mem_s16x4 v = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
       (__attribute__((address_space(3))) mem_s16x4*)(p));
@@ -251,422 +252,438 @@ DRTC_DEVICE bf16x8 mem_join(bf16x4 lo, bf16x4 hi) {
   for (int j = 0; j < 4; ++j) { v[j] = lo[j]; v[4 + j] = hi[j]; }
   return v;
 }
-DRTC_DEVICE bf16x8 mem_zero8() {
-  bf16x8 z;
-#pragma unroll
-  for (int j = 0; j < 8; ++j) z[j] = f2bf(0.f);
-  return z;
+// 16 / 8 bytes at a 32-bit byte offset from a base all lanes share
+DRTC_DEVICE bf16x8 mem_at8(const bf16_t* base, unsigned off) {
+  return *reinterpret_cast<const bf16x8*>(reinterpret_cast<const char*>(base) + off);
 }
-DRTC_DEVICE float lane_scan_sum(float v, int lane) {
-#pragma unroll
-  for (int o = 1; o < 64; o <<= 1) {
-    const float u = __shfl_up(v, o, 64);
-    if (lane >= o) v += u;
-  }
-  return v;
+DRTC_DEVICE bf16x4 mem_at4(const bf16_t* base, unsigned off) {
+  return *reinterpret_cast<const bf16x4*>(reinterpret_cast<const char*>(base) + off);
 }
-DRTC_DEVICE float lane_scan_max(float v, int lane) {
-#pragma unroll
-  for (int o = 1; o < 64; o <<= 1) {
-    const float u = __shfl_up(v, o, 64);
-    if (lane >= o) v = fmaxf(v, u);
-  }
-  return v;
+// v of another lane by DPP; lanes without a source: `other`
+template <int CTRL, int ROWS>
+DRTC_DEVICE float lane_from(float v, float other) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(__float_as_int(other), __float_as_int(v), CTRL,
+                                                    ROWS, 0xF, false));
+}
+// Inclusive scan over the lanes of a wave: within rows of 16, then the rows' last lanes on.
+template <class Op>
+DRTC_DEVICE float lane_scan(float v, float zero, Op op) {
+  v = op(v, lane_from<0x111, 0xF>(v, zero));
+  v = op(v, lane_from<0x112, 0xF>(v, zero));
+  v = op(v, lane_from<0x114, 0xF>(v, zero));
+  v = op(v, lane_from<0x118, 0xF>(v, zero));
+  v = op(v, lane_from<0x142, 0xA>(v, zero));
+  return op(v, lane_from<0x143, 0xC>(v, zero));
+}
+DRTC_DEVICE float last_lane(float v) {
+  return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63));
+}
+// cap tanh(x / cap) and log2 sigmoid by hardware exp2 / log2; for large x the latter's series, where
+// 1 + e^-x would round
+DRTC_DEVICE float cap_hw(float x, float cap, float inv) {
+  return cap - 2.f * cap * __builtin_amdgcn_rcpf(1.f + fast_exp2(x * inv * (2.f * kLog2e)));
+}
+DRTC_DEVICE float logsig2_hw(float x) {
+  const float e = fast_exp2(-x * kLog2e);
+  const float l = __builtin_amdgcn_logf(1.f + e), y = e * (1.f - e * (0.5f - e * (1.f / 3.f))) * kLog2e;
+  return x < -30.f ? x * kLog2e : x > 6.f ? -y : -l;
 }
 
-// KS: 32-dim steps of a key (padded); NW waves of CT column tiles
-template <int KS, int NW, int CT>
+// KS: 32-dim steps of a key (padded); NW waves of 16 columns
+template <int KS, int NW>
 struct MemLds {
-  static constexpr int DP = 32 * KS, COLS = 16 * CT * NW;
+  static constexpr int DP = 32 * KS, COLS = 16 * NW, NG = NW / 4;
   static constexpr int QROW = DP + 8, KROW = DP + 16, VROW = COLS + 16, PROW = kMC + 8;
   // bf16 elements, then floats
   static constexpr int q = 0, k = q + kMC * QROW, v = k + kMC * KROW, p = v + kMC * VROW;
   static constexpr int bf = p + kMC * PROW;
-  static constexpr int n = 0, g = n + DP, m = g + kMC, in = m + kMC, em = in + kMC, w = em + kMC;
-  static constexpr int qn = w + kMC, rs = qn + kMC, ss = rs + 2 * kMC, fl = ss + NW * kMC;
+  // gates of two chunks: g, M, 2^(m_0 - M), 2^-m, update weights, the state's factor
+  static constexpr int G = 5 * kMC + 4, m = kMC, in = 2 * kMC, em = 3 * kMC, w = 4 * kMC, ga = 5 * kMC;
+  static constexpr int n = 2 * G, qn = n + 2 * DP, rs = qn + kMC, ss = rs + NG * kMC, fl = ss + NW * kMC;  // ss [token][wave]
   static constexpr size_t BYTES = (size_t)bf * 2 + (size_t)fl * 4;
 };
 
-template <int KS, int NW, int CT, bool GATED>
+template <int KS, int NW, bool GATED, bool ROT>
 __global__ __launch_bounds__(64 * NW, 2) void memory_chunk_kernel(MemoryArgs a) {
-  using L = MemLds<KS, NW, CT>;
-  constexpr int NTHR = 64 * NW, PU = L::DP / 16, NU = (kMC * PU + NTHR - 1) / NTHR, NV = 2 * CT;
+  using L = MemLds<KS, NW>;
+  constexpr int NTHR = 64 * NW, PU = L::DP / 16, NU = (kMC * PU + NTHR - 1) / NTHR, NV = 2;
   extern __shared__ __attribute__((aligned(16))) bf16_t mb[];
   float* fl = reinterpret_cast<float*>(mb + L::bf);
   const int seg = blockIdx.x, h = blockIdx.y, sl = blockIdx.z, c0 = sl * L::COLS;
   const int slot = a.seg_state[seg];
   const int n = a.seg_len[seg], row0 = a.seg_row[seg], pos0 = a.seg_pos[seg];
   const int tid = threadIdx.x, w = wave_id_uniform(), lane = tid & 63, col = lane & 15, g = lane >> 4;
-  bf16_t* out = (bf16_t*)a.out + h * a.vdim;
+  const int cols = min(L::COLS, a.vdim - c0);
+  bf16_t* out = (bf16_t*)a.out + (int64_t)row0 * a.ldo + h * a.vdim + c0;
   if (slot < 0) {
-    const int cols = min(L::COLS, a.vdim - c0);
-    for (int i = tid; i < n * cols; i += NTHR)
-      out[(int64_t)(row0 + i / cols) * a.ldo + c0 + i % cols] = f2bf(0.f);
+    for (int i = tid; i < n * cols; i += NTHR) out[(int64_t)(i / cols) * a.ldo + i % cols] = f2bf(0.f);
     return;
   }
   const bf16_t* proj = (const bf16_t*)a.proj + (int64_t)row0 * a.ldp;
-  const int cw = c0 + 16 * CT * w;  // this wave's first column
-  float* S = a.state + ((int64_t)slot * a.H + h) * a.dim * a.vdim;
+  const int cw = 16 * w;  // this wave's first column of the workgroup's
+  const bool own = cw < cols;
+  const int nwave = (cols - 1) >> 4;  // keeps the normaliser
+  float* S = a.state + ((int64_t)slot * a.H + h) * a.dim * a.vdim + c0;
   float* N = GATED ? a.nrm + (((int64_t)slot * a.H + h) * a.slices + sl) * a.dim : nullptr;
   float* top = GATED ? a.top + ((int64_t)slot * a.H + h) * a.slices + sl : nullptr;
 
-  f32x4 st[2 * KS][CT];
+  f32x4 st[2 * KS];
 #pragma unroll
   for (int t = 0; t < 2 * KS; ++t)
 #pragma unroll
-    for (int ct = 0; ct < CT; ++ct)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = 16 * t + 4 * g + r, x = cw + 16 * ct + col;
-        st[t][ct][r] = pos0 > 0 && d < a.dim && x < a.vdim ? S[(int64_t)d * a.vdim + x] : 0.f;
-      }
-  float m0 = 0.f;  // log2 units
+    for (int r = 0; r < 4; ++r) {
+      const int d = 16 * t + 4 * g + r, x = cw + col;
+      st[t][r] = pos0 > 0 && d < a.dim && x < cols ? S[d * a.vdim + x] : 0.f;
+    }
   if constexpr (GATED) {
-    if (pos0 > 0) m0 = top[0] * kLog2e;
     for (int d = tid; d < L::DP; d += NTHR) fl[L::n + d] = pos0 > 0 && d < a.dim ? N[d] : 0.f;
   }
-  const float f2 = GATED ? 0.f : a.log_decay[h] * kLog2e;
-  f32x4 nw[CT];
-#pragma unroll
-  for (int ct = 0; ct < CT; ++ct)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int x = cw + 16 * ct + 4 * g + r;
-      nw[ct][r] = a.norm_w && x < a.vdim ? a.norm_w[h * a.vdim + x] : 1.f;
-    }
 
   // staging: a unit is two 8-element vectors of a token's query and key - the two halves of eight
-  // rotated pairs, or neighbours behind the rotated part
+  // rotated pairs, or neighbours behind the rotated part.  Tokens behind the portion repeat its
+  // last one: their weights are zero.
   const int half = a.rot_dims >> 1;
-  auto unit = [&](int i, int& tok, int& e0, int& e1, bool& turn) {
-    const int u = tid + i * NTHR;
-    tok = u / PU;
-    const int pr = u % PU;
-    turn = 16 * pr < a.rot_dims;
-    e0 = turn ? 8 * pr : 16 * pr;
-    e1 = turn ? 8 * pr + half : 16 * pr + 8;
-    return u < kMC * PU;
-  };
+  int tok[NU], e0[NU], e1[NU];
+  bool in_u[NU], turn[NU];
+#pragma unroll
+  for (int i = 0; i < NU; ++i) {
+    const int u = tid + i * NTHR, pr = u % PU;
+    in_u[i] = u < kMC * PU && 16 * pr < a.dim;
+    tok[i] = in_u[i] ? u / PU : 0;
+    turn[i] = ROT && in_u[i] && 16 * pr < a.rot_dims;
+    e0[i] = !in_u[i] ? 0 : turn[i] ? 8 * pr : 16 * pr;
+    e1[i] = turn[i] ? e0[i] + half : e0[i] + 8;
+  }
   bf16x8 pq[NU][2], pk[NU][2], pv[NV];
-  float gi = 0.f, gf = 0.f;
+  float cs[ROT ? NU : 1][2][8];
+  // without branches, so that no wait for one load becomes a wait for all
   auto prefetch = [&](int t0) {
+    const bf16_t *qb = proj + (int64_t)t0 * a.ldp + h * a.dim, *kb = qb + a.off_k;
+    const float* cb = a.cos_sin + (int64_t)(pos0 + t0) * a.rot_dims;
+    const int last = n - 1 - t0;
 #pragma unroll
     for (int i = 0; i < NU; ++i) {
-      int tok, e0, e1;
-      bool turn;
-      const bool in = unit(i, tok, e0, e1, turn) && t0 + tok < n;
-      const bf16_t* r = proj + (int64_t)(t0 + tok) * a.ldp + h * a.dim;
-      const bool in0 = in && e0 < a.dim, in1 = in && e1 < a.dim;
-      pq[i][0] = in0 ? load_bf16x8(r + e0) : mem_zero8();
-      pq[i][1] = in1 ? load_bf16x8(r + e1) : mem_zero8();
-      pk[i][0] = in0 ? load_bf16x8(r + a.off_k + e0) : mem_zero8();
-      pk[i][1] = in1 ? load_bf16x8(r + a.off_k + e1) : mem_zero8();
+      const unsigned tk = min(tok[i], last), r = tk * a.ldp;
+      const unsigned o0 = 2 * (r + e0[i]), o1 = 2 * (r + e1[i]);
+      pq[i][0] = mem_at8(qb, o0);
+      pq[i][1] = mem_at8(qb, o1);
+      pk[i][0] = mem_at8(kb, o0);
+      pk[i][1] = mem_at8(kb, o1);
+      if constexpr (ROT) {
+        const unsigned c = tk * a.rot_dims + (turn[i] ? e0[i] : 0);
+        load8(cs[i][0], cb + c);
+        load8(cs[i][1], cb + c + half);
+      }
     }
+    const bf16_t* vb = proj + (int64_t)t0 * a.ldp + a.off_v + h * a.vdim + c0;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int v = tid + i * NTHR, tok = v / (L::COLS / 8), c = c0 + (v % (L::COLS / 8)) * 8;
-      pv[i] = t0 + tok < n && c < a.vdim
-          ? load_bf16x8(proj + (int64_t)(t0 + tok) * a.ldp + a.off_v + h * a.vdim + c) : mem_zero8();
-    }
-    if (GATED && t0 + lane < n) {
-      const bf16_t* r = proj + (int64_t)(t0 + lane) * a.ldp + h;
-      gi = bf2f(r[a.off_i]);
-      gf = bf2f(r[a.off_f]);
+      const int v = tid + i * NTHR, tk = v / (L::COLS / 8), c = (v % (L::COLS / 8)) * 8;
+      pv[i] = mem_at8(vb, 2u * (unsigned)(min(tk, last) * a.ldp + min(c, cols - 8)));
     }
   };
   prefetch(0);
-  const int tr_k = ((col >> 2) + 4 * g) * L::KROW + 4 * (col & 3);
-  const int tr_v = ((col >> 2) + 4 * g) * L::VROW + 4 * (col & 3) + 16 * CT * w;
-  const float ib = GATED ? a.i_bias[h] : 0.f, fb = GATED ? a.f_bias[h] : 0.f;
+  {  // columns behind the head and the values stay zero
+    bf16x8 z;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) z[j] = f2bf(0.f);
+    const int dv = L::DP / 8, lo = a.dim / 8;
+    for (int i = tid; i < kMC * (dv - lo); i += NTHR) {
+      const int t = i / (dv - lo), c = (lo + i % (dv - lo)) * 8;
+      store_bf16x8(mb + L::q + t * L::QROW + c, z);
+      store_bf16x8(mb + L::k + t * L::KROW + c, z);
+    }
+    const int vv = L::COLS / 8, vlo = cols / 8;
+    for (int i = tid; i < kMC * (vv - vlo); i += NTHR)
+      store_bf16x8(mb + L::v + (i / (vv - vlo)) * L::VROW + (vlo + i % (vv - vlo)) * 8, z);
+  }
 
-  for (int t0 = 0; t0 < n; t0 += kMC) {
+  // gates of a chunk, one token to a lane of the first wave, a chunk ahead of their use
+  float m0 = 0.f;  // log2 units
+  bf16_t gi = f2bf(0.f), gf = f2bf(0.f);
+  const float f2 = GATED ? 0.f : a.log_decay[h] * kLog2e;
+  const float lk = log2f(a.k_scale), lq = log2f(a.q_scale), inv_cap = GATED ? 1.f / a.cap : 0.f;
+  const float ib = GATED ? a.i_bias[h] : 0.f, fb = GATED ? a.f_bias[h] : 0.f;
+  auto load_gates = [&](int t0) {
+    if constexpr (GATED) {
+      const bf16_t* r = proj + (int64_t)min(t0 + lane, n - 1) * a.ldp + h;
+      gi = r[a.off_i];
+      gf = r[a.off_f];
+    }
+  };
+  auto gates = [&](int t0, float* b) {
     const int nt = min(kMC, n - t0);
-    // gates: one token to a lane, every wave for itself
     float F, gg, M;
     if constexpr (GATED) {
-      const float i = a.cap * tanhf((gi + ib) / a.cap), f = mem_logsig(a.cap * tanhf((gf + fb) / a.cap));
-      F = lane_scan_sum(lane < nt ? f * kLog2e : 0.f, lane);
-      gg = lane < nt ? i * kLog2e - F : kNegBig;
-      M = fmaxf(m0, lane_scan_max(gg, lane));
+      const float f = logsig2_hw(cap_hw(bf2f(gf) + fb, a.cap, inv_cap));
+      F = lane_scan(lane < nt ? f : 0.f, 0.f, [](float x, float y) { return x + y; });
+      gg = lane < nt ? cap_hw(bf2f(gi) + ib, a.cap, inv_cap) * kLog2e - F : kNegBig;
+      M = fmaxf(m0, lane_scan(gg, kNegBig, [](float x, float y) { return fmaxf(x, y); }));
     } else {
       F = (float)min(lane + 1, nt) * f2;
       gg = -F;
       M = -F;
     }
-    const float M1 = __shfl(M, 63, 64), gamma = fast_exp2(m0 - M1);
-    if (w == 0) {
-      fl[L::g + lane] = gg;
-      fl[L::m + lane] = M;
-      fl[L::in + lane] = fast_exp2(m0 - M);
-      fl[L::em + lane] = fast_exp2(-(F + M));
-      fl[L::w + lane] = lane < nt ? fast_exp2(gg - M1) : 0.f;
+    const float M1 = last_lane(M);
+    b[lane] = gg + lk;
+    b[L::m + lane] = M - lq;
+    b[L::in + lane] = fast_exp2(m0 - M) * a.q_scale;
+    b[L::em + lane] = fast_exp2(-(F + M));
+    b[L::w + lane] = lane < nt ? fast_exp2(gg - M1) * a.k_scale : 0.f;
+    if (lane == 0) b[L::ga] = fast_exp2(m0 - M1);
+    if constexpr (GATED) m0 = last_lane(F) + M1;
+  };
+  if (w == 0) {
+    if (GATED && pos0 > 0) m0 = top[0] * kLog2e;
+    load_gates(0);
+    gates(0, fl);
+    load_gates(kMC);
+  }
+  const int tr_k = ((col >> 2) + 4 * g) * L::KROW + 4 * (col & 3);
+  const int tr_v = ((col >> 2) + 4 * g) * L::VROW + 4 * (col & 3) + cw;
+  f32x4 nw;
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+    nw[r] = a.norm_w && cw + 4 * g + r < cols ? a.norm_w[h * a.vdim + c0 + cw + 4 * g + r] : 1.f;
+  const float inv_dv = 1.f / (float)a.vdim;
+
+  float* cur = fl;
+  for (int t0 = 0; t0 < n; t0 += kMC) {
+    float* nxt = cur == fl ? fl + L::G : fl;
+    const float* nc = fl + L::n + (cur == fl ? 0 : L::DP);  // the normaliser, and after this chunk
+    float* nn = fl + L::n + (cur == fl ? L::DP : 0);
+    const int nt = min(kMC, n - t0);
+    bf16x4 gate[4];  // read-out gates of this chunk
+    {
+      const bf16_t* base = proj + (int64_t)t0 * a.ldp + a.off_g + h * a.vdim + c0;
+      const int x = min(cw + 4 * g, cols - 4);
+#pragma unroll
+      for (int tt = 0; tt < 4; ++tt)
+        gate[tt] = mem_at4(base, 2u * (unsigned)(min(16 * tt + col, nt - 1) * a.ldp + x));
     }
-    if constexpr (GATED) m0 = __shfl(F, 63, 64) + M1;
 #pragma unroll
     for (int i = 0; i < NU; ++i) {
-      int tok, e0, e1;
-      bool turn;
-      if (!unit(i, tok, e0, e1, turn)) continue;
-      float x[2][8], y[2][8];
+      if constexpr (ROT) {
+        if (turn[i]) {
+          auto rotate = [&](bf16x8 (&x)[2]) {
 #pragma unroll
-      for (int j = 0; j < 8; ++j)
-#pragma unroll
-        for (int e = 0; e < 2; ++e) {
-          x[e][j] = bf2f(pq[i][e][j]);
-          y[e][j] = bf2f(pk[i][e][j]);
-        }
-      if (turn && t0 + tok < n) {
-        const float* cs = a.cos_sin + (int64_t)(pos0 + t0 + tok) * a.rot_dims + e0;
-        float c[8], s[8];
-        load8(c, cs);
-        load8(s, cs + half);
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const float u = x[0][j], v = x[1][j], z = y[0][j], zz = y[1][j];
-          x[0][j] = u * c[j] - v * s[j];
-          x[1][j] = v * c[j] + u * s[j];
-          y[0][j] = z * c[j] - zz * s[j];
-          y[1][j] = zz * c[j] + z * s[j];
+            for (int j = 0; j < 8; ++j) {
+              const float c = cs[i][0][j], s = cs[i][1][j], x0 = bf2f(x[0][j]), x1 = bf2f(x[1][j]);
+              x[0][j] = f2bf(x0 * c - x1 * s);
+              x[1][j] = f2bf(x1 * c + x0 * s);
+            }
+          };
+          rotate(pq[i]);
+          rotate(pk[i]);
         }
       }
-      // columns behind the head (and, unrotated, their vectors) are zeros
-#pragma unroll
-      for (int e = 0; e < 2; ++e) {
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          x[e][j] *= a.q_scale;
-          y[e][j] *= a.k_scale;
-        }
-        const int at = e ? e1 : e0;
-        store8(mb + L::q + tok * L::QROW + at, x[e]);
-        store8(mb + L::k + tok * L::KROW + at, y[e]);
+      if (in_u[i]) {
+        bf16_t *qd = mb + L::q + tok[i] * L::QROW, *kd = mb + L::k + tok[i] * L::KROW;
+        store_bf16x8(qd + e0[i], pq[i][0]);
+        store_bf16x8(qd + e1[i], pq[i][1]);
+        store_bf16x8(kd + e0[i], pk[i][0]);
+        store_bf16x8(kd + e1[i], pk[i][1]);
       }
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int v = tid + i * NTHR;
-      store_bf16x8(mb + L::v + (v / (L::COLS / 8)) * L::VROW + (v % (L::COLS / 8)) * 8, pv[i]);
+      const int v = tid + i * NTHR, c = (v % (L::COLS / 8)) * 8;
+      if (c < cols) store_bf16x8(mb + L::v + (v / (L::COLS / 8)) * L::VROW + c, pv[i]);
     }
-    prefetch(t0 + kMC);
+    prefetch(min(t0 + kMC, n - 1));
     __syncthreads();
 
-    // weighted scores of 16 tokens to a wave (8 waves: every other key tile each)
+    // what does not need the scores of other waves: the weighted scores of 16 tokens to a wave (8
+    // waves: every other key tile), the read-out of the state, its update
     {
       const int tt = w & 3, t = 16 * tt + col;
-      const float Mt = fl[L::m + t];
+      const float Mt = cur[L::m + t];
       bf16x8 qf[KS];
 #pragma unroll
       for (int s = 0; s < KS; ++s) qf[s] = load_bf16x8(mb + L::q + t * L::QROW + 32 * s + 8 * g);
       float rsum = 0.f;
 #pragma unroll
-      for (int st_ = 0; st_ < 4; ++st_) {
-        if (NW == 8 && (st_ & 1) != (w >> 2)) continue;
-        if (st_ > (tt | 1)) continue;
+      for (int kt = 0; kt < 4; ++kt) {
+        if (kt % L::NG != (w >> 2) || kt > (tt | 1)) continue;
         bf16x4 pf;
 #pragma unroll
         for (int r = 0; r < 4; ++r) pf[r] = f2bf(0.f);
-        if (st_ <= tt) {
+        if (kt <= tt) {
           f32x4 sc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int s = 0; s < KS; ++s)
-            sc = mfma16(load_bf16x8(mb + L::k + (16 * st_ + col) * L::KROW + 32 * s + 8 * g), qf[s], sc);
-          const f32x4 gj = *reinterpret_cast<const f32x4*>(fl + L::g + 16 * st_ + 4 * g);
+            sc = mfma16(load_bf16x8(mb + L::k + (16 * kt + col) * L::KROW + 32 * s + 8 * g), qf[s], sc);
+          const f32x4 gj = *reinterpret_cast<const f32x4*>(cur + 16 * kt + 4 * g);
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            const float p = 16 * st_ + 4 * g + r <= t ? sc[r] * fast_exp2(fminf(gj[r] - Mt, 0.f)) : 0.f;
+            const float p = 16 * kt + 4 * g + r <= t ? sc[r] * fast_exp2(gj[r] - Mt) : 0.f;
             rsum += p;
             pf[r] = f2bf(p);
           }
         }
         // keys in the order of the V fragments: 4 g + r of both tiles of a 32-key step together
-        *reinterpret_cast<bf16x4*>(mb + L::p + t * L::PROW + 32 * (st_ >> 1) + 8 * g + 4 * (st_ & 1)) = pf;
+        *reinterpret_cast<bf16x4*>(mb + L::p + t * L::PROW + 32 * (kt >> 1) + 8 * g + 4 * (kt & 1)) = pf;
       }
       if constexpr (GATED) {
         rsum += __shfl_xor(rsum, 16, 64);
         rsum += __shfl_xor(rsum, 32, 64);
         if (g == 0) fl[L::rs + (w >> 2) * kMC + t] = rsum;
         constexpr int PART = L::DP / NW;  // n.q: NW lanes to a token
-        const int tok = tid / NW, part = tid % NW;
+        const int tk = tid / NW, part = tid % NW;
         float d = 0.f;
 #pragma unroll
         for (int j = 0; j < PART; j += 4) {
-          const bf16x4 q4 = load_bf16x4(mb + L::q + tok * L::QROW + part * PART + j);
-          const f32x4 n4 = *reinterpret_cast<const f32x4*>(fl + L::n + part * PART + j);
+          const bf16x4 q4 = load_bf16x4(mb + L::q + tk * L::QROW + part * PART + j);
+          const f32x4 n4 = *reinterpret_cast<const f32x4*>(nc + part * PART + j);
 #pragma unroll
           for (int r = 0; r < 4; ++r) d += bf2f(q4[r]) * n4[r];
         }
         d = NW == 4 ? quad_sum(d) : sum8(d);
-        if (part == 0) fl[L::qn + tok] = d;
+        if (part == 0) fl[L::qn + tk] = d;
+      }
+      if (w == 0 && t0 + kMC < n) {
+        gates(t0 + kMC, nxt);
+        load_gates(t0 + 2 * kMC);
       }
     }
-    __syncthreads();
-
-    bf16x4 gate[CT][4];
-    if (a.slices == 1) {
+    f32x4 o[4];
 #pragma unroll
-      for (int ct = 0; ct < CT; ++ct)
+    for (int tt = 0; tt < 4; ++tt) o[tt] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    bf16x8 vf[2];
+    if (own) {
 #pragma unroll
-        for (int tt = 0; tt < 4; ++tt) {
-          const int t = 16 * tt + col, x = cw + 16 * ct + 4 * g;
-          if (t < nt && x < a.vdim)
-            gate[ct][tt] = load_bf16x4(proj + (int64_t)(t0 + t) * a.ldp + a.off_g + h * a.vdim + x);
-        }
-    }
-    f32x4 o[CT][4];
-#pragma unroll
-    for (int ct = 0; ct < CT; ++ct)
-#pragma unroll
-      for (int tt = 0; tt < 4; ++tt) o[ct][tt] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int s = 0; s < KS; ++s) {
-      bf16x8 qf[4];
-#pragma unroll
-      for (int tt = 0; tt < 4; ++tt) {
-        const bf16_t* q = mb + L::q + (16 * tt + col) * L::QROW + 32 * s + 4 * g;
-        qf[tt] = mem_join(load_bf16x4(q), load_bf16x4(q + 16));
-      }
-#pragma unroll
-      for (int ct = 0; ct < CT; ++ct) {
+      for (int s = 0; s < KS; ++s) {
         bf16x8 hi, lo;
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          const float x = st[2 * s + (j >> 2)][ct][j & 3];
+          const float x = st[2 * s + (j >> 2)][j & 3];
           hi[j] = f2bf(x);
           lo[j] = f2bf(x - bf2f(hi[j]));
         }
 #pragma unroll
         for (int tt = 0; tt < 4; ++tt) {
-          o[ct][tt] = mfma16(hi, qf[tt], o[ct][tt]);
-          o[ct][tt] = mfma16(lo, qf[tt], o[ct][tt]);
-        }
-      }
-    }
-    float inv[4];
-#pragma unroll
-    for (int tt = 0; tt < 4; ++tt) {
-      const int t = 16 * tt + col;
-      const float in = fl[L::in + t];
-#pragma unroll
-      for (int ct = 0; ct < CT; ++ct) o[ct][tt] *= in;
-      inv[tt] = 1.f;
-      if constexpr (GATED) {
-        float d = in * fl[L::qn + t] + fl[L::rs + t];
-        if constexpr (NW == 8) d += fl[L::rs + kMC + t];
-        inv[tt] = 1.f / (fmaxf(fabsf(d), fl[L::em + t]) + 1e-6f);
-      }
-    }
-    bf16x8 vw[2][CT], wf[2];
-#pragma unroll
-    for (int ks = 0; ks < 2; ++ks) {
-      const f32x4 w0 = *reinterpret_cast<const f32x4*>(fl + L::w + 32 * ks + 4 * g);
-      const f32x4 w1 = *reinterpret_cast<const f32x4*>(fl + L::w + 32 * ks + 16 + 4 * g);
-      bf16x8 vf[CT];
-#pragma unroll
-      for (int ct = 0; ct < CT; ++ct) {
-        const bf16_t* v = mb + L::v + tr_v + 32 * ks * L::VROW + 16 * ct;
-        vf[ct] = mem_join(mem_read_tr16(v), mem_read_tr16(v + 16 * L::VROW));
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          vw[ks][ct][j] = f2bf(bf2f(vf[ct][j]) * w0[j]);
-          vw[ks][ct][4 + j] = f2bf(bf2f(vf[ct][4 + j]) * w1[j]);
+          const bf16_t* q = mb + L::q + (16 * tt + col) * L::QROW + 32 * s + 4 * g;
+          const bf16x8 qf = mem_join(load_bf16x4(q), load_bf16x4(q + 16));
+          o[tt] = mfma16(hi, qf, o[tt]);
+          o[tt] = mfma16(lo, qf, o[tt]);
         }
       }
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        wf[ks][j] = f2bf(w0[j]);
-        wf[ks][4 + j] = f2bf(w1[j]);
-      }
-#pragma unroll
-      for (int tt = 2 * ks; tt < 4; ++tt) {
-        const bf16x8 pf = load_bf16x8(mb + L::p + (16 * tt + col) * L::PROW + 32 * ks + 8 * g);
-#pragma unroll
-        for (int ct = 0; ct < CT; ++ct) o[ct][tt] = mfma16(vf[ct], pf, o[ct][tt]);
-      }
-    }
-#pragma unroll
-    for (int t = 0; t < 2 * KS; ++t) {
-      bf16x8 kf[2];
+      for (int tt = 0; tt < 4; ++tt) o[tt] *= cur[L::in + 16 * tt + col];
+      bf16x8 vw[2], wf[2];
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
-        const bf16_t* k = mb + L::k + tr_k + 32 * ks * L::KROW + 16 * t;
-        kf[ks] = mem_join(mem_read_tr16(k), mem_read_tr16(k + 16 * L::KROW));
+        const f32x4 w0 = *reinterpret_cast<const f32x4*>(cur + L::w + 32 * ks + 4 * g);
+        const f32x4 w1 = *reinterpret_cast<const f32x4*>(cur + L::w + 32 * ks + 16 + 4 * g);
+        const bf16_t* v = mb + L::v + tr_v + 32 * ks * L::VROW;
+        vf[ks] = mem_join(mem_read_tr16(v), mem_read_tr16(v + 16 * L::VROW));
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          vw[ks][j] = f2bf(bf2f(vf[ks][j]) * w0[j]);
+          vw[ks][4 + j] = f2bf(bf2f(vf[ks][4 + j]) * w1[j]);
+          if constexpr (GATED) {
+            wf[ks][j] = f2bf(w0[j]);
+            wf[ks][4 + j] = f2bf(w1[j]);
+          }
+        }
       }
+      const float gamma = cur[L::ga];
 #pragma unroll
-      for (int ct = 0; ct < CT; ++ct) {
-        st[t][ct] *= gamma;
+      for (int t = 0; t < 2 * KS; ++t) {
+        st[t] *= gamma;
+        f32x4 x = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int ks = 0; ks < 2; ++ks) st[t][ct] = mfma16(kf[ks], vw[ks][ct], st[t][ct]);
-      }
-      if constexpr (GATED) {
-        if (t % NW == w) {  // every column of the product is the sum of the weighted keys
-          f32x4 x = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-          for (int ks = 0; ks < 2; ++ks) x = mfma16(kf[ks], wf[ks], x);
-          if (col == 0) {
-            f32x4* np = reinterpret_cast<f32x4*>(fl + L::n + 16 * t + 4 * g);
-            *np = *np * gamma + x;
+        for (int ks = 0; ks < 2; ++ks) {
+          const bf16_t* k = mb + L::k + tr_k + 32 * ks * L::KROW + 16 * t;
+          const bf16x8 kf = mem_join(mem_read_tr16(k), mem_read_tr16(k + 16 * L::KROW));
+          st[t] = mfma16(kf, vw[ks], st[t]);
+          // the normaliser, by the last wave: every column of the product is the sum of the
+          // weighted keys
+          if constexpr (GATED) {
+            if (w == nwave) x = mfma16(kf, wf[ks], x);
+          }
+        }
+        if constexpr (GATED) {
+          if (w == nwave && col == 0) {
+            const int d = 16 * t + 4 * g;
+            *reinterpret_cast<f32x4*>(nn + d) = *reinterpret_cast<const f32x4*>(nc + d) * gamma + x;
           }
         }
       }
     }
+    __syncthreads();
+
+    if (own) {
 #pragma unroll
-    for (int ct = 0; ct < CT; ++ct)
+      for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
-      for (int tt = 0; tt < 4; ++tt) o[ct][tt] *= inv[tt];
-    float r[4];
+        for (int tt = 2 * ks; tt < 4; ++tt)
+          o[tt] = mfma16(vf[ks], load_bf16x8(mb + L::p + (16 * tt + col) * L::PROW + 32 * ks + 8 * g), o[tt]);
+      if constexpr (GATED) {
+#pragma unroll
+        for (int tt = 0; tt < 4; ++tt) {
+          const int t = 16 * tt + col;
+          float d = cur[L::in + t] * fl[L::qn + t];
+#pragma unroll
+          for (int i = 0; i < L::NG; ++i) d += fl[L::rs + i * kMC + t];
+          o[tt] *= __builtin_amdgcn_rcpf(fmaxf(fabsf(d), cur[L::em + t]) + 1e-6f);
+        }
+      }
+    }
     if (a.slices == 1) {
 #pragma unroll
       for (int tt = 0; tt < 4; ++tt) {
         float ss = 0.f;
+        if (own) {
 #pragma unroll
-        for (int ct = 0; ct < CT; ++ct)
-#pragma unroll
-          for (int j = 0; j < 4; ++j) ss += o[ct][tt][j] * o[ct][tt][j];
+          for (int j = 0; j < 4; ++j) ss += o[tt][j] * o[tt][j];
+        }
         ss += __shfl_xor(ss, 16, 64);
         ss += __shfl_xor(ss, 32, 64);
-        if (g == 0) fl[L::ss + w * kMC + 16 * tt + col] = ss;
+        if (g == 0) fl[L::ss + (16 * tt + col) * NW + w] = ss;
       }
     }
     __syncthreads();
-#pragma unroll
-    for (int tt = 0; tt < 4; ++tt) {
-      float ss = 0.f;
-      if (a.slices == 1) {
-#pragma unroll
-        for (int i = 0; i < NW; ++i) ss += fl[L::ss + i * kMC + 16 * tt + col];
-      }
-      r[tt] = 1.f / sqrtf(ss / (float)a.vdim + a.eps);
-    }
+    // stores without branches (rows behind the portion and columns behind the head are beyond the
+    // buffer's end), so that the next wait for loads does not wait for them
+    const __amdgpu_buffer_rsrc_t ob = __builtin_amdgcn_make_buffer_rsrc(
+        (void*)(out + (int64_t)t0 * a.ldo), (short)0, 2 * nt * a.ldo, 0x00020000);
 #pragma unroll
     for (int tt = 0; tt < 4; ++tt) {
       const int t = 16 * tt + col;
-      if (t >= nt) continue;
-      bf16_t* op = out + (int64_t)(row0 + t0 + t) * a.ldo;
+      if (a.slices == 1) {
+        float ss = 0.f;
 #pragma unroll
-      for (int ct = 0; ct < CT; ++ct) {
-        const int x = cw + 16 * ct + 4 * g;
-        if (x >= a.vdim) continue;
-        bf16x4 y;
+        for (int i = 0; i < NW; i += 4) {
+          const f32x4 x = *reinterpret_cast<const f32x4*>(fl + L::ss + t * NW + i);
+          ss += (x[0] + x[1]) + (x[2] + x[3]);
+        }
+        o[tt] *= __builtin_amdgcn_rsqf(ss * inv_dv + a.eps);
+        if (a.norm_w) o[tt] *= nw;
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-          y[j] = f2bf(a.slices > 1 ? o[ct][tt][j]
-                                   : o[ct][tt][j] * r[tt] * nw[ct][j] *
-                                         mem_gate<bf16_t>(bf2f(gate[ct][tt][j]), a.silu));
-        *reinterpret_cast<bf16x4*>(op + x) = y;
+        for (int j = 0; j < 4; ++j) o[tt][j] *= mem_gate<bf16_t>(bf2f(gate[tt][j]), a.silu);
       }
+      bf16x4 y;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) y[j] = f2bf(o[tt][j]);
+      __builtin_amdgcn_raw_buffer_store_b64(
+          __builtin_bit_cast(u32x2, y), ob,
+          cw + 4 * g < cols ? 2u * (unsigned)(t * a.ldo + cw + 4 * g) : 0xFFFFFFF0u, 0, 0);
     }
+    cur = nxt;
   }
+  int gl = g;  // addresses of the state are computed again rather than kept through the loop
+  asm volatile("" : "+v"(gl));
 #pragma unroll
   for (int t = 0; t < 2 * KS; ++t)
 #pragma unroll
-    for (int ct = 0; ct < CT; ++ct)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = 16 * t + 4 * g + r, x = cw + 16 * ct + col;
-        if (d < a.dim && x < a.vdim) S[(int64_t)d * a.vdim + x] = st[t][ct][r];
-      }
+    for (int r = 0; r < 4; ++r) {
+      const int d = 16 * t + 4 * gl + r, x = cw + col;
+      if (d < a.dim && x < cols) S[d * a.vdim + x] = st[t][r];
+    }
   if constexpr (GATED) {
-    for (int d = tid; d < a.dim; d += NTHR) N[d] = fl[L::n + d];
+    const float* nc = fl + L::n + (cur == fl ? 0 : L::DP);
+    for (int d = tid; d < a.dim; d += NTHR) N[d] = nc[d];
     if (tid == 0) top[0] = m0 * (1.f / kLog2e);
   }
 }
@@ -824,26 +841,26 @@ static int mem_scan_t(const MemoryArgs& a, hipStream_t st) {
   return mem_scan_go<T, 32>(a, st);
 }
 
-template <int KS, int NW, int CT>
+template <int KS, int NW>
 static int mem_chunk_go(const MemoryArgs& a, hipStream_t st) {
-  using L = MemLds<KS, NW, CT>;
+  using L = MemLds<KS, NW>;
   const dim3 grid(a.nseg, a.H, a.slices), blk(64 * NW);
-  if (a.log_decay) memory_chunk_kernel<KS, NW, CT, false><<<grid, blk, L::BYTES, st>>>(a);
-  else memory_chunk_kernel<KS, NW, CT, true><<<grid, blk, L::BYTES, st>>>(a);
+  if (!a.log_decay) memory_chunk_kernel<KS, NW, true, false><<<grid, blk, L::BYTES, st>>>(a);
+  else if (a.rot_dims) memory_chunk_kernel<KS, NW, false, true><<<grid, blk, L::BYTES, st>>>(a);
+  else memory_chunk_kernel<KS, NW, false, false><<<grid, blk, L::BYTES, st>>>(a);
   return 0;
 }
 template <int KS>
-static int mem_chunk_c(const MemoryArgs& a, hipStream_t st) {
-  constexpr bool wide = KS == 8;  // 8 waves of one column tile: as many accumulators to a wave
-  if (a.slices == 1 && a.vdim > 128) return mem_chunk_go<KS, 8, 2>(a, st);
-  if (a.slices == 1 && a.vdim <= 64) return mem_chunk_go<KS, 4, 1>(a, st);
-  return mem_chunk_go<KS, wide ? 8 : 4, wide ? 1 : 2>(a, st);
+static int mem_chunk_w(const MemoryArgs& a, hipStream_t st) {
+  if (a.slices == 1 && a.vdim <= 64) return mem_chunk_go<KS, 4>(a, st);
+  return mem_chunk_go<KS, 8>(a, st);
 }
 
 static int mem_check(const MemoryArgs& a) {
   if (a.H < 1 || a.dim < 1 || a.dim > 256 || a.vdim < 1 || a.vdim > 1024) return -1;
-  if (a.slices != (a.vdim <= 256 ? 1 : (a.vdim + 127) / 128)) return -1;
+  if (a.slices != (a.vdim + 127) / 128) return -1;
   if (a.rot_dims < 0 || a.rot_dims % 2 || a.rot_dims > a.dim || (a.rot_dims && !a.cos_sin)) return -1;
+  if (!a.log_decay && a.rot_dims) return -1;
   if (!a.log_decay && (!a.i_bias || !a.f_bias || !a.nrm || !a.top || !(a.cap > 0.f))) return -1;
   return 0;
 }
@@ -854,13 +871,13 @@ int launch_memory_scan(int f32, const MemoryArgs& a, int plain, hipStream_t st) 
   if (mem_check(a)) return -1;
   const bool chunk = !f32 && !plain && a.dim % 16 == 0 && a.rot_dims % 16 == 0 && a.vdim % 8 == 0 &&
                      a.ldp % 8 == 0 && a.off_k % 8 == 0 && a.off_v % 8 == 0 && a.off_g % 4 == 0 &&
-                     a.ldo % 4 == 0;
+                     a.ldo % 4 == 0 && a.ldp < (1 << 23) && a.ldo < (1 << 23);
   int rc;
   if (chunk) {
-    if (a.dim <= 32) rc = mem_chunk_c<1>(a, st);
-    else if (a.dim <= 64) rc = mem_chunk_c<2>(a, st);
-    else if (a.dim <= 128) rc = mem_chunk_c<4>(a, st);
-    else rc = mem_chunk_c<8>(a, st);
+    if (a.dim <= 32) rc = mem_chunk_w<1>(a, st);
+    else if (a.dim <= 64) rc = mem_chunk_w<2>(a, st);
+    else if (a.dim <= 128) rc = mem_chunk_w<4>(a, st);
+    else rc = mem_chunk_w<8>(a, st);
   } else {
     rc = f32 ? mem_scan_t<float>(a, st) : mem_scan_t<bf16_t>(a, st);
   }
@@ -889,19 +906,20 @@ int launch_memory_decode(int f32, const MemoryArgs& a, hipStream_t st) {
 }
 
 // dynamic LDS above 64 KB
-template <int KS, int NW, int CT>
+template <int KS, int NW>
 static int mem_attr() {
-  const int n = (int)MemLds<KS, NW, CT>::BYTES;
-  static_assert(MemLds<KS, NW, CT>::BYTES <= 160 * 1024, "LDS of a CU");
-  return (int)hipFuncSetAttribute((const void*)memory_chunk_kernel<KS, NW, CT, true>,
-                                  hipFuncAttributeMaxDynamicSharedMemorySize, n) |
-         (int)hipFuncSetAttribute((const void*)memory_chunk_kernel<KS, NW, CT, false>,
-                                  hipFuncAttributeMaxDynamicSharedMemorySize, n);
+  const int n = (int)MemLds<KS, NW>::BYTES;
+  static_assert(MemLds<KS, NW>::BYTES <= 160 * 1024, "LDS of a CU");
+  int e = 0;
+  for (const void* f : {(const void*)memory_chunk_kernel<KS, NW, true, false>,
+                        (const void*)memory_chunk_kernel<KS, NW, false, true>,
+                        (const void*)memory_chunk_kernel<KS, NW, false, false>})
+    e |= (int)hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, n);
+  return e;
 }
 template <int KS>
 static int mem_attrs() {
-  return mem_attr<KS, 8, 2>() | mem_attr<KS, 4, 1>() |
-         mem_attr<KS, KS == 8 ? 8 : 4, KS == 8 ? 1 : 2>();
+  return mem_attr<KS, 4>() | mem_attr<KS, 8>();
 }
 int configure_memory() {
   return mem_attrs<1>() | mem_attrs<2>() | mem_attrs<4>() | mem_attrs<8>();

@@ -20,14 +20,13 @@ import torch.nn.functional as F
 from ._ext import check, hipk, on_gpu, ptr, stream_ptr
 from .delta import Portions
 
-MEMORY_COLUMNS = 256  # value columns one workgroup takes with the norm of the read-out
-SLICE_COLUMNS = 128   # of a wider head: columns of a workgroup, the norm behind it
+SLICE_COLUMNS = 128  # a workgroup's value columns
 
 
 def memory_slices(vdim: int) -> int:
     """Workgroups a head's columns are split over; each keeps its own copy of the normaliser and the
     running maximum."""
-    return 1 if vdim <= MEMORY_COLUMNS else -(-vdim // SLICE_COLUMNS)
+    return -(-vdim // SLICE_COLUMNS)
 
 
 @dataclass
