@@ -77,6 +77,11 @@ void bind_hybrid(py::module_& m) {
   m.def("stream_add", [](int f32, u64 out, u64 h, u64 y, int64_t ldy, int rows, int W, u64 st) {
     return drtc::launch_stream_add(f32, P<void>(out), P<float>(h), P<void>(y), ldy, rows, W, S(st));
   });
+  m.def("side_gate_gemm", [](u64 out, u64 x, u64 w, u64 embed, int64_t lde, int off, u64 ids, int T,
+                             int N, int K, u64 st) {
+    return drtc::launch_side_gate_gemm(P<void>(out), P<void>(x), P<void>(w), P<void>(embed), lde, off,
+                                       P<const int>(ids), T, N, K, S(st));
+  });
   m.def("side_gate", [](int f32, u64 out, u64 z, u64 embed, int64_t lde, int off, u64 ids, int rows,
                         int dim, u64 st) {
     return drtc::launch_side_gate(f32, P<void>(out), P<void>(z), P<void>(embed), lde, off,

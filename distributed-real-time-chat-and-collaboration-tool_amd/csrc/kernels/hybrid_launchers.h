@@ -361,6 +361,8 @@ struct SideNormArgs {
 int launch_side_norm(int f32, const SideNormArgs& a, hipStream_t st);
 int launch_stream_add(int f32, void* out, float* h, const void* y, int64_t ldy, int rows, int W,
                       hipStream_t st);
+int launch_side_gate_gemm(void* out, const void* x, const void* w, const void* embed, int64_t lde,
+                          int off, const int* ids, int T, int N, int K, hipStream_t st);
 int launch_side_gate(int f32, void* out, const void* z, const void* embed, int64_t lde, int off,
                      const int* ids, int rows, int dim, hipStream_t st);
 

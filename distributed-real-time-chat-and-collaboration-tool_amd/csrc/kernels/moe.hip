@@ -100,16 +100,24 @@ __global__ __launch_bounds__(kMoeRouteWG) void moe_route_kernel(
     for (int j = 0; j < KM; ++j) { v[j] = -INFINITY; id[j] = 0x7fffffff; }
     for (int g = 0; g < groups; ++g) {
       if (!(open >> g & 1)) continue;
-      for (int e = g * per; e < (g + 1) * per; ++e) {
-        float x = logit_f32(lr[(int64_t)e * les]);
-        int xi = e;
+      for (int e0 = g * per; e0 < (g + 1) * per; e0 += 8) {
+        const int ne = min(8, (g + 1) * per - e0);
+        float xs[8];  // loads in flight together
 #pragma unroll
-        for (int j = 0; j < KM; ++j) {
-          // order (value desc, id asc): a displaced entry carried down the list
-          // must not overtake an equal-valued entry with a higher id
-          if (x > v[j] || (x == v[j] && xi < id[j])) {
-            const float tv = v[j]; const int ti = id[j];
-            v[j] = x; id[j] = xi; x = tv; xi = ti;
+        for (int i = 0; i < 8; ++i) xs[i] = i < ne ? logit_f32(lr[(int64_t)(e0 + i) * les]) : 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          if (i >= ne) break;
+          float x = xs[i];
+          int xi = e0 + i;
+#pragma unroll
+          for (int j = 0; j < KM; ++j) {
+            // order (value desc, id asc): a displaced entry carried down the list
+            // must not overtake an equal-valued entry with a higher id
+            if (x > v[j] || (x == v[j] && xi < id[j])) {
+              const float tv = v[j]; const int ti = id[j];
+              v[j] = x; id[j] = xi; x = tv; xi = ti;
+            }
           }
         }
       }
@@ -186,14 +194,56 @@ __global__ __launch_bounds__(64 * kRouterWaves) void moe_router_kernel(float* __
   }
 }
 
+// The same sums in the same order for decode-sized batches: 16 tokens to a workgroup, twice the steps
+// in flight, one barrier.
+template <int ET>
+__global__ __launch_bounds__(64 * kRouterWaves) void moe_router_few_kernel(
+    float* __restrict__ out, const bf16_t* __restrict__ x, int ldx, const bf16_t* __restrict__ w, int T,
+    int E, int K) {
+  __shared__ float part[kRouterWaves][16 * ET][17];
+  const int t0 = blockIdx.x * 16, lane = threadIdx.x & 63, wv = wave_id_uniform();
+  const int col = lane & 15, g = lane >> 4, t = min(t0 + col, T - 1);
+  f32x4 acc[ET];
+#pragma unroll
+  for (int i = 0; i < ET; ++i) acc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  bf16x8 zero;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) zero[j] = f2bf(0.f);
+#pragma unroll 8
+  for (int c0 = 32 * wv; c0 < K; c0 += 32 * kRouterWaves) {
+    const int c = min(c0 + 8 * g, K - 8);
+    const bool in = c0 + 8 * g < K;
+    const bf16x8 bx = load_bf16x8(x + (int64_t)t * ldx + c);
+    const bf16x8 b = in ? bx : zero;
+#pragma unroll
+    for (int i = 0; i < ET; ++i)
+      acc[i] = mfma16(load_bf16x8(w + (int64_t)min(16 * i + col, E - 1) * K + c), b, acc[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < ET; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) part[wv][16 * i + 4 * g + r][col] = acc[i][r];
+  __syncthreads();
+  for (int i = threadIdx.x; i < E * 16; i += 64 * kRouterWaves) {
+    const int e = i >> 4, c = i & 15;
+    float s = part[0][e][c];
+#pragma unroll
+    for (int o = 1; o < kRouterWaves; ++o) s += part[o][e][c];
+    if (t0 + c < T) out[(int64_t)e * T + t0 + c] = s;
+  }
+}
+
 int launch_moe_router(float* out, const void* x, int ldx, const void* w, int T, int E, int K,
                       hipStream_t st) {
   if (T == 0) return 0;
   if (E < 1 || E > 256 || K % 8 || ldx % 8 || ldx < K) return -1;
-  const dim3 grid((T + 31) / 32);
+  const dim3 grid((T + 31) / 32), few((T + 15) / 16);
   const bf16_t *xx = (const bf16_t*)x, *ww = (const bf16_t*)w;
 #define DRTC_ROUTER(N) moe_router_kernel<N><<<grid, dim3(64 * kRouterWaves), 0, st>>>(out, xx, ldx, ww, T, E, K)
-  if (E <= 16) DRTC_ROUTER(1);
+  if (T <= 1024 && E <= 32) {
+    if (E <= 16) moe_router_few_kernel<1><<<few, dim3(64 * kRouterWaves), 0, st>>>(out, xx, ldx, ww, T, E, K);
+    else moe_router_few_kernel<2><<<few, dim3(64 * kRouterWaves), 0, st>>>(out, xx, ldx, ww, T, E, K);
+  } else if (E <= 16) DRTC_ROUTER(1);
   else if (E <= 32) DRTC_ROUTER(2);
   else if (E <= 64) DRTC_ROUTER(4);
   else if (E <= 128) DRTC_ROUTER(8);

@@ -4,7 +4,8 @@
 //               h  = embed_scale * embed[ids]         (instead, at the first layer)
 //               out = (h - mean(h)) / sqrt(var(h) + eps) * w
 //   stream_add  h += y; the stream in the activation type
-//   side_gate   out = gelu_tanh(z) * embed[ids, part of a layer]
+//   side_gate   out = gelu_tanh(z) * embed[ids, part of a layer]; and, for decode-sized batches, the
+//               same with z = x . w^T formed in the kernel
 //
 // side_norm: one workgroup per row, 8 elements to a lane and step, held in registers from the add
 // to the scaling, so that the variance is the mean of squared deviations.
@@ -231,6 +232,64 @@ int launch_side_gate(int f32, void* out, const void* z, const void* embed, int64
   if (off < 0 || off + dim > lde) return -1;
   if (f32) side_gate_t<float>(out, z, embed, lde, off, ids, n, dim, st);
   else side_gate_t<bf16_t>(out, z, embed, lde, off, ids, n, dim, st);
+  return (int)hipGetLastError();
+}
+
+// z = x . w^T, gated: 16 tokens x 16 CT columns to a workgroup, whose 8 waves take every eighth
+// 32-column step of the reduction; operands straight from global memory.
+constexpr int kSideWaves = 8;
+template <int CT>
+__global__ __launch_bounds__(64 * kSideWaves) void side_gate_gemm_kernel(
+    bf16_t* __restrict__ out, const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
+    const bf16_t* __restrict__ embed, int64_t lde, int off, const int* __restrict__ ids, int T, int N,
+    int K) {
+  __shared__ float part[kSideWaves][16][16 * CT + 1];
+  const int t0 = blockIdx.x * 16, n0 = blockIdx.y * 16 * CT, lane = threadIdx.x & 63;
+  const int wv = wave_id_uniform(), col = lane & 15, g = lane >> 4;
+  const bf16_t* xr = x + (int64_t)min(t0 + col, T - 1) * K;
+  f32x4 acc[CT];
+#pragma unroll
+  for (int i = 0; i < CT; ++i) acc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  bf16x8 zero;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) zero[j] = f2bf(0.f);
+#pragma unroll 8
+  for (int c0 = 32 * wv; c0 < K; c0 += 32 * kSideWaves) {
+    const int c = min(c0 + 8 * g, K - 8);
+    const bf16x8 bx = load_bf16x8(xr + c);
+    const bf16x8 b = c0 + 8 * g < K ? bx : zero;
+#pragma unroll
+    for (int i = 0; i < CT; ++i)
+      acc[i] = mfma16(load_bf16x8(w + (int64_t)min(n0 + 16 * i + col, N - 1) * K + c), b, acc[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < CT; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) part[wv][col][16 * i + 4 * g + r] = acc[i][r];
+  __syncthreads();
+  for (int i = threadIdx.x; i < 256 * CT; i += 64 * kSideWaves) {
+    const int t = i / (16 * CT), n = i % (16 * CT);
+    if (t0 + t >= T || n0 + n >= N) continue;
+    float z = part[0][t][n];
+#pragma unroll
+    for (int o = 1; o < kSideWaves; ++o) z += part[o][t][n];
+    out[(int64_t)(t0 + t) * N + n0 + n] =
+        f2bf(act_value<1>(z) * bf2f(embed[(int64_t)ids[t0 + t] * lde + off + n0 + n]));
+  }
+}
+
+int launch_side_gate_gemm(void* out, const void* x, const void* w, const void* embed, int64_t lde,
+                          int off, const int* ids, int T, int N, int K, hipStream_t st) {
+  if (T == 0 || N == 0) return 0;
+  if (K < 8 || K % 8 || off < 0 || off + N > lde) return -1;
+  const bf16_t *xx = (const bf16_t*)x, *ww = (const bf16_t*)w, *ee = (const bf16_t*)embed;
+  const dim3 blk(64 * kSideWaves);
+  if (T <= 128)
+    side_gate_gemm_kernel<1><<<dim3((T + 15) / 16, (N + 15) / 16), blk, 0, st>>>(
+        (bf16_t*)out, xx, ww, ee, lde, off, ids, T, N, K);
+  else
+    side_gate_gemm_kernel<2><<<dim3((T + 15) / 16, (N + 31) / 32), blk, 0, st>>>(
+        (bf16_t*)out, xx, ww, ee, lde, off, ids, T, N, K);
   return (int)hipGetLastError();
 }
 

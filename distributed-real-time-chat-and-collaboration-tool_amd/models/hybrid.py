@@ -465,7 +465,7 @@ class HybridLM:
                 x = ops.stream_add(h, y)
             z = zn = None
             if cfg.side_dim:
-                g = ops.side_gate(ops.linear(x, L["side_gate"]), self.side_embed, ids, i)
+                g = ops.side_input(x, L["side_gate"], self.side_embed, ids, i)
                 z, zn = ops.linear(g, L["side_proj"]), L["side_norm"]
         return ops.linear(ops.side_norm(h, self.final.w, eps, z, zn, dtype=dt), self.lm_head)
 

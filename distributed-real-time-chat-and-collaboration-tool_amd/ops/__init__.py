@@ -30,7 +30,7 @@ from .moe import fused_moe, fused_moe_ref, router_logits, router_logits_f32
 from .norm import PendingNorm, dyt, dyt_ref, group_rms, rmsnorm, rmsnorm_ref
 from .norm_conv import (MAX_TAPS, ConvTiles, LayerNorm, conv_tile_rows, norm_conv, sinusoid_turns,
                         softcap_)
-from .norm_side import side_gate, side_norm, stream_add
+from .norm_side import side_gate, side_input, side_norm, stream_add
 from .rope import build_rope_cache, kv_write_v, kv_write_v_ref, rope_kv_, rope_kv_ref
 from .sampling import sample, sample_ref
 from .talking import (MIX_TILE, STATS_TILE, TalkDecodeWorkspace, TalkPortions, TalkWeights,
@@ -55,6 +55,6 @@ __all__ = [
     "talk_cache_shapes", "talk_decode", "talk_prefill", "GroupedDecodeWorkspace",
     "GroupedPortions", "GroupedWeights", "attn_prep", "grouped_decode", "grouped_prefill",
     "grouped_qtile", "prep_tile_rows", "group_rms", "router_logits_f32",
-    "MemoryWeights", "memory_decode", "memory_scan", "memory_slices", "side_gate", "side_norm",
+    "MemoryWeights", "memory_decode", "memory_scan", "memory_slices", "side_gate", "side_input", "side_norm",
     "stream_add",
 ]

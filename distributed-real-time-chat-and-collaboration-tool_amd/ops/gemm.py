@@ -216,6 +216,9 @@ def _resolve(M: int, N: int, K: int, ldx: int) -> tuple[str, int]:
                 return ("lt", ent[0])
     if M > DECODE_MAX_M:
         if w4_shape_ok(M, N, K):
+            # 256 x 256 tiles for a quarter of the CUs at most: smaller ones
+            if -(-M // 256) * (N // 256) <= 64 and _xd_enabled and xd_supported(M, N, K, 141):
+                return ("xd", 141)
             return ("w4", 0)
         a = _prefill_algo(M, N, K, ldx, 0)
         return ("lt", a) if a >= 0 else ("torch", 0)

@@ -61,6 +61,30 @@ def stream_add(h: torch.Tensor, y: torch.Tensor) -> torch.Tensor:
     return out
 
 
+SIDE_GEMM_ROWS = 512  # larger steps form z in a GEMM of its own
+
+
+def side_input(x: torch.Tensor, w: torch.Tensor, embed: torch.Tensor, ids: torch.Tensor,
+               layer: int) -> torch.Tensor:
+    """gelu_tanh(x @ w.T) times the tokens' own inputs to ``layer``: w [dim, W], embed [vocab,
+    layers * dim]; one kernel for decode-sized batches in bf16."""
+    from .gemm import linear
+
+    rows, K = x.shape
+    dim = w.shape[0]
+    if not (on_gpu(x) and x.dtype == torch.bfloat16 and rows <= SIDE_GEMM_ROWS and K % 8 == 0):
+        return side_gate(linear(x, w), embed, ids, layer)
+    assert x.is_contiguous() and w.is_contiguous() and embed.is_contiguous()
+    assert x.dtype == w.dtype == embed.dtype and w.shape[1] == K
+    assert ids.dtype == torch.int32 and ids.numel() == rows and ids.is_contiguous()
+    assert (layer + 1) * dim <= embed.shape[1]
+    out = x.new_empty(rows, dim)
+    check(hipk().side_gate_gemm(out.data_ptr(), x.data_ptr(), w.data_ptr(), embed.data_ptr(),
+                                embed.shape[1], layer * dim, ids.data_ptr(), rows, dim, K,
+                                stream_ptr(x)), "side_gate_gemm")
+    return out
+
+
 def side_gate(z: torch.Tensor, embed: torch.Tensor, ids: torch.Tensor, layer: int) -> torch.Tensor:
     """gelu_tanh(z) times the tokens' own inputs to ``layer``: embed [vocab, layers * dim],
     z [rows, dim]."""

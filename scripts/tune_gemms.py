@@ -23,7 +23,7 @@ import torch  # noqa: E402
 
 from drtc_amd.engine.decode_runner import DEFAULT_BUCKETS  # noqa: E402
 from drtc_amd.models import HybridConfig, get_config  # noqa: E402
-from drtc_amd.models.config import GatedAverage, GroupedAttention  # noqa: E402
+from drtc_amd.models.config import GatedAverage, GroupedAttention, LatentAttention, MatrixMemory  # noqa: E402
 from drtc_amd.models.mixers import pad_to  # noqa: E402
 from drtc_amd.models.transformer import ShardInfo  # noqa: E402
 
@@ -59,11 +59,32 @@ def grouped_shapes(cfg: HybridConfig) -> dict[str, tuple[int, int]]:
     return shapes
 
 
+def joint_shapes(cfg: HybridConfig) -> dict[str, tuple[int, int]]:
+    """Fused input projections, joint output projections, shared experts' and token inputs'
+    projections of joint layers."""
+    W, shapes = cfg.hidden_size, {"side_proj": (cfg.hidden_size, cfg.side_dim)}
+    for l in cfg.layers:
+        m, ffp = l.mixer, pad_to((l.shared if l.experts else l.ff) or 0)
+        if isinstance(m, LatentAttention):
+            own = m.kv_from is None
+            kind, rows = "latent" if own else "latent_shared", pad_to(m.heads * (m.dim + m.rot_dim))
+            rows += (pad_to(m.kv_rank + m.rot_dim) if own else 0) + (pad_to(m.heads) if m.gate else 0)
+        else:
+            rows = 2 * pad_to(m.heads * m.dim) + 2 * pad_to(m.heads * m.vdim)
+            kind = "memory" if isinstance(m, MatrixMemory) else "retention"
+            rows += 2 * pad_to(m.heads) if kind == "memory" else 0
+        shapes[f"in_{kind}"] = (pad_to(rows, 256) if rows >= 2048 else rows, W)
+        shapes["out"] = (W, pad_to(m.heads * m.vdim) + ffp)
+        if ffp:
+            shapes["up"] = (ffp, W)
+    return shapes
+
+
 def projection_shapes(name: str, tp: int) -> dict[str, tuple[int, int]]:
     """(N, K) of each decode projection of one TP shard."""
     cfg = get_config(name)
     if isinstance(cfg, HybridConfig):
-        return parallel_shapes(cfg) if cfg.block == "parallel" else grouped_shapes(cfg)
+        return {"parallel": parallel_shapes, "joint": joint_shapes}.get(cfg.block, grouped_shapes)(cfg)
     sh = ShardInfo(cfg, SimpleNamespace(tp_size=tp, tp_rank=0, ep_size=1, ep_rank=0))
     H, D = cfg.hidden_size, cfg.head_dim
     shapes = {"qkv": ((sh.hq + 2 * sh.hkv) * D, H), "o": (H, sh.hq * D),

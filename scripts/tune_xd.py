@@ -70,7 +70,8 @@ def main() -> None:
     ap.add_argument("--ms", default=",".join(map(str, BUCKETS)))
     ap.add_argument("--min-gain", type=float, default=0.03)
     ap.add_argument("--out", default="gpurun_out/xd_tuned.json")
-    ap.add_argument("--gemms", default="qkv,o,gate_up,down,in_grouped,in_talk,in_average,up,out_talk,out_average",
+    ap.add_argument("--gemms", default="qkv,o,gate_up,down,in_grouped,in_talk,in_average,up,out_talk,out_average,"
+                    "out,in_memory,in_retention,in_latent,in_latent_shared",
                     help="projections to tune (lm_head too: profiles/r5ak)")
     ap.add_argument("--nt-any", action="store_true",
                     help="non-temporal forms among the candidates at every M, not only where "

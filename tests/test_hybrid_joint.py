@@ -71,7 +71,8 @@ def test_layer_norm_behind_side_input(target, W):
 
 
 @on
-@pytest.mark.parametrize("rows,W,dim", [(5, 256, 16), (1, 64, 7), (33, 100, 24), (300, 512, 128), (2, 99, 1)])
+@pytest.mark.parametrize("rows,W,dim", [(5, 256, 16), (1, 64, 7), (33, 100, 24), (300, 512, 128), (2, 99, 1), (17, 296, 40),
+                                        (200, 128, 72), (600, 256, 32), (1, 2048, 128)])
 def test_stream_add_and_side_gate(target, rows, W, dim):
     dev, dt = target
     h, h64 = rnd(rows, W, seed=1, dev=dev)
@@ -85,6 +86,9 @@ def test_stream_add_and_side_gate(target, rows, W, dim):
     for layer in range(3):
         want = O.gelu_tanh(z64) * e64[ids.long().cpu(), layer * dim:(layer + 1) * dim]
         close(ops.side_gate(z, e, ids, layer), want, tol(dt, 2e-6, 5e-3))
+        w, w64 = rnd(dim, W, seed=5 + layer, dtype=dt, dev=dev, std=W ** -0.5)
+        want = O.gelu_tanh(y64 @ w64.T) * e64[ids.long().cpu(), layer * dim:(layer + 1) * dim]
+        close(ops.side_input(y, w, e, ids, layer), want, tol(dt, 2e-6, 1e-2))
 
 
 # ------------------------------------------------------------------ retention and matrix memory
