@@ -620,6 +620,7 @@ int xd_launch(const XdParams& p, int epi, hipStream_t st) {
     case XD_CLAMP:  // built for the tiles of the grouped mode
       if constexpr (C::NF == 4 || C::NF == 8) return xd_launch_e<C, XD_CLAMP>(p, st);
       else return -1;
+    case XD_RELU2: return xd_launch_e<C, XD_RELU2>(p, st);
     default: return xd_launch_e<C, XD_GELU>(p, st);
   }
 }
@@ -644,7 +645,8 @@ int xd_cfg() {
   for (const void* f : {(const void*)gemm_xd_kernel<C, XD_STORE>,
                         (const void*)gemm_xd_kernel<C, XD_RESIDUAL>,
                         (const void*)gemm_xd_kernel<C, XD_SILU>,
-                        (const void*)gemm_xd_kernel<C, XD_GELU>})
+                        (const void*)gemm_xd_kernel<C, XD_GELU>,
+                        (const void*)gemm_xd_kernel<C, XD_RELU2>})
     e |= (int)hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, C::ALLOC);
   if constexpr (C::NF == 4 || C::NF == 8)
     e |= (int)hipFuncSetAttribute((const void*)gemm_xd_kernel<C, XD_CLAMP>,
@@ -743,8 +745,8 @@ int launch_gemm_xd(void* c, const void* a, const void* b, const void* r, int M, 
                    float limit, hipStream_t st) {
   const bool nt = (mt & 16) != 0;  // mt bit 4: non-temporal weight loads
   mt &= 15;
-  if (epi < XD_STORE || epi > XD_CLAMP) return -1;
-  const bool glu = epi >= XD_SILU;
+  if (epi < XD_STORE || epi > XD_RELU2) return -1;
+  const bool glu = epi >= XD_SILU && epi <= XD_CLAMP;
   const int stages = xd_stages(mt, nf);
   if (stages == 0 || splitk < 1 || splitk > 8 || (glu && nf % 2)) return -1;
   if (lda % 8 || ldb % 8 || ldc % 8) return -1;

@@ -156,22 +156,31 @@ __global__ __launch_bounds__(64 * kRouterWaves) void moe_router_kernel(float* __
   bf16x8 zero;
 #pragma unroll
   for (int j = 0; j < 8; ++j) zero[j] = f2bf(0.f);
-#pragma unroll 4
-  for (int c0 = 32 * wv; c0 < K; c0 += 32 * kRouterWaves) {
-    const int c = c0 + 8 * g;
-    const bool in = c < K;
-    bf16x8 b[2];
+  // U steps' loads ahead of their products; steps behind the end add zeros
+  constexpr int U = ET <= 2 ? 4 : ET <= 4 ? 2 : 1;
+  const bf16_t* xr[2];
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      const int t = t0 + 16 * j + col;
-      b[j] = in && t < T ? load_bf16x8(x + (int64_t)t * ldx + c) : zero;
+  for (int j = 0; j < 2; ++j) xr[j] = x + (int64_t)min(t0 + 16 * j + col, T - 1) * ldx;
+  for (int c0 = 32 * wv; c0 < K; c0 += 32 * kRouterWaves * U) {
+    bf16x8 b[U][2], a[U][ET];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int c = min(c0 + 32 * kRouterWaves * u + 8 * g, K - 8);
+#pragma unroll
+      for (int j = 0; j < 2; ++j) b[u][j] = load_bf16x8(xr[j] + c);
+#pragma unroll
+      for (int i = 0; i < ET; ++i)
+        a[u][i] = load_bf16x8(w + (int64_t)min(16 * i + col, E - 1) * K + c);
     }
 #pragma unroll
-    for (int i = 0; i < ET; ++i) {
-      const int e = 16 * i + col;
-      const bf16x8 a = in && e < E ? load_bf16x8(w + (int64_t)e * K + c) : zero;
+    for (int u = 0; u < U; ++u) {
+      const bool in = c0 + 32 * kRouterWaves * u + 8 * g < K;
 #pragma unroll
-      for (int j = 0; j < 2; ++j) acc[i][j] = mfma16(a, b[j], acc[i][j]);
+      for (int j = 0; j < 2; ++j) b[u][j] = in ? b[u][j] : zero;
+#pragma unroll
+      for (int i = 0; i < ET; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i][j] = mfma16(a[u][i], b[u][j], acc[i][j]);
     }
   }
   for (int o = 0; o < kRouterWaves; ++o) {
@@ -209,15 +218,23 @@ __global__ __launch_bounds__(64 * kRouterWaves) void moe_router_few_kernel(
   bf16x8 zero;
 #pragma unroll
   for (int j = 0; j < 8; ++j) zero[j] = f2bf(0.f);
-#pragma unroll 8
-  for (int c0 = 32 * wv; c0 < K; c0 += 32 * kRouterWaves) {
-    const int c = min(c0 + 8 * g, K - 8);
-    const bool in = c0 + 8 * g < K;
-    const bf16x8 bx = load_bf16x8(x + (int64_t)t * ldx + c);
-    const bf16x8 b = in ? bx : zero;
+  constexpr int U = 8;
+  for (int c0 = 32 * wv; c0 < K; c0 += 32 * kRouterWaves * U) {
+    bf16x8 b[U], a[U][ET];
 #pragma unroll
-    for (int i = 0; i < ET; ++i)
-      acc[i] = mfma16(load_bf16x8(w + (int64_t)min(16 * i + col, E - 1) * K + c), b, acc[i]);
+    for (int u = 0; u < U; ++u) {
+      const int c = min(c0 + 32 * kRouterWaves * u + 8 * g, K - 8);
+      b[u] = load_bf16x8(x + (int64_t)t * ldx + c);
+#pragma unroll
+      for (int i = 0; i < ET; ++i)
+        a[u][i] = load_bf16x8(w + (int64_t)min(16 * i + col, E - 1) * K + c);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      b[u] = c0 + 32 * kRouterWaves * u + 8 * g < K ? b[u] : zero;
+#pragma unroll
+      for (int i = 0; i < ET; ++i) acc[i] = mfma16(a[u][i], b[u], acc[i]);
+    }
   }
 #pragma unroll
   for (int i = 0; i < ET; ++i)
@@ -236,7 +253,7 @@ __global__ __launch_bounds__(64 * kRouterWaves) void moe_router_few_kernel(
 int launch_moe_router(float* out, const void* x, int ldx, const void* w, int T, int E, int K,
                       hipStream_t st) {
   if (T == 0) return 0;
-  if (E < 1 || E > 256 || K % 8 || ldx % 8 || ldx < K) return -1;
+  if (E < 1 || E > 256 || K < 8 || K % 8 || ldx % 8 || ldx < K) return -1;
   const dim3 grid((T + 31) / 32), few((T + 15) / 16);
   const bf16_t *xx = (const bf16_t*)x, *ww = (const bf16_t*)w;
 #define DRTC_ROUTER(N) moe_router_kernel<N><<<grid, dim3(64 * kRouterWaves), 0, st>>>(out, xx, ldx, ww, T, E, K)

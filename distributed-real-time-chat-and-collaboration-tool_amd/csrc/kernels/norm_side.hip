@@ -253,14 +253,24 @@ __global__ __launch_bounds__(64 * kSideWaves) void side_gate_gemm_kernel(
   bf16x8 zero;
 #pragma unroll
   for (int j = 0; j < 8; ++j) zero[j] = f2bf(0.f);
-#pragma unroll 8
-  for (int c0 = 32 * wv; c0 < K; c0 += 32 * kSideWaves) {
-    const int c = min(c0 + 8 * g, K - 8);
-    const bf16x8 bx = load_bf16x8(xr + c);
-    const bf16x8 b = c0 + 8 * g < K ? bx : zero;
+  // U steps' loads ahead of their products; steps behind the end add zeros
+  constexpr int U = 8;
+  for (int c0 = 32 * wv; c0 < K; c0 += 32 * kSideWaves * U) {
+    bf16x8 b[U], a[U][CT];
 #pragma unroll
-    for (int i = 0; i < CT; ++i)
-      acc[i] = mfma16(load_bf16x8(w + (int64_t)min(n0 + 16 * i + col, N - 1) * K + c), b, acc[i]);
+    for (int u = 0; u < U; ++u) {
+      const int c = min(c0 + 32 * kSideWaves * u + 8 * g, K - 8);
+      b[u] = load_bf16x8(xr + c);
+#pragma unroll
+      for (int i = 0; i < CT; ++i)
+        a[u][i] = load_bf16x8(w + (int64_t)min(n0 + 16 * i + col, N - 1) * K + c);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      b[u] = c0 + 32 * kSideWaves * u + 8 * g < K ? b[u] : zero;
+#pragma unroll
+      for (int i = 0; i < CT; ++i) acc[i] = mfma16(a[u][i], b[u], acc[i]);
+    }
   }
 #pragma unroll
   for (int i = 0; i < CT; ++i)

@@ -833,7 +833,8 @@ def gated(x: torch.Tensor, w: torch.Tensor, act: str = "silu", limit: float = 0.
 
 def squared_relu(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     """out = relu(x @ w.T)^2, into rows of any stride (columns of a wider operand): in the
-    epilogue of gemm_w4 at prefill size, else a pass behind ``linear``."""
+    epilogue of gemm_w4 at prefill size and of gemm_xd where ``linear`` takes that, else a pass
+    behind ``linear``."""
     M, K = x.shape
     assert out.shape == (M, w.shape[0]) and out.stride(1) == 1
     if not on_gpu(x):
@@ -842,6 +843,10 @@ def squared_relu(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> torch.T
     if w4_ok(x, w) and out.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0:
         return mfma_gemm(x, w, "relu2", out=out, variant=_w4v(K),
                          group_m=w4_group_m(M, w.shape[0], K))
+    if _gpu_bf16(x, w) and _aligned(x, w) and out.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0:
+        kind, form = route(M, w.shape[0], K, x.stride(0))
+        if kind == "xd":
+            return xd_gemm(x, w, "relu2", out=out, form=form)
     y = linear(x, w)
     check(hipk().relu2(int(y.dtype == torch.float32), out.data_ptr(), out.stride(0), y.data_ptr(),
                        M, w.shape[0], stream_ptr(x)), "relu2")
@@ -849,7 +854,7 @@ def squared_relu(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> torch.T
 
 
 # ------------------------------------------------------------------ XCD-partitioned decode GEMM
-XD_EPI = {"store": 0, "residual": 1, "silu": 2, "gelu_tanh": 3, "clamped": 4}
+XD_EPI = {"store": 0, "residual": 1, "silu": 2, "gelu_tanh": 3, "clamped": 4, "relu2": 5}
 # tile shapes built in gemm_xd.hip, (mt, nf) -> LDS ring depth (128 mt x 32 nf tiles); a form
 # is mt * 100 + nf * 10 + splitk (K split over 1..8 slices), + 1000 for non-temporal weight
 # loads (the tiles of XD_NT_TILES)
@@ -916,7 +921,7 @@ def xd_gemm(x: torch.Tensor, w: torch.Tensor, epi: str = "store",
     its own weight column panels through its L2 for every row tile).  epi "store";
     "residual" (``out`` may be ``residual``); "silu" / "gelu_tanh": w is the fused [gate; up]
     weight [2I, K] and y[:, n] = act(x . gate_n) * (x . up_n); "clamped": bounded by ``limit``
-    (tiles of XD_CLAMP_NF).  ``form`` = mt * 100 + nf * 10 + splitk (+ 1000: non-temporal weight loads; 0: ``xd_default_form``)."""
+    (tiles of XD_CLAMP_NF); "relu2": relu(x @ w.T)^2.  ``form`` = mt * 100 + nf * 10 + splitk (+ 1000: non-temporal weight loads; 0: ``xd_default_form``)."""
     M, K = x.shape
     glu = epi in GATED
     N = w.shape[0] // 2 if glu else w.shape[0]

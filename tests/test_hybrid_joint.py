@@ -434,3 +434,16 @@ def test_experts_on_wide_tiles():
     for v in (None, 1, 2, 3, 4):
         got = ops.fused_moe(x, ops.router_logits_f32(x, r), up, dn, top, "relu2", variant=v)
         close(got[sure.to("cuda")], want, 2e-2)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("form", [121, 141, 142, 161, 241, 261, 281])
+def test_squared_relu_on_xcd_tiles(form):
+    """The epilogue of the XCD-partitioned GEMM, into columns of a wider operand."""
+    M, N, K = 200, 768, 768
+    x, x64 = rnd(M, K, seed=1, dtype=BF16, dev="cuda")
+    w, w64 = rnd(N, K, seed=2, dtype=BF16, dev="cuda", std=K ** -0.5)
+    a = torch.full((M, 8 + N + 8), 5.0, dtype=BF16, device="cuda")
+    ops.gemm.xd_gemm(x, w, "relu2", out=a[:, 8:8 + N], form=form)
+    close(a[:, 8:8 + N], torch.relu(x64 @ w64.T).square(), 1e-2)
+    assert (a[:, :8] == 5).all() and (a[:, 8 + N:] == 5).all()
