@@ -104,12 +104,11 @@ __global__ __launch_bounds__(kMoeRouteWG) void moe_route_kernel(
         const int ne = min(8, (g + 1) * per - e0);
         float xs[8];  // loads in flight together
 #pragma unroll
-        for (int i = 0; i < 8; ++i) xs[i] = i < ne ? logit_f32(lr[(int64_t)(e0 + i) * les]) : 0.f;
+        for (int i = 0; i < 8; ++i) xs[i] = logit_f32(lr[(int64_t)(e0 + min(i, ne - 1)) * les]);
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-          if (i >= ne) break;
-          float x = xs[i];
-          int xi = e0 + i;
+          float x = i < ne ? xs[i] : -INFINITY;  // behind the last: never in the list
+          int xi = i < ne ? e0 + i : 0x7fffffff;
 #pragma unroll
           for (int j = 0; j < KM; ++j) {
             // order (value desc, id asc): a displaced entry carried down the list
@@ -218,7 +217,7 @@ __global__ __launch_bounds__(64 * kRouterWaves) void moe_router_few_kernel(
   bf16x8 zero;
 #pragma unroll
   for (int j = 0; j < 8; ++j) zero[j] = f2bf(0.f);
-  constexpr int U = 8;
+  constexpr int U = 16;
   for (int c0 = 32 * wv; c0 < K; c0 += 32 * kRouterWaves * U) {
     bf16x8 b[U], a[U][ET];
 #pragma unroll

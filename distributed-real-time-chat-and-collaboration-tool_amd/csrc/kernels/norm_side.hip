@@ -253,8 +253,13 @@ __global__ __launch_bounds__(64 * kSideWaves) void side_gate_gemm_kernel(
   bf16x8 zero;
 #pragma unroll
   for (int j = 0; j < 8; ++j) zero[j] = f2bf(0.f);
+  // this thread's output and its token's input, on the way during the products
+  static_assert(CT <= 2, "an output to a thread");
+  const int ot = threadIdx.x / (16 * CT), on = threadIdx.x % (16 * CT);
+  const bool mine = threadIdx.x < 256 * CT && t0 + ot < T && n0 + on < N;
+  const bf16_t e = mine ? embed[(int64_t)ids[t0 + ot] * lde + off + n0 + on] : zero[0];
   // U steps' loads ahead of their products; steps behind the end add zeros
-  constexpr int U = 8;
+  constexpr int U = 16;
   for (int c0 = 32 * wv; c0 < K; c0 += 32 * kSideWaves * U) {
     bf16x8 b[U], a[U][CT];
 #pragma unroll
@@ -277,15 +282,11 @@ __global__ __launch_bounds__(64 * kSideWaves) void side_gate_gemm_kernel(
 #pragma unroll
     for (int r = 0; r < 4; ++r) part[wv][col][16 * i + 4 * g + r] = acc[i][r];
   __syncthreads();
-  for (int i = threadIdx.x; i < 256 * CT; i += 64 * kSideWaves) {
-    const int t = i / (16 * CT), n = i % (16 * CT);
-    if (t0 + t >= T || n0 + n >= N) continue;
-    float z = part[0][t][n];
+  if (!mine) return;
+  float z = part[0][ot][on];
 #pragma unroll
-    for (int o = 1; o < kSideWaves; ++o) z += part[o][t][n];
-    out[(int64_t)(t0 + t) * N + n0 + n] =
-        f2bf(act_value<1>(z) * bf2f(embed[(int64_t)ids[t0 + t] * lde + off + n0 + n]));
-  }
+  for (int o = 1; o < kSideWaves; ++o) z += part[o][ot][on];
+  out[(int64_t)(t0 + ot) * N + n0 + on] = f2bf(act_value<1>(z) * bf2f(e));
 }
 
 int launch_side_gate_gemm(void* out, const void* x, const void* w, const void* embed, int64_t lde,
